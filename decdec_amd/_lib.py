@@ -1,4 +1,5 @@
-"""ctypes binding of libdecdec_hip.so (the C ABI declared in include/decdec_hip.h).
+"""ctypes bindings of libdecdec_hip.so (the C ABI declared in include/decdec_hip.h) and of libdecdec_mixers.so
+(include/decdec_mixers.h).
 
 There is no CPU fallback: if the library is missing or cannot be loaded, every op raises.
 """
@@ -10,7 +11,10 @@ import os
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libdecdec_hip.so")
 
+MIXERS_LIB_PATH = os.path.join(_HERE, "libdecdec_mixers.so")
+
 _lib = None
+_mixers = None
 
 
 class ConfigInfo(ctypes.Structure):
@@ -99,6 +103,64 @@ def load():
         fn.restype = restype
     _lib = lib
     return lib
+
+
+class Recurrence(ctypes.Structure):
+    """Mirror of ``decdec_recurrence``."""
+    _fields_ = ([("proj", _vp)] + [(n, _u32) for n in (
+        "ld", "off_q", "off_k", "off_v", "off_g", "off_a", "off_b", "heads", "kv_heads", "dim", "vdim", "taps", "delta")]
+        + [(n, _vp) for n in ("decay", "conv_q", "conv_k", "conv_v", "A_log", "dt_bias", "ring", "state", "pos")])
+
+
+class Latent(ctypes.Structure):
+    """Mirror of ``decdec_latent``."""
+    _fields_ = ([("proj", _vp)] + [(n, _u32) for n in (
+        "ld", "off_q", "off_c", "heads", "dim", "rot", "vdim", "rank", "max_seq")] + [("eps", _f32), ("scale", _f32)]
+        + [(n, _vp) for n in ("norm", "uk", "uv", "sink", "cos_table", "sin_table", "cache", "pos")])
+
+
+_rec, _lat = ctypes.POINTER(Recurrence), ctypes.POINTER(Latent)
+MIXERS_SIGNATURES = {
+    "decdec_mix_gemv": [_vp, _vp, _vp, _vp, _u32, _i32, _u32, _u32, _vp],
+    "decdec_mix_embed": [_vp, _vp, _vp, _vp, _i32, _u32, _u32, _u32, _vp],
+    "decdec_mix_gated_residual": [_vp, _vp, _vp, _u32, _vp, _vp, _vp, _vp, _vp, _i32, _u32, _u32, _f32, _vp],
+    "decdec_mix_rmsnorm": [_vp, _vp, _vp, _i32, _u32, _u32, _f32, _vp],
+    "decdec_mix_xielu": [_vp, _u32, _vp, _vp, _i32, _u32, _u32, _vp],
+    "decdec_mix_group_norm_gate": [_vp, _vp, _u32, _vp, _vp, _i32, _u32, _u32, _u32, _f32, _i32, _vp],
+    "decdec_mix_recurrence_step": [_rec, _vp, _vp, _vp, _f32, _i32, _i32, _vp],
+    "decdec_mix_recurrence_step_fuses": [_u32, _u32],
+    "decdec_mix_recurrence_rows": [_rec, _vp, _vp, _u64, _i32, _u32, _vp],
+    "decdec_mix_latent_append": [_lat, _vp, _i32, _u32, _vp],
+    "decdec_mix_latent_attention": [_lat, _vp, _vp, _vp, _u32, _vp, _i32, _u32, _u32, _vp],
+    "decdec_mix_latent_step": [_lat, _vp, _vp, _u64, _i32, _vp],
+}
+MIXERS_OTHER = {"decdec_mixers_last_error": ([], ctypes.c_char_p),
+                "decdec_mix_recurrence_workspace": ([_rec, _u32], _u64),
+                "decdec_mix_latent_step_workspace": ([_lat], _u64)}
+
+
+def load_mixers():
+    """Load libdecdec_mixers.so once; raise RuntimeError if it has not been built."""
+    global _mixers
+    if _mixers is not None:
+        return _mixers
+    if not os.path.exists(MIXERS_LIB_PATH):
+        raise RuntimeError(f"{MIXERS_LIB_PATH} is missing: build it with `python -m decdec_amd.build` "
+                           "(there is no CPU or PyTorch fallback for these ops)")
+    lib = ctypes.CDLL(MIXERS_LIB_PATH)
+    for name, argtypes in MIXERS_SIGNATURES.items():
+        fn = getattr(lib, name)
+        fn.argtypes, fn.restype = argtypes, _i32
+    for name, (argtypes, restype) in MIXERS_OTHER.items():
+        fn = getattr(lib, name)
+        fn.argtypes, fn.restype = argtypes, restype
+    _mixers = lib
+    return lib
+
+
+def check_mixers(status: int) -> None:
+    if status != 0:
+        raise RuntimeError(load_mixers().decdec_mixers_last_error().decode("utf-8", "replace"))
 
 
 def last_error() -> str:

@@ -1,8 +1,9 @@
-"""Builds libdecdec_hip.so (the gfx950 kernels + C ABI) in-tree with hipcc.
+"""Builds the gfx950 libraries in-tree with hipcc: libdecdec_hip.so (quantised linears, DEC, decode helpers) and
+libdecdec_mixers.so (recurrences, latent attention and the row kernels of decoders built from them).
 
-Usage: ``python -m decdec_amd.build`` or ``decdec_amd.build.build_library()``.
+Usage: ``python -m decdec_amd.build`` or ``decdec_amd.build.build_library()``; ``build_library(["mixers"])`` builds one.
 hipcc cross-compiles for gfx950 without a GPU.  The translation units are compiled in parallel and
-linked into ``decdec_amd/libdecdec_hip.so``.
+linked into ``decdec_amd/``.
 """
 from __future__ import annotations
 
@@ -18,7 +19,10 @@ CSRC = os.path.join(HERE, "csrc")
 OBJ_DIR = os.path.join(CSRC, "obj")
 LIB_PATH = os.path.join(HERE, "libdecdec_hip.so")
 RESOURCES_PATH = os.path.join(OBJ_DIR, "kernel_resources.json")
+MIXERS_LIB_PATH = os.path.join(HERE, "libdecdec_mixers.so")
 SOURCES = ["k_dec.hip", "k_anyprec.hip", "k_lutgemm.hip", "k_sqllm.hip", "k_decode.hip", "capi.hip"]
+MIXERS_SOURCES = ["k_rows.hip", "k_recurrence.hip", "k_latent.hip", "capi_mixers.hip"]
+LIBRARIES = {"linears": (LIB_PATH, SOURCES), "mixers": (MIXERS_LIB_PATH, MIXERS_SOURCES)}
 ARCH = "gfx950"
 
 # -packed-fp32-ops switches the packed-FP32 VALU forms off for the device pass (the host pass
@@ -79,7 +83,7 @@ def check_resources(kernels: dict) -> list:
       (a kernel with scratch pays for its set-up at every wave launch)."""
     bad = []
     for name, r in kernels.items():
-        two = "Lb1E" in name and "dec_" in name
+        two = "Lb1E" in name and re.search(r"dec_(anyprec|lutgemm|sqllm)", name) is not None
         fp32 = "kernelILi0E" in name
         if two and not fp32 and "lutgemm" not in name and (r.get("occupancy", 0) < 8 or r.get("scratch", 0) != 0):
             bad.append(f"{name}: budgeted instance has occupancy {r.get('occupancy')} / scratch {r.get('scratch')}")
@@ -91,25 +95,32 @@ def check_resources(kernels: dict) -> list:
     return bad
 
 
-def build_library(verbose: bool = True) -> str:
+def build_library(names=None, verbose: bool = True) -> str:
+    """Compiles and links the libraries `names` (all by default); returns the path of the last one."""
     os.makedirs(OBJ_DIR, exist_ok=True)
-    with ThreadPoolExecutor(max_workers=min(len(SOURCES), 8)) as ex:
-        results = list(ex.map(_compile, SOURCES))
-    objs = [o for o, _ in results]
+    libs = [LIBRARIES[n] for n in (names or LIBRARIES)]
+    sources = [src for _, srcs in libs for src in srcs]
+    with ThreadPoolExecutor(max_workers=min(len(sources), 8)) as ex:
+        results = dict(zip(sources, ex.map(_compile, sources)))
     kernels = {}
-    for _, k in results:
+    for _, k in results.values():
         kernels.update(k)
-    with open(RESOURCES_PATH, "w") as f:
-        json.dump(kernels, f, indent=1, sort_keys=True)
+    if names is None:
+        with open(RESOURCES_PATH, "w") as f:
+            json.dump(kernels, f, indent=1, sort_keys=True)
     for msg in check_resources(kernels):
         print(f"register budget: {msg}", file=sys.stderr)
-    cmd = [_hipcc(), f"--offload-arch={ARCH}", "-shared", "-fPIC", "-o", LIB_PATH, *objs]
-    proc = subprocess.run(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
-    if proc.returncode != 0:
-        raise RuntimeError(f"link failed:\n{proc.stdout}")
-    if verbose:
-        print(f"built {LIB_PATH}")
-    return LIB_PATH
+    for path, srcs in libs:
+        # linked under a name of its own and moved into place, so that nothing ever loads half a library
+        part = f"{path}.{os.getpid()}.part"
+        cmd = [_hipcc(), f"--offload-arch={ARCH}", "-shared", "-fPIC", "-o", part, *[results[s][0] for s in srcs]]
+        proc = subprocess.run(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
+        if proc.returncode != 0:
+            raise RuntimeError(f"link failed:\n{proc.stdout}")
+        os.replace(part, path)
+        if verbose:
+            print(f"built {path}")
+    return libs[-1][0]
 
 
 if __name__ == "__main__":

@@ -1,0 +1,626 @@
+// Linear recurrences with a 32-bit state per head: a decayed sum of outer products, and the gated delta rule.
+//
+// One token (decode): one kernel reads the state once, updates it in place and forms the read-out.
+// Many tokens: chunks of 64.  With G_i the log-decay summed from the chunk's start to token i, S0 the state before the
+// chunk and u_j the vector token j writes (its value in the plain form),
+//     o_i = e^{G_i} q_i S0 + sum_{j <= i} e^{G_i - G_j} (q_i . k_j) u_j
+//     S1  = e^{G_C} S0 + sum_j e^{G_C - G_j} k_j u_j^T
+// and for the delta rule, with A_ij = beta_i e^{G_i - G_j} (k_i . k_j) below the diagonal,
+//     (I + A) u = diag(beta) v - diag(beta e^G) k S0   =>   u = U - W S0.
+// Kernels: inputs (activation, convolution, unit norms, gates), U and W of every chunk (all chunks at once), states (one
+// walk over the chunks per head and 16 state columns), read-out (all chunks at once).  All of it in fp32, the products on
+// v_mfma_f32_16x16x4_f32.
+#include "mixers.h"
+#include "mma.h"
+
+namespace decdec {
+
+constexpr uint32_t C = kChunkRows;
+
+template <int DT>
+__device__ __forceinline__ float log_decay(const decdec_recurrence& p, const void* proj, size_t row, uint32_t h) {
+    using E = Elem<DT>;
+    return -expf(E::load(p.A_log, h)) * softplus_f(E::load(proj, row + p.off_a + h) + E::load(p.dt_bias, h));
+}
+
+// ---- one token --------------------------------------------------------------------------------------------
+// grid (heads, column splits); a thread owns RPT rows (of `dim`) of one state column.  cw columns per workgroup.
+template <int DT, bool DELTA, int RPT>
+__global__ __launch_bounds__(1024) void recurrence_step_kernel(const decdec_recurrence p, float* __restrict__ o_out,
+                                                               void* __restrict__ out, const void* __restrict__ norm_weight,
+                                                               const float eps, const int kind, const uint32_t cw) {
+    using E = Elem<DT>;
+    __shared__ float qs[512], ks[512], red[17], pa[1024], pb[1024];
+    const uint32_t tid = threadIdx.x, h = blockIdx.x, kg = tid / cw, KG = blockDim.x / cw;
+    const uint32_t D = p.dim, V = p.vdim, col = blockIdx.y * cw + tid % cw;
+    const bool live = col < V;
+    const long long pos = *p.pos;
+    const bool fresh = pos <= 0;
+    float* S = p.state + (size_t)h * D * V;
+    float s[RPT];
+#pragma unroll
+    for (int i = 0; i < RPT; ++i) {
+        const uint32_t r = kg + (uint32_t)i * KG;
+        s[i] = (r < D && live && !fresh) ? S[(size_t)r * V + col] : 0.f;
+    }
+    float v = 0.f, g = 0.f, beta = 1.f;
+    if constexpr (!DELTA) {
+        for (uint32_t i = tid; i < D; i += blockDim.x) {
+            qs[i] = silu_f(E::load(p.proj, p.off_q + h * D + i));
+            ks[i] = silu_f(E::load(p.proj, p.off_k + h * D + i));
+        }
+        if (live) v = silu_f(E::load(p.proj, p.off_v + h * V + col));
+        g = p.decay[(size_t)h * 65u + 1u];
+    } else {
+        const uint32_t share = p.heads / p.kv_heads, kvh = h / share, taps = p.taps;
+        const uint32_t qk = p.kv_heads * D, chans = 2u * qk + p.heads * V;
+        const bool keeper = h % share == 0u && blockIdx.y == 0u;
+        const uint32_t slot = (uint32_t)(pos < 0 ? 0 : pos % (long long)taps);
+        // channel c of the ring, whose projection is proj[src] and whose taps are w[wc * taps ..]
+        auto conv = [&](uint32_t src, uint32_t c, const void* w, uint32_t wc, bool keep) {
+            const uint32_t raw = E::load_raw(p.proj, src);
+            float y = E::load(w, (size_t)wc * taps + taps - 1u) * E::from_raw(raw);
+            for (uint32_t b = 1; b < taps; ++b) {                          // b tokens back
+                if (pos < (long long)b) break;
+                const uint32_t sl = (slot + taps - b) % taps;
+                y = __builtin_fmaf(E::load(w, (size_t)wc * taps + taps - 1u - b), E::load(p.ring, (size_t)sl * chans + c), y);
+            }
+            if (keep) ((typename LaneOf<DT>::t*)p.ring)[(size_t)slot * chans + c] = ((const typename LaneOf<DT>::t*)p.proj)[src];
+            return silu_f(y);
+        };
+        float sq = 0.f, sk = 0.f;
+        for (uint32_t i = tid; i < 2u * D; i += blockDim.x) {
+            const bool isq = i < D;
+            const uint32_t ch = kvh * D + (isq ? i : i - D);
+            const float y = conv((isq ? p.off_q : p.off_k) + ch, (isq ? 0u : qk) + ch, isq ? p.conv_q : p.conv_k, ch, keeper);
+            (isq ? qs : ks)[isq ? i : i - D] = y;
+            sq += isq ? y * y : 0.f;
+            sk += isq ? 0.f : y * y;
+        }
+        if (live) v = conv(p.off_v + h * V + col, 2u * qk + h * V + col, p.conv_v, h * V + col, kg == 0u);
+        g = expf(log_decay<DT>(p, p.proj, 0, h));
+        beta = sigmoid_f(E::load(p.proj, p.off_b + h));
+        sq = block_sum(sq, red);
+        sk = block_sum(sk, red);
+        const float rq = 1.f / sqrtf(sq + 1e-6f) / sqrtf((float)D), rk = 1.f / sqrtf(sk + 1e-6f);
+        for (uint32_t i = tid; i < D; i += blockDim.x) { qs[i] *= rq; ks[i] *= rk; }
+    }
+    __syncthreads();
+    // a = k . gS, b = q . gS over this thread's rows; o = b + (q . k) u
+    float a = 0.f, b = 0.f, qk = 0.f;
+#pragma unroll
+    for (int i = 0; i < RPT; ++i) {
+        const uint32_t r = kg + (uint32_t)i * KG;
+        const float kr = r < D ? ks[r] : 0.f, qr = r < D ? qs[r] : 0.f;
+        s[i] *= g;
+        a = __builtin_fmaf(kr, s[i], a);
+        b = __builtin_fmaf(qr, s[i], b);
+        qk = __builtin_fmaf(kr, qr, qk);
+    }
+    pa[tid] = DELTA ? a : qk;
+    pb[tid] = b;
+    __shared__ float pq[1024];
+    if constexpr (DELTA) pq[tid] = qk;
+    __syncthreads();
+    a = 0.f; b = 0.f; qk = 0.f;
+    for (uint32_t j = 0; j < KG; ++j) {
+        const uint32_t at = j * cw + tid % cw;
+        a += pa[at];
+        b += pb[at];
+        if constexpr (DELTA) qk += pq[at];
+    }
+    float u;
+    if constexpr (DELTA) u = beta * (v - a); else { u = v; qk = a; }
+    const float o = __builtin_fmaf(qk, u, b);
+#pragma unroll
+    for (int i = 0; i < RPT; ++i) {
+        const uint32_t r = kg + (uint32_t)i * KG;
+        if (r < D && live) S[(size_t)r * V + col] = __builtin_fmaf(ks[r], u, s[i]);
+    }
+    if (out == nullptr) {
+        if (kg == 0u && live) o_out[(size_t)h * V + col] = o;
+        return;
+    }
+    const float ss = block_sum(kg == 0u && live ? o * o : 0.f, red);
+    if (kg == 0u && live) {
+        const float z = E::load(p.proj, p.off_g + h * V + col);
+        const float gt = kind == DECDEC_GATE_SILU ? silu_f(z) : sigmoid_f(z);
+        E::store(out, (size_t)h * V + col, o / sqrtf(ss / (float)V + eps) * E::load(norm_weight, col) * gt);
+    }
+}
+
+struct StepShape { uint32_t cw, threads, rpt; };
+static StepShape step_shape(uint32_t D, uint32_t V, bool whole_head) {
+    uint32_t cw = 32;
+    if (whole_head) while (cw < V && cw < 1024u) cw *= 2;
+    const uint32_t threads = whole_head ? 1024u : 512u, KG = threads / cw;
+    return {cw, threads, (D + KG - 1u) / KG};
+}
+
+bool recurrence_step_fuses(uint32_t dim, uint32_t vdim) {
+    const StepShape s = step_shape(dim, vdim, true);
+    return s.cw >= vdim && s.rpt <= 32u;
+}
+
+template <int DT, bool DELTA>
+static hipError_t step_dt(const decdec_recurrence& p, float* o, void* out, const void* nw, float eps, int kind, hipStream_t s) {
+    const StepShape sh = step_shape(p.dim, p.vdim, out != nullptr);
+    const dim3 grid(p.heads, (p.vdim + sh.cw - 1u) / sh.cw), block(sh.threads);
+    if (sh.rpt <= 4) hipLaunchKernelGGL((recurrence_step_kernel<DT, DELTA, 4>), grid, block, 0, s, p, o, out, nw, eps, kind, sh.cw);
+    else if (sh.rpt <= 16) hipLaunchKernelGGL((recurrence_step_kernel<DT, DELTA, 16>), grid, block, 0, s, p, o, out, nw, eps, kind, sh.cw);
+    else if (sh.rpt <= 32) hipLaunchKernelGGL((recurrence_step_kernel<DT, DELTA, 32>), grid, block, 0, s, p, o, out, nw, eps, kind, sh.cw);
+    else return hipErrorInvalidValue;
+    return hipGetLastError();
+}
+
+hipError_t launch_recurrence_step(int dt, const decdec_recurrence& p, float* o, void* out, const void* nw, float eps, int kind,
+                                  hipStream_t s) {
+    if (dt == kBF16) return p.delta ? step_dt<kBF16, true>(p, o, out, nw, eps, kind, s) : step_dt<kBF16, false>(p, o, out, nw, eps, kind, s);
+    return p.delta ? step_dt<kFP32, true>(p, o, out, nw, eps, kind, s) : step_dt<kFP32, false>(p, o, out, nw, eps, kind, s);
+}
+
+// ---- many tokens ------------------------------------------------------------------------------------------
+struct ChunkParams {
+    const float* q;          // [rows][kv_heads][dim]
+    const float* k;
+    const float* v;          // [rows][heads][vdim]
+    const float* lg;         // [rows][heads] log-decays (delta)
+    const float* beta;       // [rows][heads] (delta)
+    float* u;                // [rows][heads][vdim]: U, then the written vectors (delta; the values themselves otherwise)
+    float* w;                // [rows][heads][dim] (delta)
+    float* states;           // [chunks][heads][dim][vdim]
+    const float* decay;      // [heads][65] (plain)
+    float* state;
+    float* o;
+    const long long* pos;
+    uint32_t rows, heads, kv_heads, dim, vdim;
+};
+
+template <int DT>
+__global__ __launch_bounds__(256) void plain_inputs_kernel(const decdec_recurrence p, float* __restrict__ q, float* __restrict__ k,
+                                                           float* __restrict__ v) {
+    using E = Elem<DT>;
+    const uint32_t t = blockIdx.x, nq = p.heads * p.dim, nv = p.heads * p.vdim;
+    const size_t row = (size_t)t * p.ld;
+    for (uint32_t i = threadIdx.x; i < nq; i += 256u) {
+        q[(size_t)t * nq + i] = silu_f(E::load(p.proj, row + p.off_q + i));
+        k[(size_t)t * nq + i] = silu_f(E::load(p.proj, row + p.off_k + i));
+    }
+    for (uint32_t i = threadIdx.x; i < nv; i += 256u) v[(size_t)t * nv + i] = silu_f(E::load(p.proj, row + p.off_v + i));
+}
+
+template <int DT>
+__global__ __launch_bounds__(256) void delta_inputs_kernel(const decdec_recurrence p, float* __restrict__ q, float* __restrict__ k,
+                                                           float* __restrict__ v, float* __restrict__ lg, float* __restrict__ beta) {
+    using E = Elem<DT>;
+    const uint32_t t = blockIdx.x, tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, D = p.dim, taps = p.taps;
+    const uint32_t nqk = p.kv_heads * D, nv = p.heads * p.vdim, chans = 2u * nqk + nv;
+    const long long pos0 = *p.pos;
+    auto conv = [&](uint32_t off, uint32_t c, const void* w, uint32_t wc) {
+        float y = 0.f;
+        for (uint32_t b = 0; b < taps; ++b) {                              // b tokens back
+            float in;
+            if (b <= t) in = E::load(p.proj, (size_t)(t - b) * p.ld + off + wc);
+            else if (pos0 + (long long)t >= (long long)b) in = E::load(p.ring, (size_t)((pos0 + t - b) % taps) * chans + c);
+            else break;
+            y = __builtin_fmaf(E::load(w, (size_t)wc * taps + taps - 1u - b), in, y);
+        }
+        return silu_f(y);
+    };
+    for (uint32_t j = wave; j < 2u * p.kv_heads; j += 4u) {
+        const bool isq = j < p.kv_heads;
+        const uint32_t ch0 = (isq ? j : j - p.kv_heads) * D;
+        float y[8], ss = 0.f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            const uint32_t i = lane + 64u * e;
+            y[e] = i < D ? conv(isq ? p.off_q : p.off_k, (isq ? 0u : nqk) + ch0 + i, isq ? p.conv_q : p.conv_k, ch0 + i) : 0.f;
+            ss += y[e] * y[e];
+        }
+        float r = 1.f / sqrtf(wave_sum(ss) + 1e-6f);
+        if (isq) r /= sqrtf((float)D);
+        float* dst = (isq ? q : k) + (size_t)t * nqk + ch0;
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+            if (lane + 64u * e < D) dst[lane + 64u * e] = y[e] * r;
+    }
+    for (uint32_t i = tid; i < nv; i += 256u) v[(size_t)t * nv + i] = conv(p.off_v, 2u * nqk + i, p.conv_v, i);
+    for (uint32_t h = tid; h < p.heads; h += 256u) {
+        lg[(size_t)t * p.heads + h] = log_decay<DT>(p, p.proj, (size_t)t * p.ld, h);
+        beta[(size_t)t * p.heads + h] = sigmoid_f(E::load(p.proj, (size_t)t * p.ld + p.off_b + h));
+    }
+}
+
+// The last min(rows, taps) projections into the ring (after delta_inputs has read the old ones).
+template <int DT>
+__global__ __launch_bounds__(256) void ring_update_kernel(const decdec_recurrence p, const uint32_t rows) {
+    using T = typename LaneOf<DT>::t;
+    const uint32_t nqk = p.kv_heads * p.dim, nv = p.heads * p.vdim, chans = 2u * nqk + nv;
+    const uint32_t c = blockIdx.x * 256u + threadIdx.x, t = rows - 1u - blockIdx.y;
+    if (c >= chans) return;
+    const uint32_t src = c < nqk ? p.off_q + c : (c < 2u * nqk ? p.off_k + c - nqk : p.off_v + c - 2u * nqk);
+    const uint32_t slot = (uint32_t)((*p.pos + (long long)t) % p.taps);
+    ((T*)p.ring)[(size_t)slot * chans + c] = ((const T*)p.proj)[(size_t)t * p.ld + src];
+}
+
+// Log-decays of a chunk summed up, in double: exponents are taken of differences, which must not lose what a long sum
+// has swallowed.  One wave.
+__device__ __forceinline__ void chunk_log_decay(const ChunkParams& p, uint32_t t0, uint32_t n, uint32_t h, double* G) {
+    const uint32_t lane = threadIdx.x & 63u;
+    double x = lane < n ? (double)p.lg[(size_t)(t0 + lane) * p.heads + h] : 0.0;
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) {
+        const double y = __shfl_up(x, off, 64);
+        if ((int)lane >= off) x += y;
+    }
+    G[lane] = x;
+}
+
+// eight floats of a row, zero past `valid`
+__device__ __forceinline__ Frag<kFP32> row_frag(const float* p, int valid, bool vec) {
+    Frag<kFP32> f;
+    if (vec && valid >= 8) return frag_load(p);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) f.v[i] = i < valid ? p[i] : 0.f;
+    return f;
+}
+
+// 64 rows x 32 columns of an array of rows (stride ld) into LDS [64][36]; rows past n and columns past D are zero.
+__device__ __forceinline__ void load_slice(const float* src, size_t ld, uint32_t n, uint32_t c0, uint32_t D, float (*dst)[36], bool vec) {
+    const uint32_t tid = threadIdx.x;
+#pragma unroll
+    for (uint32_t e = 0; e < 2; ++e) {
+        const uint32_t i = tid + 256u * e, r = i >> 3, c = (i & 7u) * 4u;
+        f32x4 x = {0.f, 0.f, 0.f, 0.f};
+        if (r < n) {
+            const float* s = src + (size_t)r * ld + c0 + c;
+            if (vec && c0 + c + 4u <= D) x = *(const f32x4*)s;
+            else
+#pragma unroll
+                for (int j = 0; j < 4; ++j) x[j] = c0 + c + (uint32_t)j < D ? s[j] : 0.f;
+        }
+        *(f32x4*)&dst[r][c] = x;
+    }
+}
+
+// U and W of a chunk: grid (chunks, heads).
+__global__ __launch_bounds__(256) void delta_solve_kernel(const ChunkParams p) {
+    __shared__ __align__(16) float Ks[C][36];
+    __shared__ __align__(16) float A[C][C + 4];
+    __shared__ __align__(16) float T[C][20];                // inverses of the diagonal blocks
+    __shared__ double G[C];
+    __shared__ float beta[C];
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, h = blockIdx.y, kvh = h / (p.heads / p.kv_heads);
+    const uint32_t t0 = blockIdx.x * C, n = p.rows - t0 < C ? p.rows - t0 : C, D = p.dim, V = p.vdim;
+    const float* k = p.k + ((size_t)t0 * p.kv_heads + kvh) * D;
+    const size_t kld = (size_t)p.kv_heads * D;
+    const bool vec = D % 4u == 0;
+    if (wave == 0) {
+        chunk_log_decay(p, t0, n, h, G);
+        beta[lane] = lane < n ? p.beta[(size_t)(t0 + lane) * p.heads + h] : 0.f;
+    }
+    f32x4 acc[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (uint32_t c0 = 0; c0 < D; c0 += 32u) {
+        __syncthreads();
+        load_slice(k, kld, n, c0, D, Ks, vec);
+        __syncthreads();
+        const Frag<kFP32> a = frag_load(&Ks[16u * wave + (lane & 15u)][8u * (lane >> 4)]);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) mma(a, frag_load(&Ks[16u * j + (lane & 15u)][8u * (lane >> 4)]), acc[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            const uint32_t r = 16u * wave + 4u * (lane >> 4) + (uint32_t)v, c = 16u * (uint32_t)j + (lane & 15u);
+            A[r][c] = c < r ? beta[r] * acc[j][v] * expf((float)(G[r] - G[c])) : 0.f;
+        }
+    __syncthreads();
+    // inverses of the four unit lower-triangular 16 x 16 blocks on the diagonal, a thread per column
+    if (tid < C) {
+        const uint32_t b = tid & ~15u, j = tid & 15u;
+        float t[16];
+#pragma unroll
+        for (uint32_t i = 0; i < 16u; ++i) {
+            float y = i == j ? 1.f : 0.f;
+#pragma unroll
+            for (uint32_t m = 0; m < i; ++m) y = __builtin_fmaf(-A[b + i][b + m], t[m], y);
+            t[i] = y;
+            T[b + i][j] = y;
+        }
+    }
+    __syncthreads();
+    // (I + A) X = B, block row by block row, a wave per 16 columns of B: an accumulator tile is at once the right
+    // operand of the next product (row 4 (lane / 16) + v of the block in register v)
+    const uint32_t l16 = lane & 15u, lg = lane >> 4;
+    for (uint32_t c0 = 16u * wave; c0 < V + D; c0 += 64u) {
+        const uint32_t c = c0 + l16;
+        const bool isv = c < V, live = c < V + D;
+        const float* src = isv ? p.v + ((size_t)t0 * p.heads + h) * V + c : k + (live ? c - V : 0u);
+        const size_t ld = isv ? (size_t)p.heads * V : kld;
+        float* dst = isv ? p.u + ((size_t)t0 * p.heads + h) * V + c : p.w + ((size_t)t0 * p.heads + h) * D + (live ? c - V : 0u);
+        const size_t dld = (size_t)p.heads * (isv ? V : D);
+        f32x4 x[4];
+#pragma unroll
+        for (uint32_t b = 0; b < 4u; ++b)
+#pragma unroll
+            for (uint32_t v = 0; v < 4u; ++v) {
+                const uint32_t i = 16u * b + 4u * lg + v;
+                float y = (live && i < n) ? src[(size_t)i * ld] * beta[i] : 0.f;
+                if (!isv) y *= expf((float)G[i]);
+                x[b][v] = y;
+            }
+#pragma unroll
+        for (uint32_t b = 0; b < 4u; ++b) {
+#pragma unroll
+            for (uint32_t m = 0; m < b; ++m) {
+                const f32x4 a = *(const f32x4*)&A[16u * b + l16][16u * m + 4u * lg];
+#pragma unroll
+                for (uint32_t e = 0; e < 4u; ++e) x[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(-a[e], x[m][e], x[b], 0, 0, 0);
+            }
+            const f32x4 a = *(const f32x4*)&T[16u * b + l16][4u * lg];
+            f32x4 y = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (uint32_t e = 0; e < 4u; ++e) y = __builtin_amdgcn_mfma_f32_16x16x4f32(a[e], x[b][e], y, 0, 0, 0);
+            x[b] = y;
+        }
+#pragma unroll
+        for (uint32_t b = 0; b < 4u; ++b)
+#pragma unroll
+            for (uint32_t v = 0; v < 4u; ++v) {
+                const uint32_t i = 16u * b + 4u * lg + v;
+                if (live && i < n) dst[(size_t)i * dld] = x[b][v];
+            }
+    }
+}
+
+// States: grid (heads, vdim / 16), one walk over the chunks.  Wave w owns the state's row tiles w, w + 4, ... (NT of them).
+template <bool DELTA, int NT>
+__global__ __launch_bounds__(256) void chunk_state_kernel(const ChunkParams p, const uint32_t chunks) {
+    extern __shared__ __align__(16) float lds[];
+    __shared__ double G[C];
+    __shared__ __align__(16) float Vl[C][20];
+    __shared__ float pw[C + 1];
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, l16 = lane & 15u, lg = lane >> 4;
+    const uint32_t h = blockIdx.x, kvh = h / (p.heads / p.kv_heads), D = p.dim, V = p.vdim, v0 = blockIdx.y * 16u;
+    const uint32_t Dp = (D + 31u) & ~31u, KL = Dp + 4u, tiles = Dp / 16u;
+    float* Kl = lds;                        // [C][KL]
+    float* Sl = lds + C * KL;               // [Dp][20]
+    const bool fresh = *p.pos <= 0, vec = D % 4u == 0, vec8 = D % 8u == 0, col = v0 + l16 < V;
+    float* S = p.state + (size_t)h * D * V + v0 + l16;
+    if constexpr (!DELTA) { for (uint32_t i = tid; i <= C; i += 256u) pw[i] = p.decay[(size_t)h * 65u + i]; }
+    f32x4 s[NT];
+#pragma unroll
+    for (int i = 0; i < NT; ++i)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            const uint32_t r = 16u * (wave + 4u * (uint32_t)i) + 4u * lg + (uint32_t)v;
+            s[i][v] = (r < D && col && !fresh) ? S[(size_t)r * V] : 0.f;
+        }
+    for (uint32_t ch = 0; ch < chunks; ++ch) {
+        const uint32_t t0 = ch * C, n = p.rows - t0 < C ? p.rows - t0 : C;
+        const float* k = p.k + ((size_t)t0 * p.kv_heads + kvh) * D;
+        const size_t kld = (size_t)p.kv_heads * D;
+        for (uint32_t i = tid; i < C * (Dp / 4u); i += 256u) {
+            const uint32_t r = i / (Dp / 4u), c = (i % (Dp / 4u)) * 4u;
+            f32x4 x = {0.f, 0.f, 0.f, 0.f};
+            if (r < n) {
+                if (vec && c + 4u <= D) x = *(const f32x4*)(k + (size_t)r * kld + c);
+                else
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) x[j] = c + (uint32_t)j < D ? k[(size_t)r * kld + c + j] : 0.f;
+            }
+            *(f32x4*)&Kl[r * KL + c] = x;
+        }
+        if constexpr (DELTA) { if (wave == 3) chunk_log_decay(p, t0, n, h, G); }
+        float* st = p.states + ((size_t)ch * p.heads + h) * D * V + v0 + l16;
+#pragma unroll
+        for (int i = 0; i < NT; ++i)
+#pragma unroll
+            for (int v = 0; v < 4; ++v) {
+                const uint32_t r = 16u * (wave + 4u * (uint32_t)i) + 4u * lg + (uint32_t)v;
+                if (r < Dp) Sl[r * 20u + l16] = s[i][v];
+                if (r < D && col) st[(size_t)r * V] = s[i][v];
+            }
+        __syncthreads();
+        const float gend = DELTA ? expf((float)G[C - 1]) : pw[n];
+        {
+            // what the tokens write, 16 rows per wave
+            f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+            if constexpr (DELTA) {
+                const uint32_t ar = 16u * wave + l16;
+                const float* w = p.w + ((size_t)(t0 + (ar < n ? ar : 0u)) * p.heads + h) * D;
+                for (uint32_t c0 = 0; c0 < D; c0 += 32u) {
+                    const uint32_t kk = c0 + 8u * lg;
+                    const Frag<kFP32> a = row_frag(w + kk, ar < n ? (int)D - (int)kk : 0, vec8);
+                    mma(a, frag_gather(Sl + kk * 20u + l16, 20u), acc);
+                }
+            }
+#pragma unroll
+            for (int v = 0; v < 4; ++v) {
+                const uint32_t r = 16u * wave + 4u * lg + (uint32_t)v;
+                float x = 0.f;
+                if (r < n && col) {
+                    const size_t at = ((size_t)(t0 + r) * p.heads + h) * V + v0 + l16;
+                    if constexpr (DELTA) {
+                        x = p.u[at] - acc[v];
+                        p.u[at] = x;
+                        x *= expf((float)(G[C - 1] - G[r]));
+                    } else {
+                        x = p.v[at] * pw[n - 1u - r];
+                    }
+                }
+                Vl[r][l16] = x;
+            }
+        }
+        __syncthreads();
+#pragma unroll
+        for (int i = 0; i < NT; ++i) {
+            const uint32_t tile = wave + 4u * (uint32_t)i;
+            s[i] *= gend;
+            if (tile < tiles) {
+#pragma unroll
+                for (uint32_t j0 = 0; j0 < C; j0 += 32u)
+                    mma(frag_gather(Kl + (j0 + 8u * lg) * KL + 16u * tile + l16, KL), frag_gather(&Vl[j0 + 8u * lg][l16], 20u), s[i]);
+            }
+        }
+        __syncthreads();
+    }
+#pragma unroll
+    for (int i = 0; i < NT; ++i)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            const uint32_t r = 16u * (wave + 4u * (uint32_t)i) + 4u * lg + (uint32_t)v;
+            if (r < D && col) S[(size_t)r * V] = s[i][v];
+        }
+}
+
+// Read-out: grid (chunks, heads, vdim / 64).
+template <bool DELTA>
+__global__ __launch_bounds__(256) void chunk_output_kernel(const ChunkParams p) {
+    __shared__ __align__(16) float Qs[C][36];
+    __shared__ __align__(16) float Ks[C][36];
+    __shared__ __align__(16) float Ss[32][68];
+    __shared__ __align__(16) float Ps[C][68];
+    __shared__ __align__(16) float Vs[C][68];
+    __shared__ double G[C];
+    __shared__ float pw[C + 1];
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, l16 = lane & 15u, lg = lane >> 4;
+    const uint32_t h = blockIdx.y, kvh = h / (p.heads / p.kv_heads), D = p.dim, V = p.vdim, v0 = blockIdx.z * 64u;
+    const uint32_t t0 = blockIdx.x * C, n = p.rows - t0 < C ? p.rows - t0 : C;
+    const bool vec = D % 4u == 0;
+    const size_t kld = (size_t)p.kv_heads * D;
+    const float* q = p.q + ((size_t)t0 * p.kv_heads + kvh) * D;
+    const float* k = p.k + ((size_t)t0 * p.kv_heads + kvh) * D;
+    const float* vv = (DELTA ? p.u : p.v) + ((size_t)t0 * p.heads + h) * V;
+    const float* S = p.states + ((size_t)blockIdx.x * p.heads + h) * D * V;
+    if constexpr (DELTA) { if (wave == 0) chunk_log_decay(p, t0, n, h, G); }
+    else { for (uint32_t i = tid; i <= C; i += 256u) pw[i] = p.decay[(size_t)h * 65u + i]; }
+    for (uint32_t i = tid; i < C * 64u; i += 256u) {
+        const uint32_t r = i >> 6, c = i & 63u;
+        Vs[r][c] = (r < n && v0 + c < V) ? vv[(size_t)r * p.heads * V + v0 + c] : 0.f;
+    }
+    f32x4 pr[4], o[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) { pr[j] = f32x4{0.f, 0.f, 0.f, 0.f}; o[j] = f32x4{0.f, 0.f, 0.f, 0.f}; }
+    for (uint32_t c0 = 0; c0 < D; c0 += 32u) {
+        __syncthreads();
+        load_slice(q, kld, n, c0, D, Qs, vec);
+        load_slice(k, kld, n, c0, D, Ks, vec);
+        for (uint32_t i = tid; i < 32u * 64u; i += 256u) {
+            const uint32_t r = i >> 6, c = i & 63u;
+            Ss[r][c] = (c0 + r < D && v0 + c < V) ? S[(size_t)(c0 + r) * V + v0 + c] : 0.f;
+        }
+        __syncthreads();
+        const Frag<kFP32> a = frag_load(&Qs[16u * wave + l16][8u * lg]);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            if ((uint32_t)j <= wave) mma(a, frag_load(&Ks[16u * j + l16][8u * lg]), pr[j]);
+            mma(a, frag_gather(&Ss[8u * lg][16u * j + l16], 68u), o[j]);
+        }
+    }
+    __syncthreads();                               // decays are in LDS also where D is a single slice; Ps follows
+#pragma unroll
+    for (int v = 0; v < 4; ++v) {
+        const uint32_t r = 16u * wave + 4u * lg + (uint32_t)v;
+        const float f0 = DELTA ? expf((float)G[r]) : pw[r + 1u];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const uint32_t c = 16u * (uint32_t)j + l16;
+            float d = 0.f;
+            if (c <= r) d = DELTA ? expf((float)(G[r] - G[c])) : pw[r - c];
+            Ps[r][c] = pr[j][v] * d;
+            o[j][v] *= f0;
+        }
+    }
+    __syncthreads();
+#pragma unroll
+    for (uint32_t j0 = 0; j0 < C; j0 += 32u) {
+        if (j0 > 16u * wave + 15u) break;
+        const Frag<kFP32> a = frag_load(&Ps[16u * wave + l16][j0 + 8u * lg]);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) mma(a, frag_gather(&Vs[j0 + 8u * lg][16u * j + l16], 68u), o[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            const uint32_t r = 16u * wave + 4u * lg + (uint32_t)v, c = v0 + 16u * (uint32_t)j + l16;
+            if (r < n && c < V) p.o[((size_t)(t0 + r) * p.heads + h) * V + c] = o[j][v];
+        }
+}
+
+static size_t pad4(size_t n) { return (n + 3u) & ~(size_t)3u; }
+static ChunkParams chunk_layout(const decdec_recurrence& p, uint32_t rows, float* base, size_t& floats) {
+    ChunkParams c{};
+    const size_t nq = pad4((size_t)rows * p.kv_heads * p.dim), nv = pad4((size_t)rows * p.heads * p.vdim), nh = pad4((size_t)rows * p.heads);
+    const size_t chunks = (rows + C - 1u) / C;
+    size_t at = 0;
+    auto take = [&](size_t n) { float* r = base == nullptr ? nullptr : base + at; at += n; return r; };
+    c.q = take(nq);
+    c.k = take(nq);
+    c.v = take(nv);
+    if (p.delta) {
+        c.lg = take(nh);
+        c.beta = take(nh);
+        c.u = take(nv);
+        c.w = take(pad4((size_t)rows * p.heads * p.dim));
+    }
+    c.states = take(pad4(chunks * p.heads * p.dim * p.vdim));
+    floats = at;
+    c.decay = p.decay;
+    c.state = p.state;
+    c.pos = (const long long*)p.pos;
+    c.rows = rows; c.heads = p.heads; c.kv_heads = p.kv_heads; c.dim = p.dim; c.vdim = p.vdim;
+    return c;
+}
+
+size_t recurrence_workspace(const decdec_recurrence& p, uint32_t rows) {
+    size_t n;
+    chunk_layout(p, rows, nullptr, n);
+    return n * sizeof(float);
+}
+
+template <bool DELTA, int NT>
+static hipError_t launch_state(const ChunkParams& c, uint32_t chunks, dim3 grid, size_t lds, hipStream_t s) {
+    if (hipError_t e = allow_lds<chunk_state_kernel<DELTA, NT>>(lds); e != hipSuccess) return e;
+    hipLaunchKernelGGL((chunk_state_kernel<DELTA, NT>), grid, dim3(256), lds, s, c, chunks);
+    return hipGetLastError();
+}
+
+template <bool DELTA>
+static hipError_t launch_chunks(const ChunkParams& c, hipStream_t s) {
+    const uint32_t chunks = (c.rows + C - 1u) / C, Dp = (c.dim + 31u) & ~31u, nt = (Dp / 16u + 3u) / 4u;
+    const size_t lds = ((size_t)C * (Dp + 4u) + (size_t)Dp * 20u) * sizeof(float);
+    const dim3 grid(c.heads, (c.vdim + 15u) / 16u), block(256);
+    hipError_t e = nt == 1u ? launch_state<DELTA, 1>(c, chunks, grid, lds, s) : nt == 2u ? launch_state<DELTA, 2>(c, chunks, grid, lds, s)
+                 : nt <= 4u ? launch_state<DELTA, 4>(c, chunks, grid, lds, s) : hipErrorInvalidValue;
+    if (e != hipSuccess) return e;
+    hipLaunchKernelGGL((chunk_output_kernel<DELTA>), dim3(chunks, c.heads, (c.vdim + 63u) / 64u), block, 0, s, c);
+    return hipGetLastError();
+}
+
+template <int DT>
+static hipError_t rows_dt(const decdec_recurrence& p, const ChunkParams& c, hipStream_t s) {
+    if (!p.delta) {
+        hipLaunchKernelGGL((plain_inputs_kernel<DT>), dim3(c.rows), dim3(256), 0, s, p, (float*)c.q, (float*)c.k, (float*)c.v);
+        return launch_chunks<false>(c, s);
+    }
+    hipLaunchKernelGGL((delta_inputs_kernel<DT>), dim3(c.rows), dim3(256), 0, s, p, (float*)c.q, (float*)c.k, (float*)c.v,
+                       (float*)c.lg, (float*)c.beta);
+    const uint32_t chans = 2u * p.kv_heads * p.dim + p.heads * p.vdim, keep = c.rows < p.taps ? c.rows : p.taps;
+    hipLaunchKernelGGL((ring_update_kernel<DT>), dim3((chans + 255u) / 256u, keep), dim3(256), 0, s, p, c.rows);
+    hipLaunchKernelGGL(delta_solve_kernel, dim3((c.rows + C - 1u) / C, p.heads), dim3(256), 0, s, c);
+    return launch_chunks<true>(c, s);
+}
+
+hipError_t launch_recurrence_rows(int dt, const decdec_recurrence& p, float* o, void* ws, uint32_t rows, hipStream_t s) {
+    size_t n;
+    ChunkParams c = chunk_layout(p, rows, (float*)ws, n);
+    c.o = o;
+    return dt == kBF16 ? rows_dt<kBF16>(p, c, s) : rows_dt<kFP32>(p, c, s);
+}
+
+}  // namespace decdec

@@ -1,0 +1,45 @@
+// Launch interface between the mixer kernels and their C ABI.
+#pragma once
+#include <hip/hip_runtime.h>
+#include "../../include/decdec_mixers.h"
+#include "common.h"
+
+namespace decdec {
+
+constexpr uint32_t kChunkRows = 64;        // tokens per chunk of a recurrence
+
+// Lets a kernel take more than 64 KB of dynamic LDS.
+template <auto Kernel>
+inline hipError_t allow_lds(size_t bytes) {
+    static thread_local size_t allowed = 64 * 1024;
+    if (bytes <= allowed) return hipSuccess;
+    const hipError_t e = hipFuncSetAttribute((const void*)Kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes);
+    if (e == hipSuccess) allowed = bytes;
+    return e;
+}
+
+hipError_t launch_mix_gemv(int dt, const void* w, const void* x, void* out, const void* act, uint32_t act_rows, uint32_t N,
+                           uint32_t K, hipStream_t s);
+hipError_t launch_mix_embed(int dt, const void* table, const long long* tokens, float* x, void* xe, uint32_t rows,
+                            uint32_t vocab, uint32_t dim, hipStream_t s);
+hipError_t launch_mix_gated_residual(int dt, float* x, const void* y, const void* gate, uint32_t gate_ld, const void* bias,
+                                     const void* weight, void* xe, const void* fw, void* fo, uint32_t rows, uint32_t dim,
+                                     float eps, hipStream_t s);
+hipError_t launch_mix_rmsnorm(int dt, const float* x, const void* weight, void* out, uint32_t rows, uint32_t dim, float eps,
+                              hipStream_t s);
+hipError_t launch_mix_xielu(int dt, const void* in, uint32_t ld, const void* act, void* out, uint32_t rows, uint32_t n,
+                            hipStream_t s);
+hipError_t launch_mix_group_norm_gate(int dt, const float* o, const void* gate, uint32_t ld, const void* weight, void* out,
+                                      uint32_t rows, uint32_t groups, uint32_t n, float eps, int kind, hipStream_t s);
+bool recurrence_step_fuses(uint32_t dim, uint32_t vdim);
+hipError_t launch_recurrence_step(int dt, const decdec_recurrence& p, float* o, void* out, const void* nw, float eps, int kind,
+                                  hipStream_t s);
+size_t recurrence_workspace(const decdec_recurrence& p, uint32_t rows);
+hipError_t launch_recurrence_rows(int dt, const decdec_recurrence& p, float* o, void* ws, uint32_t rows, hipStream_t s);
+hipError_t launch_latent_append(int dt, const decdec_latent& p, void* q_out, uint32_t rows, hipStream_t s);
+hipError_t launch_latent_attention(int dt, const decdec_latent& p, const void* q, const void* k, const void* vt, uint32_t vt_ld,
+                                   void* out, uint32_t start, uint32_t rows, hipStream_t s);
+size_t latent_step_workspace(const decdec_latent& p);
+hipError_t launch_latent_step(int dt, const decdec_latent& p, void* out, void* ws, hipStream_t s);
+
+}  // namespace decdec

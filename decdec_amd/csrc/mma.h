@@ -1,0 +1,95 @@
+// 16 x 16 matrix-core tiles with a contraction of 32, in one shape for bf16 and for fp32 operands.
+//
+// A lane holds eight consecutive elements (along the contraction) of one row of A and of one column of B: row / column
+// lane % 16, elements 8 (lane / 16) .. + 7.  bf16: one v_mfma_f32_16x16x32_bf16.  fp32: eight v_mfma_f32_16x16x4_f32, the
+// i-th with element i of every lane -- the contraction index runs in another order, the same one for A and B.
+// The result has row 4 (lane / 16) + v, column lane % 16 in register v.
+#pragma once
+#include "common.h"
+
+namespace decdec {
+
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+
+template <int DT> struct Frag;
+template <> struct Frag<kBF16> { u32x4 v; };
+template <> struct Frag<kFP32> { float v[8]; };
+
+__device__ __forceinline__ void mma(const Frag<kBF16>& a, const Frag<kBF16>& b, f32x4& c) {
+    bf16x8 x, y;
+    __builtin_memcpy(&x, &a.v, 16);
+    __builtin_memcpy(&y, &b.v, 16);
+    c = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x, y, c, 0, 0, 0);
+}
+__device__ __forceinline__ void mma(const Frag<kFP32>& a, const Frag<kFP32>& b, f32x4& c) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.v[i], b.v[i], c, 0, 0, 0);
+}
+
+// eight consecutive elements (16-byte aligned)
+__device__ __forceinline__ Frag<kBF16> frag_load(const uint16_t* p) {
+    Frag<kBF16> f;
+    f.v = *(const u32x4*)p;
+    return f;
+}
+__device__ __forceinline__ Frag<kFP32> frag_load(const float* p) {
+    Frag<kFP32> f;
+    const f32x4 a = *(const f32x4*)p, b = *(const f32x4*)(p + 4);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) { f.v[i] = a[i]; f.v[4 + i] = b[i]; }
+    return f;
+}
+// eight elements a stride apart
+__device__ __forceinline__ Frag<kFP32> frag_gather(const float* p, uint32_t stride) {
+    Frag<kFP32> f;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) f.v[i] = p[(size_t)i * stride];
+    return f;
+}
+__device__ __forceinline__ Frag<kBF16> frag_gather(const uint16_t* p, uint32_t stride) {
+    Frag<kBF16> f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+        f.v[i] = (uint32_t)p[(size_t)(2 * i) * stride] | ((uint32_t)p[(size_t)(2 * i + 1) * stride] << 16);
+    return f;
+}
+// fp32 values as operands: exact for fp32; for bf16 the sum of a leading and a trailing part (16 significant bits)
+__device__ __forceinline__ void frag_split(const float (&x)[8], Frag<kBF16>& hi, Frag<kBF16>& lo) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const uint32_t h0 = f32_to_bf16_bits(x[2 * i]), h1 = f32_to_bf16_bits(x[2 * i + 1]);
+        hi.v[i] = h0 | (h1 << 16);
+        lo.v[i] = (uint32_t)f32_to_bf16_bits(x[2 * i] - __uint_as_float(h0 << 16)) |
+                  ((uint32_t)f32_to_bf16_bits(x[2 * i + 1] - __uint_as_float(h1 << 16)) << 16);
+    }
+}
+__device__ __forceinline__ void frag_split(const float (&x)[8], Frag<kFP32>& hi, Frag<kFP32>&) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) hi.v[i] = x[i];
+}
+
+template <int DT> struct LaneOf { using t = uint16_t; };
+template <> struct LaneOf<kFP32> { using t = float; };
+
+__device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + __expf(-z)); }
+__device__ __forceinline__ float silu_f(float z) { return z * sigmoid_f(z); }
+__device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+// xIELU with the softplus of its two numbers already taken
+__device__ __forceinline__ float xielu_f(float z, float sp, float sq) {
+    return z > 0.f ? (sp * z + 0.5f) * z : (0.5f + sq) * (expm1f(z) - z) + 0.5f * z;
+}
+
+// Sum over a workgroup of `blockDim.x` (a multiple of 64) threads; red: at least 17 floats of LDS, free at the call.
+__device__ __forceinline__ float block_sum(float v, float* red) {
+    v = wave_sum(v);
+    const uint32_t lane = threadIdx.x & 63u, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
+    __syncthreads();
+    if (lane == 0) red[wave] = v;
+    __syncthreads();
+    float t = 0.f;
+    for (uint32_t w = 0; w < nw; ++w) t += red[w];
+    return t;
+}
+
+}  // namespace decdec
