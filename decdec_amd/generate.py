@@ -20,7 +20,7 @@ import time
 
 import torch
 
-from . import _lib, artifacts, decode_ops
+from . import _lib, artifacts, decode_ops, registry
 from .linear import APLinear, LUTGEMMLinear, SQLLMLinear
 from .model import DEC_MODULE_KEYS, Transformer
 
@@ -102,12 +102,54 @@ def random_dec_data(model: Transformer, thresholds: dict, seed: int = 2, residua
 # ----------------------------------------------------------------------------------------------------
 # decode
 # ----------------------------------------------------------------------------------------------------
+def model_device(model) -> torch.device:
+    return model.device if hasattr(model, "device") else model.tok_embeddings.weight.device
+
+
+class Session:
+    """One sequence being fed to a model in portions of any size: every portion runs only its own tokens, from the caches
+    and states the earlier ones left."""
+
+    def __init__(self, model, max_tokens: int, portion: int = 4096):
+        self.model, self.portion = model, portion
+        model.setup_caches(1, min(max_tokens, model.config.block_size))
+        assert max_tokens <= model.max_seq_length, "the sequence exceeds the cache"
+        model.state.release()
+
+    @property
+    def length(self) -> int:
+        return self.model.state.length
+
+    @torch.no_grad()
+    def feed(self, tokens, want=()) -> torch.Tensor:
+        """Runs `tokens` (ids, a list or a tensor); returns the logits [len(want), vocab] of the places `want` among them."""
+        dev = model_device(self.model)
+        tokens = torch.as_tensor(tokens, dtype=torch.int64).view(-1).to(dev)
+        n, want = tokens.numel(), list(want)
+        if any(not 0 <= w < n for w in want):
+            raise ValueError(f"wanted places {want} among {n} tokens")
+        rows = {}
+        for lo in range(0, n, self.portion):
+            hi, start = min(n, lo + self.portion), self.length
+            here = sorted({w for w in want if lo <= w < hi})
+            self.model.state.advance(start, hi - lo)
+            logits = self.model(tokens[None, lo:hi], torch.arange(start, start + hi - lo, device=dev), start=start,
+                                want=[w - lo for w in here])
+            if here:                                          # a one-token step returns its logits whatever is wanted
+                rows.update(zip(here, logits[0]))
+        return torch.stack([rows[w] for w in want]) if want else torch.empty(0, self.model.config.vocab_size, device=dev)
+
+    def close(self) -> None:
+        """Gives back what the sequence holds."""
+        self.model.state.release()
+
+
 class DecodeStep:
     """One greedy decode step on static buffers: logits of `token` at `pos`, argmax, the new token appended
     to `seq`, fed back into `token`, `pos` advanced.  `capture()` records it in a HIP graph."""
 
     def __init__(self, model: Transformer, max_tokens: int, keep_logits: bool = False):
-        dev = model.tok_embeddings.weight.device
+        dev = model_device(model)
         self.model = model
         self.token = torch.zeros(1, 1, dtype=torch.int64, device=dev)
         self.pos = torch.zeros(1, dtype=torch.int64, device=dev)
@@ -140,6 +182,7 @@ class DecodeStep:
     def capture(self):
         stream = torch.cuda.Stream()
         tok, pos, cnt = self.token.clone(), self.pos.clone(), self.count.clone()
+        saved = self.model.state.snapshot()
         # everything queued so far (weights being initialised, the zero fill of the step's own buffers, a prefill)
         # must have run before the step does: an unordered step would read its token before it was written
         stream.wait_stream(torch.cuda.current_stream())
@@ -151,6 +194,7 @@ class DecodeStep:
             self._step()
         torch.cuda.current_stream().wait_stream(stream)
         self.token.copy_(tok); self.pos.copy_(pos); self.count.copy_(cnt)
+        self.model.state.restore(saved)       # the warm-up step advanced the recurrent layers
         torch.cuda.synchronize()
 
     def run(self, n: int):
@@ -163,16 +207,16 @@ class DecodeStep:
 
 
 @torch.no_grad()
-def generate(model: Transformer, prompt: torch.Tensor, max_new_tokens: int, use_graph: bool = True,
+def generate(model, prompt: torch.Tensor, max_new_tokens: int, use_graph: bool = True,
              max_seq_length: int | None = None):
     """Greedy decode; returns (tokens [T + max_new_tokens], seconds spent on the max_new_tokens - 1 decode steps)."""
     T = prompt.numel()
     total = T + max_new_tokens
-    model.setup_caches(1, min(max_seq_length or total, model.config.block_size))
-    assert total <= model.max_seq_length, "prompt + new tokens exceed the cache"
     dev = prompt.device
-    logits = model(prompt.view(1, -1), torch.arange(T, device=dev))
-    first = int(torch.argmax(logits[0, -1]))
+    session = Session(model, min(max_seq_length or total, model.config.block_size))
+    assert total <= model.max_seq_length, "prompt + new tokens exceed the cache"
+    logits = session.feed(prompt, [T - 1])
+    first = int(torch.argmax(logits[0]))
     step = DecodeStep(model, max_new_tokens)
     step.start(first, T)
     if use_graph:
@@ -182,6 +226,8 @@ def generate(model: Transformer, prompt: torch.Tensor, max_new_tokens: int, use_
     step.run(max_new_tokens - 1)
     torch.cuda.synchronize()
     dt = time.perf_counter() - t0
+    model.state.advance(T, max_new_tokens - 1)
+    session.close()
     seq = torch.cat((prompt.view(-1), torch.tensor([first], device=dev), step.seq[:max_new_tokens - 1]))
     return seq, dt
 
@@ -201,9 +247,26 @@ def build_model(name: str, algo: str, bitwidth: int, group_size: int = 128, dtyp
     return model.eval()
 
 
+def generate_from_checkpoint(args) -> None:
+    """Greedy generation with the model of a checkpoint folder; one JSON line with the tokens and the rates."""
+    model = registry.load_model(args.model, getattr(torch, args.dtype))
+    if args.prompt_tokens is not None:
+        prompt = torch.tensor([int(t) for t in args.prompt_tokens.split(",")])
+    else:
+        prompt = torch.randint(0, model.config.vocab_size, (args.prompt_len,), generator=torch.Generator().manual_seed(3))
+    seq, dt = generate(model, prompt.cuda(), args.max_new_tokens, not args.no_graph, max(args.max_seq_length, prompt.numel() + args.max_new_tokens))
+    n = args.max_new_tokens - 1
+    print(json.dumps({"metric": "tokens/s, batch-1 greedy decode", "model": model.config.model_name, "n_layer": model.config.n_layer,
+                      "dtype": args.dtype, "prompt_len": prompt.numel(), "new_tokens": args.max_new_tokens, "graph": not args.no_graph,
+                      "tokens_per_s": round(n / dt, 2) if n else None, "tokens": seq[prompt.numel():].tolist()}), flush=True)
+
+
 def main(argv=None):
     ap = argparse.ArgumentParser(description=__doc__.split("\n")[0])
-    ap.add_argument("--model", default="Meta-Llama-3-8B-Instruct")
+    ap.add_argument("--model", default="Meta-Llama-3-8B-Instruct",
+                    help="a named model with random quantised weights, or the folder of a checkpoint (config.json, model.safetensors)")
+    ap.add_argument("--dtype", choices=["bfloat16", "float32"], default="bfloat16", help="storage type of a checkpoint's weights and activations")
+    ap.add_argument("--prompt-tokens", default=None, help="token ids of the prompt, with commas (a checkpoint; random by default)")
     ap.add_argument("--algo", choices=sorted(LINEAR_CLASSES), default="sqllm")
     ap.add_argument("--bitwidth", type=int, default=4)
     ap.add_argument("--group-size", type=int, default=128)
@@ -219,6 +282,8 @@ def main(argv=None):
     ap.add_argument("--option", action="append", default=[], metavar="NAME=VALUE",
                     help="library option (decdec_set_option), e.g. fusion=0; may be repeated")
     args = ap.parse_args(argv)
+    if registry.is_checkpoint(args.model):
+        return generate_from_checkpoint(args)
     for kv in args.option:
         name, _, value = kv.partition("=")
         _lib.set_option(name, int(value))

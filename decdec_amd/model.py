@@ -12,12 +12,15 @@ helper kernels
 """
 from __future__ import annotations
 
+import math
 from dataclasses import dataclass
 from typing import Optional
 
 import torch
 import torch.nn as nn
 import torch.nn.functional as F
+
+from .cache import KVCache, SequenceState
 
 
 def find_multiple(n: int, k: int) -> int:
@@ -80,13 +83,36 @@ class RMSNorm(nn.Module):
         return F.rms_norm(x, (x.shape[-1],), self.weight, self.eps)
 
 
-def rope_tables(head_dim: int, max_pos: int, base: float, device=None):
-    """cos / sin [max_pos, head_dim] in fp32 for the half-rotation form: pair (i, i + head_dim/2) is
-    rotated by pos * base^(-2i/head_dim)."""
-    inv_freq = 1.0 / (base ** (torch.arange(0, head_dim, 2, dtype=torch.float32, device=device) / head_dim))
-    ang = torch.arange(max_pos, dtype=torch.float32, device=device)[:, None] * inv_freq[None, :]
-    ang = torch.cat((ang, ang), dim=-1)
-    return ang.cos(), ang.sin()
+def rope_frequencies(dims: int, base: float, scaling: Optional[dict] = None):
+    """(pair frequencies [dims / 2] in fp64, magnitude of cos and sin).  `scaling` (factor, original, fast, slow) is YaRN's:
+    pairs that turn fewer than `slow` times over `original` positions are slowed down by `factor`, pairs that turn more
+    than `fast` times are left alone, with a linear ramp over the pair index in between."""
+    inv = base ** (-torch.arange(0, dims, 2, dtype=torch.float64) / dims)
+    if not scaling:
+        return inv, 1.0
+    turns_to_dim = lambda t: dims * math.log(scaling["original"] / (2 * math.pi * t)) / (2 * math.log(base))
+    lo = max(math.floor(turns_to_dim(scaling["fast"])), 0)
+    hi = min(math.ceil(turns_to_dim(scaling["slow"])), dims - 1)
+    ramp = ((torch.arange(dims // 2, dtype=torch.float64) - lo) / max(hi - lo, 0.001)).clamp(0, 1)
+    return inv / scaling["factor"] * ramp + inv * (1 - ramp), 0.1 * math.log(scaling["factor"]) + 1.0
+
+
+def rope_tables(head_dim: int, max_pos: int, base: float, device=None, layout: str = "half", dims: Optional[int] = None,
+                scaling: Optional[dict] = None):
+    """cos / sin in fp32.  layout "half": [max_pos, head_dim] for the half-rotation form, pair (i, i + head_dim/2) is
+    rotated by pos * base^(-2i/head_dim).  layout "pairs": [max_pos, head_dim / 2], pair (2i, 2i + 1); the first `dims`
+    elements (all by default) turn, the rest keep their values; `scaling` as in rope_frequencies."""
+    if layout == "half":
+        inv_freq = 1.0 / (base ** (torch.arange(0, head_dim, 2, dtype=torch.float32, device=device) / head_dim))
+        ang = torch.arange(max_pos, dtype=torch.float32, device=device)[:, None] * inv_freq[None, :]
+        ang = torch.cat((ang, ang), dim=-1)
+        return ang.cos(), ang.sin()
+    dims = head_dim if dims is None else dims
+    freq, mag = rope_frequencies(dims, base, scaling)
+    ang = torch.arange(max_pos, dtype=torch.float64)[:, None] * freq[None, :]
+    cos, sin = torch.ones(max_pos, head_dim // 2), torch.zeros(max_pos, head_dim // 2)
+    cos[:, :dims // 2], sin[:, :dims // 2] = (ang.cos() * mag).float(), (ang.sin() * mag).float()
+    return cos.to(device), sin.to(device)
 
 
 def apply_rope(x: torch.Tensor, cos: torch.Tensor, sin: torch.Tensor) -> torch.Tensor:
@@ -94,19 +120,6 @@ def apply_rope(x: torch.Tensor, cos: torch.Tensor, sin: torch.Tensor) -> torch.T
     half = x.shape[-1] // 2
     rot = torch.cat((-x[..., half:], x[..., :half]), dim=-1)
     return x * cos + rot * sin
-
-
-class KVCache(nn.Module):
-    def __init__(self, max_batch_size: int, max_seq_length: int, n_heads: int, head_dim: int, dtype, device):
-        super().__init__()
-        shape = (max_batch_size, n_heads, max_seq_length, head_dim)
-        self.register_buffer("k_cache", torch.zeros(shape, dtype=dtype, device=device), persistent=False)
-        self.register_buffer("v_cache", torch.zeros(shape, dtype=dtype, device=device), persistent=False)
-
-    def update(self, input_pos: torch.Tensor, k: torch.Tensor, v: torch.Tensor):
-        self.k_cache.index_copy_(2, input_pos, k)
-        self.v_cache.index_copy_(2, input_pos, v)
-        return self.k_cache, self.v_cache
 
 
 class Attention(nn.Module):
@@ -232,6 +245,7 @@ class Transformer(nn.Module):
         for b in self.layers:
             b.attention.kv_cache = KVCache(max_batch_size, max_seq_length, self.config.n_local_heads,
                                            self.config.head_dim, self.dtype, dev)
+        self.state = SequenceState([b.attention.kv_cache for b in self.layers], max_seq_length)
         self.causal_mask = torch.tril(torch.ones(max_seq_length, max_seq_length, dtype=torch.bool, device=dev))
         cos, sin = rope_tables(self.config.head_dim, max_seq_length, self.config.rope_base, dev)
         self.rope_cos, self.rope_sin = cos.to(self.dtype), sin.to(self.dtype)
@@ -257,8 +271,9 @@ class Transformer(nn.Module):
             l.external_zero = True
             off += find_multiple(l.out_features, 64)
 
-    def forward(self, idx: torch.Tensor, input_pos: torch.Tensor) -> torch.Tensor:
-        """idx [B, S] token ids, input_pos [S] positions (int64); returns logits [B, S, vocab]."""
+    def forward(self, idx: torch.Tensor, input_pos: torch.Tensor, start: Optional[int] = None, want=None) -> torch.Tensor:
+        """idx [B, S] token ids, input_pos [S] positions (int64); returns logits [B, S, vocab], or [B, len(want), vocab]
+        for the places `want` among the S tokens.  `start` (the first position) is not needed here."""
         assert self.max_seq_length > 0, "Caches must be initialized first"
         assert idx.shape[1] <= self.max_seq_length and input_pos.numel() == idx.shape[1], \
             f"{idx.shape[1]} positions do not fit a cache of {self.max_seq_length} (input_pos must hold one position per token)"
@@ -283,6 +298,8 @@ class Transformer(nn.Module):
         cos, sin = self.rope_cos.index_select(0, input_pos), self.rope_sin.index_select(0, input_pos)
         for layer in self.layers:
             x = layer(x, mask, cos, sin, input_pos)
+        if want is not None:
+            x = x[:, want]
         return self.output(self.norm(x))
 
     # ---- DEC plumbing (reference end-to-end/model.py:143-215) ----

@@ -1,0 +1,45 @@
+"""Models by name and checkpoints by architecture.
+
+A checkpoint is a folder with ``config.json`` (whose "architecture" names the design) and ``model.safetensors``."""
+from __future__ import annotations
+
+import json
+import os
+
+import torch
+
+from .hybrid import HybridDecoder
+from .model import Transformer, transformer_configs
+
+# architectures a checkpoint's config.json may name
+ARCHITECTURES = {"Fivitar": HybridDecoder}
+
+
+def model_class(config: dict):
+    name = config.get("architecture")
+    if name not in ARCHITECTURES:
+        raise KeyError(f"Unknown architecture: {name}, available: {sorted(ARCHITECTURES)}")
+    return ARCHITECTURES[name]
+
+
+def is_checkpoint(path: str) -> bool:
+    return os.path.isfile(os.path.join(path, "config.json"))
+
+
+def read_config(path: str) -> dict:
+    with open(os.path.join(path, "config.json")) as f:
+        return json.load(f)
+
+
+def load_model(path: str, dtype=torch.bfloat16, device="cuda"):
+    """The model of a checkpoint folder, ready for setup_caches."""
+    from safetensors.torch import load_file
+    cfg = read_config(path)
+    model = model_class(cfg).from_config(cfg, dtype, device=device)
+    model.load_weights(load_file(os.path.join(path, "model.safetensors")))
+    return model.eval()
+
+
+def available() -> dict:
+    """Every model the command line knows by name, and the checkpoint architectures."""
+    return {"named": sorted(transformer_configs), "architectures": sorted(ARCHITECTURES), "named_class": Transformer}
