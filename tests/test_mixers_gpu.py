@@ -1,0 +1,267 @@
+"""Mixer kernels against the plain oracle, each mechanism alone: in one portion, in portions of several sizes and token by
+token, in float32 (tight) and bfloat16."""
+import pytest
+import torch
+
+from decdec_amd import mixer_ops as M, mixers as X
+from oracle import hybrid_oracle as O
+import hybrid_cases as cases
+
+pytestmark = pytest.mark.gpu
+DTYPES = [torch.float32, torch.bfloat16]
+TOL = {torch.float32: 2e-5, torch.bfloat16: 2.5e-2}
+
+
+def _close(got, want, dtype, what="", factor=1.0):
+    got, want = got.detach().double().cpu(), want.double().cpu()
+    assert torch.isfinite(got).all(), what
+    err = float((got - want).abs().max() / (want.abs().max() + 1e-9))
+    assert err <= TOL[dtype] * factor, (what, err)
+
+
+def _rand(*shape, seed=0, scale=1.0):
+    return torch.randn(*shape, generator=torch.Generator().manual_seed(seed)) * scale
+
+
+# ---- rows --------------------------------------------------------------------------------------------------
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("N,K,act", [(5, 3, 2), (64, 84, 0), (301, 200, 100), (4100, 96, 4100), (16400, 264, 8), (40, 2056, 1), (7, 1025, 3)])
+def test_gemv_with_an_activation_on_its_first_rows(N, K, act, dtype):
+    w, x, a = _rand(N, K, seed=N).to(dtype), _rand(K, seed=1).to(dtype), torch.tensor([0.7, -0.4]).to(dtype)
+    out = torch.full((N,), 9.0, dtype=dtype, device="cuda")
+    M.gemv(w.cuda(), x.cuda(), out, a.cuda() if act else None, act)
+    y = w.double() @ x.double()
+    y[:act] = O.xielu(y[:act], a[0].double(), a[1].double())
+    _close(out, y, dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("rows,dim,gate,final", [(1, 84, True, True), (3, 84, True, False), (2, 33, True, True), (4, 4096, False, True),
+                                                 (2, 7000, True, True), (1, 16384, True, False), (2, 20000, True, True)])
+def test_gated_residual(rows, dim, gate, final, dtype):
+    eps = 1e-3
+    x, y = _rand(rows, dim, seed=1, scale=3.0), _rand(rows, dim, seed=2, scale=0.05).to(dtype)
+    g, b, w, fw = _rand(rows, dim + 12, seed=3).to(dtype), _rand(dim, seed=4).to(dtype), _rand(dim, seed=5).to(dtype), _rand(dim, seed=6).to(dtype)
+    xd, gd = x.cuda(), g.cuda()
+    xe, fo = (torch.empty(rows, dim, dtype=dtype, device="cuda") for _ in range(2))
+    M.gated_residual(xd, y.cuda(), gd[:, 8:] if gate else None, dim + 12, b.cuda() if gate else None, w.cuda(), xe, eps,
+                     fw.cuda() if final else None, fo if final else None)
+    y = y.double() * (O.sigmoid(g[:, 8:8 + dim].double() + b.double()) if gate else 1.0)
+    want = x.double() + O.rms_norm(y, w.double(), eps)
+    _close(xd, want, torch.float32)                     # the residual stream is float32 whatever the storage type
+    _close(xe, want, dtype)
+    if final:
+        _close(fo, O.rms_norm(want, fw.double(), eps), dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_embed_norm_and_activation_rows(dtype):
+    table = _rand(50, 21, seed=1).to(dtype).cuda()
+    toks = torch.tensor([3, 49, 0, 3], device="cuda")
+    x, xe = torch.empty(4, 21, device="cuda"), torch.empty(4, 21, dtype=dtype, device="cuda")
+    M.embed(table, toks, x, xe)
+    assert torch.equal(x, table[toks].float()) and torch.equal(xe, table[toks])
+    M.embed(table, torch.tensor([50, -1, 2, 1], device="cuda"), x, None)          # ids outside the table read row 0
+    assert torch.equal(x[:2], table[[0, 0]].float())
+    for rows, dim in ((3, 21), (2, 5000)):
+        v, w = _rand(rows, dim, seed=2).cuda(), _rand(dim, seed=3).to(dtype).cuda()
+        out = torch.empty(rows, dim, dtype=dtype, device="cuda")
+        M.rmsnorm(v, w, out, 0.1)
+        _close(out, O.rms_norm(v.double(), w.double(), 0.1), dtype)
+    for n, ld in ((52, 60), (7, 9), (5000, 5008)):
+        inp, a = _rand(3, ld, seed=4, scale=2.0).to(dtype).cuda(), torch.tensor([-0.3, 1.2]).to(dtype).cuda()
+        out = torch.empty(3, n, dtype=dtype, device="cuda")
+        M.xielu(inp, n, a, out)
+        _close(out, O.xielu(inp[:, :n].double(), a[0].double(), a[1].double()), dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("groups,n,kind", [(1, 140, M.GATE_SIGMOID), (3, 36, M.GATE_SILU), (2, 2048, M.GATE_SILU)])
+def test_group_norm_gate(groups, n, kind, dtype):
+    o, g, w = _rand(3, groups * n, seed=1).cuda(), _rand(3, groups * n + 5, seed=2).to(dtype).cuda(), _rand(n, seed=3).to(dtype).cuda()
+    out = torch.empty(3, groups * n, dtype=dtype, device="cuda")
+    M.group_norm_gate(o, g[:, 2:], groups * n + 5, w, out, groups, 0.01, kind)
+    z = g[:, 2:2 + groups * n].double()
+    want = O.rms_norm(o.double().view(3, groups, n), w.double(), 0.01).view(3, -1) * (O.silu(z) if kind == M.GATE_SILU else O.sigmoid(z))
+    _close(out, want, dtype)
+
+
+# ---- mixers ------------------------------------------------------------------------------------------------
+class Bench:
+    """A mixer on the GPU with random weights, and the oracle's read-out (before the output projection)."""
+
+    def __init__(self, kind, m, dtype, T, seed=0, width=40, eps=1e-5, edit=None, max_seq=None):
+        g = torch.Generator().manual_seed(seed)
+        self.w = {n: cases.random_tensor("mix." + n, s, g) for n, s in cases.mixer_shapes(kind, m, width).items()}
+        self.w["o"] = torch.eye(self.w["o"].shape[1]).to(torch.bfloat16)          # the oracle's output is the read-out itself
+        self.h = torch.randn(T, width, generator=g).to(torch.bfloat16)
+        self.m, self.kind, self.eps, self.dtype, self.T = m, kind, eps, dtype, T
+        if edit:
+            edit(self)
+        self.mixer = X.MIXER_TYPES[kind](m, X.Workspace(torch.device("cuda")))
+        names, off = [n for n, _ in self.mixer.inputs], {}
+        for n, r in self.mixer.inputs:
+            off[n] = sum(off_r for _, off_r in self.mixer.inputs[:names.index(n)])
+        rows = sum(r for _, r in self.mixer.inputs)
+        # projections in float64, rounded once to the storage type; the oracle sees the unrounded ones
+        proj = torch.cat([self.h.double() @ self.w[n].double().T for n in names], 1)
+        self.proj = torch.zeros(T, (rows + 7) // 8 * 8, dtype=dtype)
+        self.proj[:, :rows] = proj.to(dtype)
+        self.proj = self.proj.cuda()
+        self.mixer.bind({n: t.to(dtype).cuda() for n, t in self.w.items() if n not in names and n != "o"}, off, eps)
+        self.max_seq = max_seq or T
+        self.new_state()
+
+    def new_state(self):
+        self.state = self.mixer.new_state(self.max_seq, self.dtype, "cuda")
+
+    def want(self):
+        return O.MIXERS[self.kind](self.h.double(), {n: t.double() for n, t in self.w.items()}, self.m, self.eps)
+
+    def run(self, portions, t=0):
+        out = []
+        for n in portions:
+            y = torch.empty(n, self.mixer.width, dtype=self.dtype, device="cuda")
+            self.mixer(self.proj[t:t + n].contiguous(), self.state, torch.tensor([t], device="cuda"), t, y)
+            out.append(y)
+            t += n
+        return torch.cat(out)
+
+
+def _portions(T, *sizes):
+    out, i = [], 0
+    while sum(out) < T:
+        out.append(min(sizes[i % len(sizes)], T - sum(out)))
+        i += 1
+    return out
+
+
+RECURRENCES = [("lightning", cases.lightning(3, 32, 32)), ("lightning", cases.lightning(5, 12, 28, [0.0, 0.3, 0.95, 0.9999, 1.0])),
+               ("lightning", cases.lightning(2, 128, 128)), ("lightning", cases.lightning(1, 200, 72, [0.98])), ("lightning", cases.lightning(2, 1, 1)),
+               ("delta", cases.delta(2, 1, 32, 64, 4)), ("delta", cases.delta(3, 3, 20, 36, 3)), ("delta", cases.delta(4, 2, 128, 128, 4)),
+               ("delta", cases.delta(2, 2, 64, 16, 1)), ("delta", cases.delta(6, 2, 9, 130, 2)), ("delta", cases.delta(1, 1, 256, 256, 7)),
+               ("delta", cases.delta(2, 1, 16, 300, 5))]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("kind,m", RECURRENCES)
+def test_recurrence_in_portions_and_token_by_token(kind, m, dtype):
+    T = 150
+    b = Bench(kind, m, dtype, T)
+    want = b.want()
+    for sizes in ((T,), (2,), (3, 64, 1, 2), (65, 63, 5), (1,), (130, 1)):
+        # the state of the sequence before is left in place: position 0 starts afresh
+        _close(b.run(_portions(T, *sizes)), want, dtype, (kind, m, sizes), factor=4.0)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_delta_rule_with_decays_that_forget_at_once_and_never(dtype):
+    def edit(b):
+        b.w["A_log"] = torch.tensor([5.0, -12.0, 2.0]).to(torch.bfloat16)
+        b.w["dt_bias"] = torch.tensor([4.0, -6.0, 1.0]).to(torch.bfloat16)
+    b = Bench("delta", cases.delta(3, 1, 24, 24, 4), dtype, 140, edit=edit)
+    for sizes in ((140,), (37,), (1,)):
+        _close(b.run(_portions(140, *sizes)), b.want(), dtype, sizes, factor=4.0)
+
+
+def test_convolution_sees_exactly_its_taps_across_a_cut():
+    """One token's input is changed: the read-outs of a head without memory differ for `taps` tokens from there on, no
+    more and no fewer, wherever the portions are cut."""
+    taps, T = 4, 40
+
+    def edit(b):                                           # a decay of e^-150: nothing but the convolution reaches back
+        b.w["A_log"], b.w["dt_bias"] = torch.tensor([5.0]).to(torch.bfloat16), torch.tensor([4.0]).to(torch.bfloat16)
+        b.w["a"] = torch.zeros_like(b.w["a"])
+    b = Bench("delta", cases.delta(1, 1, 16, 16, taps), torch.float32, T, edit=edit)
+    for sizes in ((T,), (1,), (2,), (7, 1)):
+        base = b.run(_portions(T, *sizes))
+        keep = b.proj.clone()
+        for at in (0, 6, 7, 13):
+            b.proj[at, :48] += 1.0                         # q, k and v of one token
+            moved = (b.run(_portions(T, *sizes)) - base).abs().amax(1) > 1e-4
+            assert moved.nonzero().view(-1).tolist() == list(range(at, at + taps)), (sizes, at)
+            b.proj.copy_(keep)
+
+
+LATENTS = [cases.latent(4, 64, 32, 64, 64, scaling=cases.YARN), cases.latent(3, 22, 10, 18, 30, base=500.0), cases.latent(17, 16, 8, 24, 48, scale=0.4),
+           cases.latent(2, 128, 64, 128, 512, base=10000.0), cases.latent(1, 200, 56, 200, 96), cases.latent(2, 32, 16, 40, 72, dims=8),
+           cases.latent(1, 2, 2, 1, 1), cases.latent(2, 96, 64, 256, 136)]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("m", LATENTS)
+def test_latent_attention_in_portions_and_token_by_token(m, dtype):
+    T = 150
+    b = Bench("latent_attention", m, dtype, T)
+    want = b.want()
+    for sizes in ((T,), (2,), (3, 64, 1, 2), (65, 63, 5), (1,), (130, 1)):
+        _close(b.run(_portions(T, *sizes)), want, dtype, (m, sizes), factor=2.0)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("max_seq", [700, 8000])
+def test_latent_attention_finds_one_key_at_every_tile_edge(dtype, max_seq):
+    """A query is made to point at one key: its read-out is that token's value, wherever the key lies relative to the tiles
+    of 64 keys and to the shares of the one-token kernel's workgroups."""
+    T, m = 700, cases.latent(2, 32, 8, 32, 48, base=1e6, scale=1.0)
+    b = Bench("latent_attention", m, dtype, T, max_seq=max_seq)
+    H, D, R, V, C = 2, 32, 8, 32, 48
+    c = O.rms_norm(b.proj[:, 80:80 + C].double().cpu(), b.w["dkv.norm"].double(), b.eps)
+    kn = (c @ b.w["uk"].double().T).view(T, H, D)
+    v = (c @ b.w["uv"].double().T).view(T, H * V)
+    b.run([T - 1])
+    tried = 0
+    for key in (0, 1, 62, 63, 64, 65, 127, 128, 319, 320, 511, 512, 575, 576, 640, 697, 698):
+        q = torch.zeros(H, D + R, dtype=torch.float64)
+        for h in range(H):
+            others = torch.cat((kn[:key, h], kn[key + 1:, h]))
+            q[h, :D] = kn[key, h] * 60.0 / float(kn[key, h] @ kn[key, h] - (others @ kn[key, h]).max()).__abs__()
+        b.proj[T - 1, :80] = q.view(-1).to(dtype)
+        scores = torch.stack([kn[:, h] @ b.proj[T - 1].double().cpu()[:80].view(H, D + R)[h, :D] for h in range(H)])
+        if (scores.argmax(1) != key).any():
+            continue                                       # a longer key in the same direction wins
+        tried += 1
+        one = b.run([1], T - 1)
+        for name, got in (("one token", one[0]), ("portion", b.run([3], T - 3)[2])):
+            e = torch.exp(scores - scores.amax(1, keepdim=True))
+            want = torch.cat([(e[h] / (e[h].sum() + torch.exp(b.w["sink"][h].double() - scores[h].max()))) @ v.view(T, H, V)[:, h] for h in range(H)])
+            _close(got, want, dtype, (name, key), factor=3.0)
+    assert tried >= 14
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("sink", [-30.0, 0.0, 12.0])
+def test_sink_counts_once_whatever_the_number_of_workgroups(sink, dtype):
+    def edit(b):
+        b.w["sink"] = torch.tensor([sink, sink / 2]).to(torch.bfloat16)
+    b = Bench("latent_attention", cases.latent(2, 16, 8, 16, 24), dtype, 520, edit=edit)
+    want = b.want()
+    _close(b.run([520]), want, dtype, factor=2.0)
+    _close(b.run([1] * 5), want[:5], dtype, factor=2.0)                 # the first tokens
+    b.run([515])
+    _close(b.run([1] * 5, 515), want[515:], dtype, factor=2.0)
+
+
+def test_no_key_after_the_query_and_every_key_up_to_it():
+    """The last visible key is the query's own: changing a later token's input changes nothing, changing its own does."""
+    T = 140
+    b = Bench("latent_attention", cases.latent(2, 16, 8, 16, 24), torch.float32, T)
+    base = b.run([T])
+    for at in (0, 1, 63, 64, 127, 128, 139):
+        keep = b.proj.clone()
+        b.proj[at, 48:48 + 32] += 2.0                                    # latent and rotated key of one token
+        for sizes in ((T,), (70,), (1,)):
+            diff = (b.run(_portions(T, *sizes)) - base).abs().amax(1)
+            assert float(diff[:at].max() if at else 0.0) < 1e-5 and float(diff[at]) > 1e-4, (at, sizes)
+        b.proj.copy_(keep)
+
+
+def test_a_cache_of_a_longer_sequence_before_is_not_seen():
+    m = cases.latent(2, 16, 8, 16, 24)
+    b = Bench("latent_attention", m, torch.float32, 300)
+    b.run([300])
+    short = Bench("latent_attention", m, torch.float32, 70, seed=9, max_seq=300)
+    short.state = b.state                                                # full of the other sequence's rows
+    want = short.want()
+    _close(short.run([69]), want[:69], torch.float32)
+    _close(short.run([1], 69), want[69:], torch.float32)
