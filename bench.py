@@ -516,6 +516,71 @@ def helpers_leg(torch):
     return out
 
 
+# ---- the Fivitar decoder beside the plain decoder ------------------------------------------------------------
+HYBRID_SIZES = {"2048": dict(width=2048, heads=16, kv_heads=8, ff=7168), "4096": dict(width=4096, heads=32, kv_heads=8, ff=14336)}
+
+
+def hybrid_config(kind, width, heads, ff, layers, vocab, kv_heads=None):
+    mixers = {"lightning": {"heads": heads, "dim": 128, "vdim": 128, "decay": [1.0 - 2.0 ** (-2 - 6 * i / heads) for i in range(heads)]},
+              "delta": {"heads": heads, "kv_heads": heads // 2, "dim": 128, "vdim": 128, "conv": 4},
+              "latent_attention": {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5,
+                                   "rot": {"base": 10000.0, "dims": 64, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
+    kinds = list(mixers) if kind == "mixed" else [kind]
+    return {"architecture": "Fivitar", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+            "layers": [{"type": kinds[i % len(kinds)], "mixer": mixers[kinds[i % len(kinds)]], "mlp": {"kind": "dense", "ff": ff}}
+                       for i in range(layers)]}
+
+
+def hybrid_leg(torch, sizes, layers=6, prompts=(512, 2048, 8192), positions=(512, 2048, 8192), vocab=32000):
+    """Prefill and decode of `layers` layers (random bf16 weights, dense) per size: the Fivitar decoder with its three
+    mixers in turn and with each alone, and the plain decoder (grouped-query attention, SwiGLU) of the same width, head
+    count and feed-forward size with dense bf16 linears."""
+    from decdec_amd.generate import DecodeStep, Session
+    from decdec_amd.hybrid import HybridDecoder
+    from decdec_amd.model import ModelArgs, Transformer
+
+    def plain(width, heads, kv_heads, ff):
+        cfg = ModelArgs(block_size=1 << 20, vocab_size=vocab, n_layer=layers, n_head=heads, n_local_heads=kv_heads, dim=width, intermediate_size=ff)
+        return Transformer(torch.bfloat16, cfg, linear_class=torch.nn.Linear, linear_kwargs={"dtype": torch.bfloat16, "device": "cuda"}).eval()
+
+    rows = []
+    for size in sizes:
+        z = HYBRID_SIZES[size]
+        for kind in ("plain", "mixed", "lightning", "delta", "latent_attention"):
+            if kind == "plain":
+                m = plain(**z)
+            else:
+                m = HybridDecoder.from_config(hybrid_config(kind, layers=layers, vocab=vocab, **z), torch.bfloat16)
+                m.init_random_weights(0)
+            row = {"size": size, "model": kind, "layers": layers, "parameters": sum(t.numel() for t in list(m.parameters()) + list(m.buffers()))}
+            gen = torch.Generator().manual_seed(0)
+            toks = torch.randint(0, vocab, (max(prompts + positions) + 1,), generator=gen).cuda()
+            for n in prompts:
+                best = None
+                for _ in range(4):
+                    s = Session(m, max(positions) + 256, portion=8192)
+                    torch.cuda.synchronize()
+                    t0 = time.perf_counter()
+                    s.feed(toks[:n], [n - 1])
+                    torch.cuda.synchronize()
+                    dt = time.perf_counter() - t0
+                    best = dt if best is None else min(best, dt)
+                row[f"prefill_{n}_tokens_per_s"] = round(n / best, 0)
+            for n in positions:
+                s = Session(m, max(positions) + 256, portion=8192)
+                s.feed(toks[:n])
+                step = DecodeStep(m, 256)
+                step.start(1, n)
+                step.capture()
+                row[f"decode_at_{n}_us_per_token"] = round(time_graph(torch, step.graph, 100, 20, 0.0), 1)
+                del step
+            rows.append(row)
+            print(json.dumps(row), file=sys.stderr, flush=True)
+            del m
+            torch.cuda.empty_cache()
+    return rows
+
+
 def cpu_baseline_leg(protos, iters=20, budget_s=25.0):
     """The same per-layer path (select + residual rows + any-precision GEMV) in the C oracle on the host cores: one
     layer of each shape, median of `iters` warmed calls, scaled to a token (32 layers); with all cores and with
@@ -575,13 +640,15 @@ def main():
     ap.add_argument("--n-tb", type=int, default=32, help="workgroups DEC may occupy (the sweep shows 8..64)")
     ap.add_argument("--sweep", action="store_true", help="also sweep k_chunk x n_tb (slower)")
     ap.add_argument("--no-cpu-baseline", action="store_true")
-    ap.add_argument("--leg", choices=["all", "token", "roofline", "kernels", "helpers", "link", "trace"], default="all",
+    ap.add_argument("--leg", choices=["all", "token", "roofline", "kernels", "helpers", "link", "trace", "fivitar"], default="all",
                     help="token: only the token (batched, one launch per layer, graph branches; with DEC and base-only); "
                          "roofline: only the roofline kernel's launches and a 256 MiB device copy (short run for counter "
                          "collection); kernels: per-kernel table over the configuration shapes (k_chunk 32, n_tb 32); "
                          "helpers: the decode harness's helper kernels (output head, attention, norm, activation); "
                          "link: zero-copy reads of pinned host memory over workgroup counts and request widths; "
-                         "trace: phase timings of DEC-only launches from the role's own cycle stamps")
+                         "trace: phase timings of DEC-only launches from the role's own cycle stamps; "
+                         "fivitar: prefill and decode of the Fivitar decoder beside the plain decoder of the same size")
+    ap.add_argument("--size", nargs="+", choices=sorted(HYBRID_SIZES), default=sorted(HYBRID_SIZES), help="widths of --leg fivitar")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this path runs on one GPU; --gpus N with N > 1 is not part of this build", file=sys.stderr)
@@ -595,6 +662,9 @@ def main():
 
     if args.leg == "helpers":
         print(json.dumps({"helpers": helpers_leg(torch)}))
+        return
+    if args.leg == "fivitar":
+        print(json.dumps({"fivitar": hybrid_leg(torch, args.size)}))
         return
     if args.leg == "link":
         print(json.dumps({"link": link_leg(torch, full=True)}))
