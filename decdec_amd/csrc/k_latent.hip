@@ -93,17 +93,19 @@ hipError_t launch_latent_append(int dt, const decdec_latent& p, void* q_out, uin
 }
 
 // ---- many tokens ------------------------------------------------------------------------------------------
-// grid (query blocks, heads), four waves of 16 MT queries.  The transposed scores (keys x queries) leave a query in one
+// Workgroups of four waves with 16 MT queries each, one per query block and head; the heads are dealt to the eight dies,
+// so that the tiles of a head's keys and values are shared in one L2.  The transposed scores (keys x queries) leave a query in one
 // lane column: its running maximum and sum are lane values, its weights are at once the right operand of the value
 // product (out^T = V^T P^T), and nothing passes through LDS but the key and value tiles.  The contraction of that product
-// visits keys 4 (lane / 16) + e of one 16-key tile, then of the next, in both operands.
+// visits keys 4 (lane / 16) + e of one 16-key tile, then of the next, in both operands.  The next tile is requested into
+// registers while the present one is worked on.  Scores are kept in units of log 2.
 constexpr uint32_t kKeys = 64;
 
-template <int DT, int MT, int NK, int NV>
-__global__ __launch_bounds__(256) void latent_attention_kernel(const decdec_latent p, const void* __restrict__ q_in,
+template <int DT, int MT, int NK, int NV, bool VEC>
+__global__ __launch_bounds__(256, DT == kFP32 ? 1 : 2) void latent_attention_kernel(const decdec_latent p, const void* __restrict__ q_in,
                                                                const void* __restrict__ k_in, const void* __restrict__ vt_in,
                                                                const uint32_t vt_ld, void* __restrict__ out,
-                                                               const uint32_t start, const uint32_t rows, const uint32_t keys_total) {
+                                                               const uint32_t start, const uint32_t rows, const uint32_t blocks) {
     using T = typename LaneOf<DT>::t;
     using E = Elem<DT>;
     constexpr uint32_t PAD = DT == kFP32 ? 4u : 8u, KL = 32u * NK + PAD, VL = kKeys + PAD;
@@ -111,9 +113,10 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const decdec_late
     T* Kl = (T*)smem;                       // [kKeys][KL]
     T* Vl = Kl + kKeys * KL;                // [16 NV][VL]
     const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, l16 = lane & 15u, lg = lane >> 4;
-    const uint32_t h = blockIdx.y, Dq = p.dim + p.rot, D = p.dim, V = p.vdim;
-    const uint32_t q0 = (gridDim.x - 1u - blockIdx.x) * (64u * MT);        // longest rows first
-    const bool vec = D % 8u == 0 && p.rot % 8u == 0 && p.rank % 8u == 0 && (p.heads * D) % 8u == 0;
+    const uint32_t turn = blockIdx.x >> 3, h = (blockIdx.x & 7u) + 8u * (turn / blocks);
+    if (h >= p.heads) return;
+    const uint32_t q0 = (blocks - 1u - turn % blocks) * (64u * MT);        // longest rows first
+    const uint32_t Dq = p.dim + p.rot, D = p.dim, V = p.vdim, keys_total = start + rows;
     const T* q = (const T*)q_in;
     Frag<DT> qf[MT][NK];
     uint32_t qpos[MT];
@@ -123,9 +126,10 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const decdec_late
         qpos[m] = start + rc;
 #pragma unroll
         for (int s = 0; s < NK; ++s)
-            qf[m][s] = load8<DT>(q + ((size_t)rc * p.heads + h) * Dq + 32u * s + 8u * lg, (int)Dq - (int)(32u * s + 8u * lg), vec);
+            qf[m][s] = load8<DT>(q + ((size_t)rc * p.heads + h) * Dq + 32u * s + 8u * lg, (int)Dq - (int)(32u * s + 8u * lg), VEC);
     }
-    const float sink = p.sink != nullptr ? E::load(p.sink, h) : -__builtin_inff();
+    const float scale2 = p.scale * kLog2e;
+    const float sink = p.sink != nullptr ? E::load(p.sink, h) * kLog2e : -__builtin_inff();
     float mx[MT], sum[MT];
     f32x4 o[MT][NV];
 #pragma unroll
@@ -136,35 +140,51 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const decdec_late
         for (int n = 0; n < NV; ++n) o[m][n] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
     const uint32_t last = q0 + 64u * MT < rows ? q0 + 64u * MT : rows;     // one past the block's last query
-    const uint32_t kend = start + last;
+    const uint32_t kend = start + last, wave_first = start + q0 + 16u * MT * wave, wave_last = wave_first + 16u * MT - 1u;
+    const size_t kld = (size_t)p.heads * D, cld = p.rank + p.rot;
     const T* kb = (const T*)k_in + (size_t)h * D;
     const T* cb = (const T*)p.cache + p.rank;
     const T* vb = (const T*)vt_in + (size_t)h * V * vt_ld;
+    // A key row is [unrotated part of the head | shared rotated part]; keys past the end repeat the last one and are never
+    // weighted, value rows past vdim repeat the first one and are never stored.  A thread loads eight elements of every
+    // slice of one key, and of every 32nd value row.
+    Frag<DT> kr[VEC ? NK : 1], vr[VEC ? NV / 2 : 1];
+    const uint32_t krow = tid >> 2, kcol = (tid & 3u) * 8u, vrow = tid >> 3, vcol = (tid & 7u) * 8u;
+    auto request = [&](uint32_t k0) {
+        const uint32_t key = k0 + krow < keys_total ? k0 + krow : keys_total - 1u;
+        const T* un = kb + key * kld + kcol;
+        const T* ro = cb + key * cld + kcol;
+#pragma unroll
+        for (int j = 0; j < NK; ++j) {
+            const uint32_t c = 32u * j + kcol;
+            kr[j] = frag_load(c < D ? un + 32u * j : (c < Dq ? ro + (32 * j - (int)D) : cb));
+            if (c >= Dq) kr[j] = Frag<DT>{};
+        }
+        const T* vp = vb + k0 + vcol;
+#pragma unroll
+        for (int j = 0; j < NV / 2; ++j) vr[j] = frag_load(vp + (size_t)(vrow + 32u * j < V ? vrow + 32u * j : 0u) * vt_ld);
+    };
+    if constexpr (VEC) request(0u);
     for (uint32_t k0 = 0; k0 < kend; k0 += kKeys) {
         __syncthreads();
-        for (uint32_t i = tid; i < kKeys * 4u * NK; i += 256u) {
-            const uint32_t r = i / (4u * NK), c = (i % (4u * NK)) * 8u, key = k0 + r;
-            const bool in = key < keys_total;
-            const T* rot = cb + (size_t)key * (p.rank + p.rot);
-            Frag<DT> f;
-            if (!in) f = load8<DT>(kb, 0, false);
-            else if (vec) f = c < D ? load8<DT>(kb + (size_t)key * p.heads * D + c, 8, true) : load8<DT>(rot + (c - D), (int)Dq - (int)c, true);
-            else if (c >= D) f = load8<DT>(rot + (c - D), (int)Dq - (int)c, false);
-            else if (c + 8u <= D) f = load8<DT>(kb + (size_t)key * p.heads * D + c, 8, false);
-            else {                                                         // the unrotated part ends inside
-                T t[8];
+        if constexpr (VEC) {
 #pragma unroll
-                for (uint32_t e = 0; e < 8u; ++e)
-                    t[e] = c + e < D ? kb[(size_t)key * p.heads * D + c + e] : (c + e < Dq ? rot[c + e - D] : (T)0);
-                f = load8<DT>(t, 8, false);
+            for (int j = 0; j < NK; ++j) store8(Kl + krow * KL + kcol + 32u * j, kr[j]);
+#pragma unroll
+            for (int j = 0; j < NV / 2; ++j) store8(Vl + (vrow + 32u * j) * VL + vcol, vr[j]);
+        } else {
+            for (uint32_t i = tid; i < kKeys * 32u * NK; i += 256u) {
+                const uint32_t r = i / (32u * NK), c = i % (32u * NK), key = k0 + r < keys_total ? k0 + r : keys_total - 1u;
+                Kl[r * KL + c] = c < D ? kb[key * kld + c] : (c < Dq ? cb[key * cld + c - D] : (T)0);
             }
-            store8(Kl + r * KL + c, f);
-        }
-        for (uint32_t i = tid; i < 16u * NV * (kKeys / 8u); i += 256u) {
-            const uint32_t d = i / (kKeys / 8u), c = (i % (kKeys / 8u)) * 8u;
-            store8(Vl + d * VL + c, load8<DT>(vb + (size_t)(d < V ? d : 0u) * vt_ld + k0 + c, d < V ? 8 : 0, true));
+            for (uint32_t i = tid; i < 16u * NV * kKeys; i += 256u) {
+                const uint32_t d = i / kKeys, c = i % kKeys;
+                Vl[d * VL + c] = d < V ? vb[(size_t)d * vt_ld + k0 + c] : (T)0;
+            }
         }
         __syncthreads();
+        if constexpr (VEC) { if (k0 + kKeys < kend) request(k0 + kKeys); }
+        if (k0 > wave_last) continue;                                      // every key of the tile lies after the wave's queries
         f32x4 sc[MT][4];
 #pragma unroll
         for (int m = 0; m < MT; ++m)
@@ -178,7 +198,7 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const decdec_late
 #pragma unroll
                 for (int m = 0; m < MT; ++m) mma(a, qf[m][s], sc[m][t]);
             }
-        const bool edge = k0 + kKeys > start + q0 + 16u * MT * wave + 1u;  // some key may lie after some query of the wave
+        const bool edge = k0 + kKeys > wave_first + 1u;                    // some key may lie after some query of the wave
         Frag<DT> hi[MT][2], lo[MT][2];
 #pragma unroll
         for (int m = 0; m < MT; ++m) {
@@ -187,24 +207,26 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const decdec_late
             for (int t = 0; t < 4; ++t)
 #pragma unroll
                 for (int v = 0; v < 4; ++v) {
-                    float x = sc[m][t][v] * p.scale;
+                    float x = sc[m][t][v] * scale2;
                     if (edge && k0 + 16u * t + 4u * lg + (uint32_t)v > qpos[m]) x = -__builtin_inff();
                     sc[m][t][v] = x;
                     best = fmaxf(best, x);
                 }
             best = fmaxf(best, __shfl_xor(best, 16, 64));
             best = fmaxf(best, __shfl_xor(best, 32, 64));
-            const float corr = __expf(mx[m] - best);                       // the first key is visible to every query: best is finite
-            mx[m] = best;
-            sum[m] *= corr;
+            if (__any(best > mx[m])) {
+                const float corr = __builtin_amdgcn_exp2f(mx[m] - best);   // the first key is visible to every query: best is finite
+                mx[m] = best;
+                sum[m] *= corr;
 #pragma unroll
-            for (int n = 0; n < NV; ++n) o[m][n] *= corr;
+                for (int n = 0; n < NV; ++n) o[m][n] *= corr;
+            }
 #pragma unroll
             for (int t = 0; t < 2; ++t) {
                 float w[8];
 #pragma unroll
                 for (int e = 0; e < 8; ++e) {
-                    w[e] = __expf(sc[m][2 * t + (e >> 2)][e & 3] - best);
+                    w[e] = __builtin_amdgcn_exp2f(sc[m][2 * t + (e >> 2)][e & 3] - best);
                     sum[m] += w[e];
                 }
                 frag_split(w, hi[m][t], lo[m][t]);
@@ -214,14 +236,14 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const decdec_late
         for (int n = 0; n < NV; ++n)
 #pragma unroll
             for (int t = 0; t < 2; ++t) {
-                const T* vr = Vl + (16u * n + l16) * VL + 32u * t + 4u * lg;
+                const T* vk = Vl + (16u * n + l16) * VL + 32u * t + 4u * lg;
                 Frag<DT> a;
                 if constexpr (DT == kFP32) {
-                    const f32x4 x = *(const f32x4*)vr, y = *(const f32x4*)(vr + 16);
+                    const f32x4 x = *(const f32x4*)vk, y = *(const f32x4*)(vk + 16);
 #pragma unroll
                     for (int e = 0; e < 4; ++e) { a.v[e] = x[e]; a.v[4 + e] = y[e]; }
                 } else {
-                    const u32x2 x = *(const u32x2*)vr, y = *(const u32x2*)(vr + 16);
+                    const u32x2 x = *(const u32x2*)vk, y = *(const u32x2*)(vk + 16);
                     a.v = u32x4{x[0], x[1], y[0], y[1]};
                 }
 #pragma unroll
@@ -250,15 +272,16 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(const decdec_late
     }
 }
 
-template <int DT, int MT, int NK, int NV>
+template <int DT, int MT, int NK, int NV, bool VEC = true>
 static hipError_t attention_launch(const decdec_latent& p, const void* q, const void* k, const void* vt, uint32_t vt_ld, void* out,
                                    uint32_t start, uint32_t rows, hipStream_t s) {
     constexpr uint32_t PAD = DT == kFP32 ? 4u : 8u;
     constexpr size_t lds = (size_t)(kKeys * (32u * NK + PAD) + 16u * NV * (kKeys + PAD)) * Elem<DT>::bytes;
     static_assert(lds <= 160u * 1024u, "tiles must fit the LDS of a compute unit");
-    if (hipError_t e = allow_lds<latent_attention_kernel<DT, MT, NK, NV>>(lds); e != hipSuccess) return e;
-    hipLaunchKernelGGL((latent_attention_kernel<DT, MT, NK, NV>), dim3((rows + 64u * MT - 1u) / (64u * MT), p.heads), dim3(256), lds, s,
-                       p, q, k, vt, vt_ld, out, start, rows, start + rows);
+    if (hipError_t e = allow_lds<latent_attention_kernel<DT, MT, NK, NV, VEC>>(lds); e != hipSuccess) return e;
+    const uint32_t blocks = (rows + 64u * MT - 1u) / (64u * MT);
+    hipLaunchKernelGGL((latent_attention_kernel<DT, MT, NK, NV, VEC>), dim3(blocks * ((p.heads + 7u) / 8u * 8u)), dim3(256), lds, s,
+                       p, q, k, vt, vt_ld, out, start, rows, blocks);
     return hipGetLastError();
 }
 
@@ -274,6 +297,7 @@ template <int DT, int MT>
 static hipError_t attention_dt(const decdec_latent& p, const void* q, const void* k, const void* vt, uint32_t vt_ld, void* out,
                                uint32_t start, uint32_t rows, hipStream_t s) {
     const uint32_t Dq = p.dim + p.rot;
+    if (p.dim % 8u != 0 || p.rot % 8u != 0 || p.rank % 8u != 0) return attention_launch<DT, 1, 10, 16, false>(p, q, k, vt, vt_ld, out, start, rows, s);
     if (Dq <= 128u) return attention_nv<DT, MT, 4>(p, q, k, vt, vt_ld, out, start, rows, s);
     if (Dq <= 192u) return attention_nv<DT, MT, 6>(p, q, k, vt, vt_ld, out, start, rows, s);
     return attention_nv<DT, 1, 10>(p, q, k, vt, vt_ld, out, start, rows, s);
@@ -348,17 +372,20 @@ static uint32_t step_max_splits(const decdec_latent& p) {
     return n < tiles ? n : tiles;
 }
 
-// grid (splits, heads / 16), four waves.  Scores transposed (keys x heads) as above, each wave 16 keys of the tile (and,
-// where the tile has fewer than four 16-key blocks, a share of the contraction); the tile stays in LDS for the weighted
-// sum over its keys, whose rows (latent components) are divided among the waves.
+// grid (splits, heads / 16), sixteen waves.  Scores transposed (keys x heads) as above: the 16-key blocks of the tile times
+// shares of the contraction make sixteen wave tasks, summed through LDS; a wave then takes one head's softmax, a lane per
+// key; the tile stays in LDS for the weighted sum over its keys, whose rows (latent components) are divided among the
+// waves.  The next tile is requested into registers while the present one is worked on.
+constexpr uint32_t kStepThreads = 1024;
+
 template <int DT, int KT, int NR>
-__global__ __launch_bounds__(256) void latent_step_kernel(const decdec_latent p, const float* __restrict__ qa, float* __restrict__ parts,
-                                                          const uint32_t max_splits) {
+__global__ __launch_bounds__(kStepThreads) void latent_step_kernel(const decdec_latent p, const float* __restrict__ qa,
+                                                                   float* __restrict__ parts, const uint32_t max_splits) {
     using T = typename LaneOf<DT>::t;
-    constexpr uint32_t KB = KT / 16, SP = 4u / KB;
+    constexpr uint32_t KB = KT / 16, SP = 16u / KB, NL = (KT * 80u + kStepThreads - 1u) / kStepThreads;   // rows of at most 640
     constexpr uint32_t PAD = DT == kFP32 ? 4u : 8u, QN = DT == kFP32 ? 1u : 2u;
     extern __shared__ __align__(16) unsigned char smem[];
-    const uint32_t R = p.rank, W = R + p.rot, Wp = (W + 31u) & ~31u, KL = Wp + PAD;
+    const uint32_t R = p.rank, W = R + p.rot, Wp = (W + 31u) & ~31u, KL = Wp + PAD, W8 = Wp / 8u;
     T* Kl = (T*)smem;                                    // [KT][KL]
     T* Ql = Kl + KT * KL;                                // [QN][16][KL]: leading and trailing parts
     __shared__ float Pl[SP][KT][17];
@@ -372,8 +399,24 @@ __global__ __launch_bounds__(256) void latent_step_kernel(const decdec_latent p,
     if (blockIdx.x >= sp.splits) return;
     const uint32_t lo_key = blockIdx.x * sp.span, hi_key = lo_key + sp.span < len ? lo_key + sp.span : len;
     const bool vec = R % 8u == 0 && p.rot % 8u == 0;
-    for (uint32_t i = tid; i < 16u * (Wp / 8u); i += 256u) {
-        const uint32_t r = i / (Wp / 8u), c = (i % (Wp / 8u)) * 8u;
+    Frag<DT> kr[NL];
+    // rows past the end repeat the last one; their weights are zero
+    auto request = [&](uint32_t k0) {
+#pragma unroll
+        for (uint32_t j = 0; j < NL; ++j) {
+            const uint32_t i = tid + kStepThreads * j, r = i / W8, c = (i - r * W8) * 8u, key = k0 + r < hi_key ? k0 + r : hi_key - 1u;
+            const T* row = (const T*)p.cache + (size_t)key * W;
+            if (vec) {
+                kr[j] = frag_load(row + (c < W ? c : 0u));
+                if (c >= W) kr[j] = Frag<DT>{};
+            } else {
+                kr[j] = load8<DT>(row + c, (int)W - (int)c, false);
+            }
+        }
+    };
+    request(lo_key);
+    for (uint32_t i = tid; i < 16u * W8; i += kStepThreads) {
+        const uint32_t r = i / W8, c = (i - r * W8) * 8u;
         float x[8];
 #pragma unroll
         for (uint32_t e = 0; e < 8u; ++e) x[e] = (h0 + r < p.heads && c + e < W) ? qa[(size_t)(h0 + r) * W + c + e] : 0.f;
@@ -388,12 +431,13 @@ __global__ __launch_bounds__(256) void latent_step_kernel(const decdec_latent p,
     for (int i = 0; i < NR; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     for (uint32_t k0 = lo_key; k0 < hi_key; k0 += KT) {
         __syncthreads();
-        for (uint32_t i = tid; i < KT * (Wp / 8u); i += 256u) {
-            const uint32_t r = i / (Wp / 8u), c = (i % (Wp / 8u)) * 8u, key = k0 + r;
-            const T* src = (const T*)p.cache + (size_t)key * W + c;
-            store8(Kl + r * KL + c, load8<DT>(key < hi_key ? src : (const T*)p.cache, key < hi_key ? (int)W - (int)c : 0, vec));
+#pragma unroll
+        for (uint32_t j = 0; j < NL; ++j) {
+            const uint32_t i = tid + kStepThreads * j, r = i / W8;
+            if (r < (uint32_t)KT) store8(Kl + r * KL + (i - r * W8) * 8u, kr[j]);
         }
         __syncthreads();
+        if (k0 + KT < hi_key) request(k0 + KT);
         {
             f32x4 sc = {0.f, 0.f, 0.f, 0.f};
             const uint32_t kb = wave % KB, part = wave / KB, slices = Wp / 32u;
@@ -407,35 +451,23 @@ __global__ __launch_bounds__(256) void latent_step_kernel(const decdec_latent p,
         }
         __syncthreads();
         {
-            // 16 threads per head
-            const uint32_t hd = tid >> 4, t = tid & 15u;
-            float x[KB], best = mxs[hd];
-            const float m0 = best;
+            float x = 0.f;
+            const bool in = lane < (uint32_t)KT && k0 + lane < hi_key;
+            if (in)
 #pragma unroll
-            for (uint32_t j = 0; j < KB; ++j) {
-                const uint32_t key = t + 16u * j;
-                x[j] = 0.f;
+                for (uint32_t n = 0; n < SP; ++n) x += Pl[n][lane][wave];
+            const float m0 = mxs[wave];
+            float best = in ? fmaxf(x, m0) : m0;
 #pragma unroll
-                for (uint32_t n = 0; n < SP; ++n) x[j] += Pl[n][key][hd];
-                if (k0 + key >= hi_key) x[j] = -__builtin_inff();
-                best = fmaxf(best, x[j]);
-            }
-#pragma unroll
-            for (int off = 1; off < 16; off <<= 1) best = fmaxf(best, __shfl_xor(best, off, 64));
-            float sum = 0.f;
-#pragma unroll
-            for (uint32_t j = 0; j < KB; ++j) {
-                x[j] = __expf(x[j] - best);                                // the tile has at least one key: best is finite
-                sum += x[j];
-                Pl[0][t + 16u * j][hd] = x[j];
-            }
-#pragma unroll
-            for (int off = 1; off < 16; off <<= 1) sum += __shfl_xor(sum, off, 64);
-            if (t == 0u) {
+            for (int off = 1; off < 64; off <<= 1) best = fmaxf(best, __shfl_xor(best, off, 64));
+            const float w = in ? __expf(x - best) : 0.f;                   // the tile has at least one key: best is finite
+            if (lane < (uint32_t)KT) Pl[0][lane][wave] = w;                // only this wave reads or writes the head's column
+            const float t = wave_sum(w);
+            if (lane == 0u) {
                 const float corr = __expf(m0 - best);
-                corrs[hd] = corr;
-                sums[hd] = sums[hd] * corr + sum;
-                mxs[hd] = best;
+                corrs[wave] = corr;
+                sums[wave] = sums[wave] * corr + t;
+                mxs[wave] = best;
             }
         }
         __syncthreads();
@@ -450,7 +482,7 @@ __global__ __launch_bounds__(256) void latent_step_kernel(const decdec_latent p,
         }
 #pragma unroll
         for (int i = 0; i < NR; ++i) {
-            const uint32_t tile = wave + 4u * (uint32_t)i;
+            const uint32_t tile = wave + 16u * (uint32_t)i;
             if (16u * tile < R) {
                 o[i] *= corr;
 #pragma unroll
@@ -469,22 +501,21 @@ __global__ __launch_bounds__(256) void latent_step_kernel(const decdec_latent p,
         for (int i = 0; i < NR; ++i)
 #pragma unroll
             for (int v = 0; v < 4; ++v) {
-                const uint32_t r = 16u * (wave + 4u * (uint32_t)i) + 4u * lg + (uint32_t)v;
+                const uint32_t r = 16u * (wave + 16u * (uint32_t)i) + 4u * lg + (uint32_t)v;
                 if (r < R) dst[r] = o[i][v];
             }
         if (wave == 0u && lg == 0u) { dst[R] = mxs[l16]; dst[R + 1u] = sums[l16]; }
     }
 }
 
-// Merge of the splits and the values: grid (heads, vdim / 32).
+// Merge of the splits and the values: grid (heads, vdim / 32), sixteen waves of two value rows each.  The value matrix'
+// rows are requested first; they wait for nothing.
 template <int DT>
-__global__ __launch_bounds__(256) void latent_merge_kernel(const decdec_latent p, const float* __restrict__ parts,
-                                                           void* __restrict__ out, const uint32_t max_splits) {
+__global__ __launch_bounds__(1024) void latent_merge_kernel(const decdec_latent p, const float* __restrict__ parts,
+                                                            void* __restrict__ out, const uint32_t max_splits) {
     using E = Elem<DT>;
     using T = typename LaneOf<DT>::t;
-    extern __shared__ __align__(16) unsigned char smem[];
-    float* lat = (float*)smem;                           // [rank rounded up to 8]
-    __shared__ float ws[64];
+    __shared__ float lat[1024], share[1024], ws[64];
     const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, h = blockIdx.x, R = p.rank, V = p.vdim;
     const long long pos = *p.pos;
     if (pos < 0) return;
@@ -492,38 +523,61 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const decdec_latent p
     const uint32_t n = step_split(len, max_splits).splits;               // at most 64
     const float* ph = parts + (size_t)h * (R + 2u);
     const size_t ps = (size_t)p.heads * (R + 2u);
+    const bool vec = R % 8u == 0;
+    Frag<DT> uv[2][2];
+#pragma unroll
+    for (uint32_t i = 0; i < 2u; ++i)
+#pragma unroll
+        for (uint32_t j = 0; j < 2u; ++j) {
+            const uint32_t d = blockIdx.y * 32u + wave * 2u + i, c = lane * 8u + 512u * j;
+            uv[i][j] = load8<DT>((const T*)p.uv + ((size_t)h * V + (d < V ? d : 0u)) * R + (c < R ? c : 0u), d < V ? (int)R - (int)c : 0, vec);
+        }
+    // the splits are summed in `groups` shares of the workgroup, Rp threads each
+    const uint32_t Rp = (R + 63u) & ~63u, groups = 1024u / Rp, g = tid / Rp, r = tid - g * Rp;
+    const bool mine = g < groups && r < R;
     if (wave == 0u) {
         const float sink = p.sink != nullptr ? E::load(p.sink, h) : -__builtin_inff();
-        const float m = lane < n ? ph[lane * ps + R] : -__builtin_inff();
+        const float m = lane < n ? ph[lane * ps + R] : -__builtin_inff(), l = lane < n ? ph[lane * ps + R + 1u] : 0.f;
         float M = fmaxf(m, sink);
 #pragma unroll
         for (int off = 32; off >= 1; off >>= 1) M = fmaxf(M, __shfl_xor(M, off, 64));
         const float w = lane < n ? __expf(m - M) : 0.f;
-        const float L = wave_sum(lane < n ? w * ph[lane * ps + R + 1u] : 0.f) + (p.sink != nullptr ? __expf(sink - M) : 0.f);
+        const float L = wave_sum(w * l) + (p.sink != nullptr ? __expf(sink - M) : 0.f);
         ws[lane] = w / L;
     }
     __syncthreads();
-    for (uint32_t r = tid; r < ((R + 7u) & ~7u); r += 256u) {
-        float t = 0.f;
-        if (r < R)
-            for (uint32_t s = 0; s < n; ++s) t = __builtin_fmaf(ws[s], ph[s * ps + r], t);
-        lat[r] = t;
+    float t = 0.f;
+    if (mine) {
+        for (uint32_t s = g; s < n; s += 8u * groups) {
+            float x[8];
+#pragma unroll
+            for (uint32_t e = 0; e < 8u; ++e) x[e] = s + e * groups < n ? ph[(s + e * groups) * ps + r] : 0.f;
+#pragma unroll
+            for (uint32_t e = 0; e < 8u; ++e) t = __builtin_fmaf(s + e * groups < n ? ws[s + e * groups] : 0.f, x[e], t);
+        }
+    }
+    share[tid] = t;
+    __syncthreads();
+    {
+        float a = 0.f;
+        if (tid < R)
+            for (uint32_t k = 0; k < groups; ++k) a += share[k * Rp + tid];
+        lat[tid] = a;                                                      // zero past the rank
     }
     __syncthreads();
-    const bool vec = R % 8u == 0;
-    for (uint32_t i = 0; i < 8u; ++i) {
-        const uint32_t d = blockIdx.y * 32u + wave * 8u + i;
-        if (d >= V) break;                                                 // uniform over the wave
-        const T* uv = (const T*)p.uv + ((size_t)h * V + d) * R;
-        float acc = 0.f;
-        for (uint32_t c = lane * 8u; c < R; c += 512u) {
-            float w[8];
-            frag_values(load8<DT>(uv + c, (int)R - (int)c, vec), w);
 #pragma unroll
-            for (int e = 0; e < 8; ++e) acc = __builtin_fmaf(w[e], lat[c + e], acc);
+    for (uint32_t i = 0; i < 2u; ++i) {
+        const uint32_t d = blockIdx.y * 32u + wave * 2u + i;
+        float acc = 0.f;
+#pragma unroll
+        for (uint32_t j = 0; j < 2u; ++j) {
+            float w[8];
+            frag_values(uv[i][j], w);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) acc = __builtin_fmaf(w[e], lat[lane * 8u + 512u * j + e], acc);
         }
         acc = wave_sum(acc);
-        if (lane == 0u) E::store(out, (size_t)h * V + d, acc);
+        if (lane == 0u && d < V) E::store(out, (size_t)h * V + d, acc);
     }
 }
 
@@ -534,23 +588,22 @@ size_t latent_step_workspace(const decdec_latent& p) {
 template <int DT, int KT, int NR>
 static hipError_t step_launch(const decdec_latent& p, const float* qa, float* parts, dim3 grid, size_t lds, uint32_t splits, hipStream_t s) {
     if (hipError_t e = allow_lds<latent_step_kernel<DT, KT, NR>>(lds); e != hipSuccess) return e;
-    hipLaunchKernelGGL((latent_step_kernel<DT, KT, NR>), grid, dim3(256), lds, s, p, qa, parts, splits);
+    hipLaunchKernelGGL((latent_step_kernel<DT, KT, NR>), grid, dim3(kStepThreads), lds, s, p, qa, parts, splits);
     return hipGetLastError();
 }
 
 template <int DT, int KT>
 static hipError_t step_dt(const decdec_latent& p, void* out, float* qa, float* parts, hipStream_t s) {
     constexpr uint32_t PAD = DT == kFP32 ? 4u : 8u, QN = DT == kFP32 ? 1u : 2u;
-    const uint32_t splits = step_max_splits(p), Wp = (p.rank + p.rot + 31u) & ~31u, tiles = ((p.rank + 15u) / 16u + 3u) / 4u;
+    const uint32_t splits = step_max_splits(p), Wp = (p.rank + p.rot + 31u) & ~31u, tiles = ((p.rank + 15u) / 16u + 15u) / 16u;
     const size_t lds = (size_t)(KT + QN * 16u) * (Wp + PAD) * Elem<DT>::bytes;
     if (lds > 140u * 1024u) return hipErrorInvalidValue;
     const dim3 grid(splits, (p.heads + 15u) / 16u), block(256);
     hipLaunchKernelGGL((latent_absorb_kernel<DT>), dim3(p.heads + 1u, (p.rank + 63u) / 64u), block, 0, s, p, qa);
-    hipError_t e = tiles <= 2u ? step_launch<DT, KT, 2>(p, qa, parts, grid, lds, splits, s)
-                 : tiles <= 8u ? step_launch<DT, KT, 8>(p, qa, parts, grid, lds, splits, s)
-                 : tiles <= 16u ? step_launch<DT, KT, 16>(p, qa, parts, grid, lds, splits, s) : hipErrorInvalidValue;
+    hipError_t e = tiles <= 1u ? step_launch<DT, KT, 1>(p, qa, parts, grid, lds, splits, s)
+                 : tiles <= 3u ? step_launch<DT, KT, 3>(p, qa, parts, grid, lds, splits, s) : hipErrorInvalidValue;
     if (e != hipSuccess) return e;
-    hipLaunchKernelGGL((latent_merge_kernel<DT>), dim3(p.heads, (p.vdim + 31u) / 32u), block, ((size_t)p.rank + 8u) * 4u, s, p, parts, out, splits);
+    hipLaunchKernelGGL((latent_merge_kernel<DT>), dim3(p.heads, (p.vdim + 31u) / 32u), dim3(1024), 0, s, p, parts, out, splits);
     return hipGetLastError();
 }
 

@@ -58,12 +58,21 @@ __global__ __launch_bounds__(1024) void recurrence_step_kernel(const decdec_recu
         const uint32_t slot = (uint32_t)(pos < 0 ? 0 : pos % (long long)taps);
         // channel c of the ring, whose projection is proj[src] and whose taps are w[wc * taps ..]
         auto conv = [&](uint32_t src, uint32_t c, const void* w, uint32_t wc, bool keep) {
-            const uint32_t raw = E::load_raw(p.proj, src);
-            float y = E::load(w, (size_t)wc * taps + taps - 1u) * E::from_raw(raw);
-            for (uint32_t b = 1; b < taps; ++b) {                          // b tokens back
-                if (pos < (long long)b) break;
-                const uint32_t sl = (slot + taps - b) % taps;
-                y = __builtin_fmaf(E::load(w, (size_t)wc * taps + taps - 1u - b), E::load(p.ring, (size_t)sl * chans + c), y);
+            const float in = E::load(p.proj, src);
+            float y = E::load(w, (size_t)wc * taps + taps - 1u) * in;
+            for (uint32_t b0 = 1; b0 < taps; b0 += 4u) {                   // b tokens back, four requested together
+                float wv[4], xv[4];
+                bool ok[4];
+#pragma unroll
+                for (uint32_t e = 0; e < 4u; ++e) {
+                    const uint32_t b = b0 + e;
+                    ok[e] = b < taps && pos >= (long long)b;
+                    const uint32_t bc = ok[e] ? b : 0u;
+                    wv[e] = E::load(w, (size_t)wc * taps + taps - 1u - bc);
+                    xv[e] = E::load(p.ring, (size_t)((slot + taps - bc) % taps) * chans + c);
+                }
+#pragma unroll
+                for (uint32_t e = 0; e < 4u; ++e) y += ok[e] ? wv[e] * xv[e] : 0.f;
             }
             if (keep) ((typename LaneOf<DT>::t*)p.ring)[(size_t)slot * chans + c] = ((const typename LaneOf<DT>::t*)p.proj)[src];
             return silu_f(y);
@@ -231,6 +240,90 @@ __global__ __launch_bounds__(256) void delta_inputs_kernel(const decdec_recurren
     }
 }
 
+// The same for at most TAPS taps and widths that are multiples of four: a workgroup takes eight tokens, a thread four
+// neighbouring channels, whose inputs (and the taps before them) are all requested at once.
+constexpr uint32_t kInputRows = 8;
+
+template <int DT>
+__device__ __forceinline__ void quad(const void* p, size_t i, float (&v)[4]) {
+    if constexpr (DT == kFP32) {
+        const f32x4 t = *(const f32x4*)((const float*)p + i);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = t[e];
+    } else {
+        const u32x2 t = *(const u32x2*)((const uint16_t*)p + i);
+        v[0] = __uint_as_float(t[0] << 16); v[1] = __uint_as_float(t[0] & 0xFFFF0000u);
+        v[2] = __uint_as_float(t[1] << 16); v[3] = __uint_as_float(t[1] & 0xFFFF0000u);
+    }
+}
+
+template <int DT, int TAPS>
+__global__ __launch_bounds__(256) void delta_inputs_quad_kernel(const decdec_recurrence p, float* __restrict__ q, float* __restrict__ k,
+                                                                float* __restrict__ v, float* __restrict__ lg, float* __restrict__ beta,
+                                                                const uint32_t rows, const uint32_t gl) {
+    using E = Elem<DT>;
+    constexpr int N = (int)kInputRows, B = TAPS - 1;
+    const uint32_t tid = threadIdx.x, D = p.dim, taps = p.taps, t0 = blockIdx.x * kInputRows;
+    const uint32_t nqk = p.kv_heads * D, nv = p.heads * p.vdim, chans = 2u * nqk + nv;
+    const long long pos0 = *p.pos;
+    // y[t] of channels off + wc .. + 3, ring channel c
+    auto conv = [&](uint32_t off, uint32_t c, const void* w, uint32_t wc, float (&y)[N][4]) {
+        float x[B + N][4], wt[TAPS][4];
+#pragma unroll
+        for (int i = 0; i < B + N; ++i) {
+            const int t = (int)t0 + i - B;                                 // token of the portion, negative before it
+            if (t >= 0) quad<DT>(p.proj, (size_t)((uint32_t)t < rows ? (uint32_t)t : rows - 1u) * p.ld + off + wc, x[i]);
+            else if (pos0 + t >= 0 && -t < (int)taps) quad<DT>(p.ring, (size_t)((pos0 + t) % taps) * chans + c, x[i]);
+            else x[i][0] = x[i][1] = x[i][2] = x[i][3] = 0.f;
+        }
+#pragma unroll
+        for (int b = 0; b < TAPS; ++b)
+#pragma unroll
+            for (uint32_t e = 0; e < 4u; ++e)
+                wt[b][e] = (uint32_t)b < taps ? E::load(w, (size_t)(wc + e) * taps + taps - 1u - (uint32_t)b) : 0.f;
+#pragma unroll
+        for (int t = 0; t < N; ++t)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                float a = 0.f;
+#pragma unroll
+                for (int b = 0; b < TAPS; ++b) a = __builtin_fmaf(wt[b][e], x[B + t - b][e], a);
+                y[t][e] = silu_f(a);
+            }
+    };
+    auto put = [&](float* dst, uint32_t t, uint32_t width, uint32_t c, const float (&y)[4], float r) {
+        if (t0 + t < rows) *(f32x4*)(dst + (size_t)(t0 + t) * width + c) = f32x4{y[0] * r, y[1] * r, y[2] * r, y[3] * r};
+    };
+    const uint32_t c4 = (tid % gl) * 4u;                                   // gl threads share a head
+    for (uint32_t j = tid / gl; j < (2u * p.kv_heads + 256u / gl - 1u) / (256u / gl) * (256u / gl); j += 256u / gl) {
+        const bool isq = j < p.kv_heads, live = j < 2u * p.kv_heads && c4 < D;
+        const uint32_t ch = live ? (isq ? j : j - p.kv_heads) * D + c4 : 0u;
+        float y[N][4];
+        conv(isq || !live ? p.off_q : p.off_k, (isq || !live ? 0u : nqk) + ch, isq || !live ? p.conv_q : p.conv_k, ch, y);
+#pragma unroll
+        for (int t = 0; t < N; ++t) {
+            float ss = live ? y[t][0] * y[t][0] + y[t][1] * y[t][1] + y[t][2] * y[t][2] + y[t][3] * y[t][3] : 0.f;
+            for (uint32_t off = 1; off < gl; off <<= 1) ss += __shfl_xor(ss, (int)off, 64);
+            float r = 1.f / sqrtf(ss + 1e-6f);
+            if (isq) r /= sqrtf((float)D);
+            if (live) put(isq ? q : k, (uint32_t)t, nqk, ch, y[t], r);
+        }
+    }
+    for (uint32_t c = 4u * tid; c < nv; c += 1024u) {
+        float y[N][4];
+        conv(p.off_v, 2u * nqk + c, p.conv_v, c, y);
+#pragma unroll
+        for (int t = 0; t < N; ++t) put(v, (uint32_t)t, nv, c, y[t], 1.f);
+    }
+    for (uint32_t i = tid; i < p.heads * kInputRows; i += 256u) {
+        const uint32_t t = t0 + i / p.heads, h = i % p.heads;
+        if (t < rows) {
+            lg[(size_t)t * p.heads + h] = log_decay<DT>(p, p.proj, (size_t)t * p.ld, h);
+            beta[(size_t)t * p.heads + h] = sigmoid_f(E::load(p.proj, (size_t)t * p.ld + p.off_b + h));
+        }
+    }
+}
+
 // The last min(rows, taps) projections into the ring (after delta_inputs has read the old ones).
 template <int DT>
 __global__ __launch_bounds__(256) void ring_update_kernel(const decdec_recurrence p, const uint32_t rows) {
@@ -265,21 +358,30 @@ __device__ __forceinline__ Frag<kFP32> row_frag(const float* p, int valid, bool 
     return f;
 }
 
-// 64 rows x 32 columns of an array of rows (stride ld) into LDS [64][36]; rows past n and columns past D are zero.
-__device__ __forceinline__ void load_slice(const float* src, size_t ld, uint32_t n, uint32_t c0, uint32_t D, float (*dst)[36], bool vec) {
-    const uint32_t tid = threadIdx.x;
+// 64 rows x 32 columns of an array of rows (stride ld), requested into registers and later put into LDS [64][36]; rows past
+// n and columns past D are zero.
+struct Slice { f32x4 x[2]; };
+__device__ __forceinline__ Slice slice_fetch(const float* src, size_t ld, uint32_t n, uint32_t c0, uint32_t D, bool vec) {
+    Slice s;
 #pragma unroll
     for (uint32_t e = 0; e < 2; ++e) {
-        const uint32_t i = tid + 256u * e, r = i >> 3, c = (i & 7u) * 4u;
-        f32x4 x = {0.f, 0.f, 0.f, 0.f};
-        if (r < n) {
-            const float* s = src + (size_t)r * ld + c0 + c;
-            if (vec && c0 + c + 4u <= D) x = *(const f32x4*)s;
-            else
+        const uint32_t i = threadIdx.x + 256u * e, r = i >> 3, c = c0 + (i & 7u) * 4u;
+        const float* row = src + (size_t)(r < n ? r : 0u) * ld;
+        if (vec) {                                         // D is a multiple of four
+            s.x[e] = *(const f32x4*)(row + (c < D ? c : 0u));
+            if (r >= n || c >= D) s.x[e] = f32x4{0.f, 0.f, 0.f, 0.f};
+        } else {
 #pragma unroll
-                for (int j = 0; j < 4; ++j) x[j] = c0 + c + (uint32_t)j < D ? s[j] : 0.f;
+            for (int j = 0; j < 4; ++j) s.x[e][j] = (r < n && c + (uint32_t)j < D) ? row[c + j] : 0.f;
         }
-        *(f32x4*)&dst[r][c] = x;
+    }
+    return s;
+}
+__device__ __forceinline__ void slice_put(const Slice& s, float (*dst)[36]) {
+#pragma unroll
+    for (uint32_t e = 0; e < 2; ++e) {
+        const uint32_t i = threadIdx.x + 256u * e;
+        *(f32x4*)&dst[i >> 3][(i & 7u) * 4u] = s.x[e];
     }
 }
 
@@ -302,10 +404,12 @@ __global__ __launch_bounds__(256) void delta_solve_kernel(const ChunkParams p) {
     f32x4 acc[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    Slice ks = slice_fetch(k, kld, n, 0u, D, vec);
     for (uint32_t c0 = 0; c0 < D; c0 += 32u) {
         __syncthreads();
-        load_slice(k, kld, n, c0, D, Ks, vec);
+        slice_put(ks, Ks);
         __syncthreads();
+        if (c0 + 32u < D) ks = slice_fetch(k, kld, n, c0 + 32u, D, vec);
         const Frag<kFP32> a = frag_load(&Ks[16u * wave + (lane & 15u)][8u * (lane >> 4)]);
 #pragma unroll
         for (int j = 0; j < 4; ++j) mma(a, frag_load(&Ks[16u * j + (lane & 15u)][8u * (lane >> 4)]), acc[j]);
@@ -377,6 +481,7 @@ __global__ __launch_bounds__(256) void delta_solve_kernel(const ChunkParams p) {
 }
 
 // States: grid (heads, vdim / 16), one walk over the chunks.  Wave w owns the state's row tiles w, w + 4, ... (NT of them).
+// What the next chunk needs from memory is requested as soon as this chunk's copy has been used.
 template <bool DELTA, int NT>
 __global__ __launch_bounds__(256) void chunk_state_kernel(const ChunkParams p, const uint32_t chunks) {
     extern __shared__ __align__(16) float lds[];
@@ -399,22 +504,61 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(const ChunkParams p, c
             const uint32_t r = 16u * (wave + 4u * (uint32_t)i) + 4u * lg + (uint32_t)v;
             s[i][v] = (r < D && col && !fresh) ? S[(size_t)r * V] : 0.f;
         }
+    const uint32_t kr = tid >> 2, kc = (tid & 3u) * 4u;                    // a thread's row of the keys, and columns kc + 16 j
+    f32x4 kreg[4 * NT];
+    Frag<kFP32> wreg[DELTA ? 2 * NT : 1];
+    float ureg[4], lreg = 0.f;
+    auto request_keys = [&](uint32_t t0) {
+        const uint32_t n = p.rows - t0 < C ? p.rows - t0 : C;
+        const float* k = p.k + ((size_t)(t0 + (kr < n ? kr : 0u)) * p.kv_heads + kvh) * D;
+#pragma unroll
+        for (int j = 0; j < 4 * NT; ++j) {
+            const uint32_t c = kc + 16u * (uint32_t)j;
+            if (vec) {
+                kreg[j] = *(const f32x4*)(k + (c < D ? c : 0u));
+                if (kr >= n || c >= D) kreg[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) kreg[j][e] = (kr < n && c + (uint32_t)e < D) ? k[c + e] : 0.f;
+            }
+        }
+        if constexpr (DELTA) lreg = (wave == 3u && lane < n) ? p.lg[(size_t)(t0 + lane) * p.heads + h] : 0.f;
+    };
+    auto request_writes = [&](uint32_t t0) {
+        const uint32_t n = p.rows - t0 < C ? p.rows - t0 : C, ar = 16u * wave + l16;
+        if constexpr (DELTA) {
+            const float* w = p.w + ((size_t)(t0 + (ar < n ? ar : 0u)) * p.heads + h) * D;
+#pragma unroll
+            for (int j = 0; j < 2 * NT; ++j) {
+                const uint32_t kk = 32u * (uint32_t)j + 8u * lg;
+                wreg[j] = row_frag(w + kk, ar < n ? (int)D - (int)kk : 0, vec8);
+            }
+        }
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            const uint32_t r = 16u * wave + 4u * lg + (uint32_t)v;
+            const size_t at = ((size_t)(t0 + (r < n ? r : 0u)) * p.heads + h) * V + v0 + (col ? l16 : 0u);
+            ureg[v] = DELTA ? p.u[at] : p.v[at];
+        }
+    };
+    request_keys(0u);
+    request_writes(0u);
     for (uint32_t ch = 0; ch < chunks; ++ch) {
         const uint32_t t0 = ch * C, n = p.rows - t0 < C ? p.rows - t0 : C;
-        const float* k = p.k + ((size_t)t0 * p.kv_heads + kvh) * D;
-        const size_t kld = (size_t)p.kv_heads * D;
-        for (uint32_t i = tid; i < C * (Dp / 4u); i += 256u) {
-            const uint32_t r = i / (Dp / 4u), c = (i % (Dp / 4u)) * 4u;
-            f32x4 x = {0.f, 0.f, 0.f, 0.f};
-            if (r < n) {
-                if (vec && c + 4u <= D) x = *(const f32x4*)(k + (size_t)r * kld + c);
-                else
 #pragma unroll
-                    for (int j = 0; j < 4; ++j) x[j] = c + (uint32_t)j < D ? k[(size_t)r * kld + c + j] : 0.f;
+        for (int j = 0; j < 4 * NT; ++j)
+            if (kc + 16u * (uint32_t)j < Dp) *(f32x4*)&Kl[kr * KL + kc + 16u * (uint32_t)j] = kreg[j];
+        if constexpr (DELTA) {
+            if (wave == 3u) {                                              // log-decays summed up, in double
+                double x = (double)lreg;
+#pragma unroll
+                for (int off = 1; off < 64; off <<= 1) {
+                    const double y = __shfl_up(x, off, 64);
+                    if ((int)lane >= off) x += y;
+                }
+                G[lane] = x;
             }
-            *(f32x4*)&Kl[r * KL + c] = x;
         }
-        if constexpr (DELTA) { if (wave == 3) chunk_log_decay(p, t0, n, h, G); }
         float* st = p.states + ((size_t)ch * p.heads + h) * D * V + v0 + l16;
 #pragma unroll
         for (int i = 0; i < NT; ++i)
@@ -425,36 +569,33 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(const ChunkParams p, c
                 if (r < D && col) st[(size_t)r * V] = s[i][v];
             }
         __syncthreads();
+        if (ch + 1u < chunks) request_keys(t0 + C);
         const float gend = DELTA ? expf((float)G[C - 1]) : pw[n];
         {
             // what the tokens write, 16 rows per wave
             f32x4 acc = {0.f, 0.f, 0.f, 0.f};
             if constexpr (DELTA) {
-                const uint32_t ar = 16u * wave + l16;
-                const float* w = p.w + ((size_t)(t0 + (ar < n ? ar : 0u)) * p.heads + h) * D;
-                for (uint32_t c0 = 0; c0 < D; c0 += 32u) {
-                    const uint32_t kk = c0 + 8u * lg;
-                    const Frag<kFP32> a = row_frag(w + kk, ar < n ? (int)D - (int)kk : 0, vec8);
-                    mma(a, frag_gather(Sl + kk * 20u + l16, 20u), acc);
-                }
+#pragma unroll
+                for (int j = 0; j < 2 * NT; ++j)
+                    if (32u * (uint32_t)j < D) mma(wreg[j], frag_gather(Sl + (32u * (uint32_t)j + 8u * lg) * 20u + l16, 20u), acc);
             }
 #pragma unroll
             for (int v = 0; v < 4; ++v) {
                 const uint32_t r = 16u * wave + 4u * lg + (uint32_t)v;
                 float x = 0.f;
                 if (r < n && col) {
-                    const size_t at = ((size_t)(t0 + r) * p.heads + h) * V + v0 + l16;
                     if constexpr (DELTA) {
-                        x = p.u[at] - acc[v];
-                        p.u[at] = x;
+                        x = ureg[v] - acc[v];
+                        p.u[((size_t)(t0 + r) * p.heads + h) * V + v0 + l16] = x;
                         x *= expf((float)(G[C - 1] - G[r]));
                     } else {
-                        x = p.v[at] * pw[n - 1u - r];
+                        x = ureg[v] * pw[n - 1u - r];
                     }
                 }
                 Vl[r][l16] = x;
             }
         }
+        if (ch + 1u < chunks) request_writes(t0 + C);
         __syncthreads();
 #pragma unroll
         for (int i = 0; i < NT; ++i) {
@@ -498,22 +639,53 @@ __global__ __launch_bounds__(256) void chunk_output_kernel(const ChunkParams p) 
     const float* S = p.states + ((size_t)blockIdx.x * p.heads + h) * D * V;
     if constexpr (DELTA) { if (wave == 0) chunk_log_decay(p, t0, n, h, G); }
     else { for (uint32_t i = tid; i <= C; i += 256u) pw[i] = p.decay[(size_t)h * 65u + i]; }
-    for (uint32_t i = tid; i < C * 64u; i += 256u) {
-        const uint32_t r = i >> 6, c = i & 63u;
-        Vs[r][c] = (r < n && v0 + c < V) ? vv[(size_t)r * p.heads * V + v0 + c] : 0.f;
+    // four neighbouring columns of a 64-column array per thread and pass, 16 rows a pass
+    const bool vecv = V % 4u == 0;
+    const uint32_t vr = tid >> 4, vc = (tid & 15u) * 4u;
+    auto value4 = [&](const float* row, bool in) {
+        f32x4 x = {0.f, 0.f, 0.f, 0.f};
+        if (vecv) {
+            x = *(const f32x4*)(row + (v0 + vc < V ? v0 + vc : 0u));
+            if (!in || v0 + vc >= V) x = f32x4{0.f, 0.f, 0.f, 0.f};
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                if (in && v0 + vc + (uint32_t)e < V) x[e] = row[v0 + vc + e];
+        }
+        return x;
+    };
+    Slice qr = slice_fetch(q, kld, n, 0u, D, vec), kr = slice_fetch(k, kld, n, 0u, D, vec);
+    f32x4 sr[2], val[4];
+    auto fetch_state = [&](uint32_t c0) {
+#pragma unroll
+        for (uint32_t e = 0; e < 2u; ++e) {
+            const uint32_t r = c0 + vr + 16u * e;
+            sr[e] = value4(S + (size_t)(r < D ? r : 0u) * V, r < D);
+        }
+    };
+    fetch_state(0u);
+#pragma unroll
+    for (uint32_t e = 0; e < 4u; ++e) {
+        const uint32_t r = vr + 16u * e;
+        val[e] = value4(vv + (size_t)(r < n ? r : 0u) * p.heads * V, r < n);
     }
+#pragma unroll
+    for (uint32_t e = 0; e < 4u; ++e) *(f32x4*)&Vs[vr + 16u * e][vc] = val[e];
     f32x4 pr[4], o[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) { pr[j] = f32x4{0.f, 0.f, 0.f, 0.f}; o[j] = f32x4{0.f, 0.f, 0.f, 0.f}; }
     for (uint32_t c0 = 0; c0 < D; c0 += 32u) {
         __syncthreads();
-        load_slice(q, kld, n, c0, D, Qs, vec);
-        load_slice(k, kld, n, c0, D, Ks, vec);
-        for (uint32_t i = tid; i < 32u * 64u; i += 256u) {
-            const uint32_t r = i >> 6, c = i & 63u;
-            Ss[r][c] = (c0 + r < D && v0 + c < V) ? S[(size_t)(c0 + r) * V + v0 + c] : 0.f;
-        }
+        slice_put(qr, Qs);
+        slice_put(kr, Ks);
+#pragma unroll
+        for (uint32_t e = 0; e < 2u; ++e) *(f32x4*)&Ss[vr + 16u * e][vc] = sr[e];
         __syncthreads();
+        if (c0 + 32u < D) {
+            qr = slice_fetch(q, kld, n, c0 + 32u, D, vec);
+            kr = slice_fetch(k, kld, n, c0 + 32u, D, vec);
+            fetch_state(c0 + 32u);
+        }
         const Frag<kFP32> a = frag_load(&Qs[16u * wave + l16][8u * lg]);
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
@@ -608,8 +780,18 @@ static hipError_t rows_dt(const decdec_recurrence& p, const ChunkParams& c, hipS
         hipLaunchKernelGGL((plain_inputs_kernel<DT>), dim3(c.rows), dim3(256), 0, s, p, (float*)c.q, (float*)c.k, (float*)c.v);
         return launch_chunks<false>(c, s);
     }
-    hipLaunchKernelGGL((delta_inputs_kernel<DT>), dim3(c.rows), dim3(256), 0, s, p, (float*)c.q, (float*)c.k, (float*)c.v,
-                       (float*)c.lg, (float*)c.beta);
+    const uint32_t es = Elem<DT>::bytes;
+    uint32_t gl = 1;
+    while (4u * gl < p.dim) gl *= 2;
+    const bool quads = ((p.dim | p.ld | p.off_q | p.off_k | p.off_v | (p.heads * p.vdim)) & 3u) == 0 && p.taps <= 8u &&
+                       (uintptr_t)p.proj % (4u * es) == 0 && (uintptr_t)p.ring % (4u * es) == 0;
+    const dim3 wide((c.rows + kInputRows - 1u) / kInputRows);
+    if (quads && p.taps <= 4u)
+        hipLaunchKernelGGL((delta_inputs_quad_kernel<DT, 4>), wide, dim3(256), 0, s, p, (float*)c.q, (float*)c.k, (float*)c.v, (float*)c.lg, (float*)c.beta, c.rows, gl);
+    else if (quads)
+        hipLaunchKernelGGL((delta_inputs_quad_kernel<DT, 8>), wide, dim3(256), 0, s, p, (float*)c.q, (float*)c.k, (float*)c.v, (float*)c.lg, (float*)c.beta, c.rows, gl);
+    else
+        hipLaunchKernelGGL((delta_inputs_kernel<DT>), dim3(c.rows), dim3(256), 0, s, p, (float*)c.q, (float*)c.k, (float*)c.v, (float*)c.lg, (float*)c.beta);
     const uint32_t chans = 2u * p.kv_heads * p.dim + p.heads * p.vdim, keep = c.rows < p.taps ? c.rows : p.taps;
     hipLaunchKernelGGL((ring_update_kernel<DT>), dim3((chans + 255u) / 256u, keep), dim3(256), 0, s, p, c.rows);
     hipLaunchKernelGGL(delta_solve_kernel, dim3((c.rows + C - 1u) / C, p.heads), dim3(256), 0, s, c);

@@ -105,31 +105,7 @@ hipError_t launch_mix_gemv(int dt, const void* w, const void* x, void* out, cons
     return hipGetLastError();
 }
 
-// ---- embedding --------------------------------------------------------------------------------------------
-template <int DT>
-__global__ __launch_bounds__(256) void mix_embed_kernel(const void* __restrict__ table, const long long* __restrict__ tokens,
-                                                        float* __restrict__ x, void* __restrict__ xe, uint32_t vocab, uint32_t dim) {
-    using E = Elem<DT>;
-    const uint32_t r = blockIdx.x;
-    long long t = tokens[r];
-    if (t < 0 || t >= (long long)vocab) t = 0;
-    for (uint32_t i = threadIdx.x; i < dim; i += blockDim.x) {
-        const float v = E::load(table, (size_t)t * dim + i);
-        x[(size_t)r * dim + i] = v;
-        if (xe != nullptr) E::store(xe, (size_t)r * dim + i, v);
-    }
-}
-
-hipError_t launch_mix_embed(int dt, const void* table, const long long* tokens, float* x, void* xe, uint32_t rows,
-                            uint32_t vocab, uint32_t dim, hipStream_t s) {
-    if (dt == kBF16) hipLaunchKernelGGL((mix_embed_kernel<kBF16>), dim3(rows), dim3(256), 0, s, table, tokens, x, xe, vocab, dim);
-    else hipLaunchKernelGGL((mix_embed_kernel<kFP32>), dim3(rows), dim3(256), 0, s, table, tokens, x, xe, vocab, dim);
-    return hipGetLastError();
-}
-
-// ---- gated residual with the norm on the sublayer's output -------------------------------------------------
-// One workgroup per row.  Four neighbouring elements per thread and pass, everything a pass needs requested at once
-// (VEC; element accesses otherwise).  The optional second norm (the model's last one) reads the row just written.
+// four neighbouring elements
 template <int DT>
 __device__ __forceinline__ void load4(const void* p, size_t i, float (&v)[4]) {
     if constexpr (DT == kFP32) {
@@ -151,12 +127,56 @@ __device__ __forceinline__ void store4(void* p, size_t i, const float (&v)[4]) {
         *(u32x4*)((float*)p + i) = t;
     } else {
         u32x2 t;
-        t[0] = (uint32_t)f32_to_bf16_bits(v[0]) | ((uint32_t)f32_to_bf16_bits(v[1]) << 16);
-        t[1] = (uint32_t)f32_to_bf16_bits(v[2]) | ((uint32_t)f32_to_bf16_bits(v[3]) << 16);
+        t[0] = pack_bf16(v[0], v[1]);
+        t[1] = pack_bf16(v[2], v[3]);
         *(u32x2*)((uint16_t*)p + i) = t;
     }
 }
 
+// ---- embedding --------------------------------------------------------------------------------------------
+template <int DT, bool VEC>
+__global__ __launch_bounds__(1024) void mix_embed_kernel(const void* __restrict__ table, const long long* __restrict__ tokens,
+                                                         float* __restrict__ x, void* __restrict__ xe, uint32_t vocab, uint32_t dim) {
+    using E = Elem<DT>;
+    const size_t r = blockIdx.x;
+    long long t = tokens[r];
+    if (t < 0 || t >= (long long)vocab) t = 0;
+    if constexpr (VEC) {
+        for (uint32_t i = 4u * threadIdx.x; i < dim; i += 4u * blockDim.x) {
+            float v[4];
+            load4<DT>(table, (size_t)t * dim + i, v);
+            store4<kFP32>(x, r * dim + i, v);
+            if (xe != nullptr) store4<DT>(xe, r * dim + i, v);
+        }
+    } else {
+        for (uint32_t i = threadIdx.x; i < dim; i += blockDim.x) {
+            const float v = E::load(table, (size_t)t * dim + i);
+            x[r * dim + i] = v;
+            if (xe != nullptr) E::store(xe, r * dim + i, v);
+        }
+    }
+}
+
+template <int DT>
+static hipError_t embed_dt(const void* table, const long long* tokens, float* x, void* xe, uint32_t rows, uint32_t vocab, uint32_t dim,
+                           hipStream_t s) {
+    const uint32_t es = Elem<DT>::bytes;
+    const bool vec = dim % 4u == 0 && (uintptr_t)x % 16u == 0 && ((uintptr_t)table | (uintptr_t)xe) % (4u * es) == 0;
+    uint32_t threads = 64;
+    while (threads < 1024u && threads < (vec ? dim / 4u : dim)) threads *= 2;
+    if (vec) hipLaunchKernelGGL((mix_embed_kernel<DT, true>), dim3(rows), dim3(threads), 0, s, table, tokens, x, xe, vocab, dim);
+    else hipLaunchKernelGGL((mix_embed_kernel<DT, false>), dim3(rows), dim3(threads), 0, s, table, tokens, x, xe, vocab, dim);
+    return hipGetLastError();
+}
+
+hipError_t launch_mix_embed(int dt, const void* table, const long long* tokens, float* x, void* xe, uint32_t rows,
+                            uint32_t vocab, uint32_t dim, hipStream_t s) {
+    return dt == kBF16 ? embed_dt<kBF16>(table, tokens, x, xe, rows, vocab, dim, s) : embed_dt<kFP32>(table, tokens, x, xe, rows, vocab, dim, s);
+}
+
+// ---- gated residual with the norm on the sublayer's output -------------------------------------------------
+// One workgroup per row.  Four neighbouring elements per thread and pass, everything a pass needs requested at once
+// (VEC; element accesses otherwise).  The optional second norm (the model's last one) reads the row just written.
 template <int DT, int PASSES>
 __global__ __launch_bounds__(1024) void gated_residual_vec_kernel(float* __restrict__ x, const void* __restrict__ y,
                                                                   const void* __restrict__ gate, const uint32_t gate_ld,
@@ -295,12 +315,17 @@ __global__ __launch_bounds__(256) void mix_xielu_kernel(const void* __restrict__
     const float sp = softplus_f(E::load(act, 0)), sq = softplus_f(E::load(act, 1));
     const size_t irow = (size_t)blockIdx.x * ld, orow = (size_t)blockIdx.x * n;
     if constexpr (VEC) {
-        for (uint32_t i = 4u * (blockIdx.y * 256u + threadIdx.x); i < n; i += 1024u * gridDim.y) {
-            float v[4];
-            load4<DT>(in, irow + i, v);
+        // four quads a workgroup's width apart, requested together
+        for (uint32_t i0 = 4u * (blockIdx.y * 1024u + threadIdx.x); i0 < n; i0 += 4096u * gridDim.y) {
+            float v[4][4];
 #pragma unroll
-            for (int e = 0; e < 4; ++e) v[e] = xielu_f(v[e], sp, sq);
-            store4<DT>(out, orow + i, v);
+            for (uint32_t k = 0; k < 4u; ++k) load4<DT>(in, irow + (i0 + 1024u * k < n ? i0 + 1024u * k : 0u), v[k]);
+#pragma unroll
+            for (uint32_t k = 0; k < 4u; ++k) {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) v[k][e] = xielu_f(v[k][e], sp, sq);
+                if (i0 + 1024u * k < n) store4<DT>(out, orow + i0 + 1024u * k, v[k]);
+            }
         }
     } else {
         for (uint32_t i = blockIdx.y * 256u + threadIdx.x; i < n; i += 256u * gridDim.y)
@@ -312,7 +337,7 @@ hipError_t launch_mix_xielu(int dt, const void* in, uint32_t ld, const void* act
                             hipStream_t s) {
     const uint32_t es = dt == kFP32 ? 4u : 2u;
     const bool vec = n % 4u == 0 && ld % 4u == 0 && (uintptr_t)in % (4 * es) == 0 && (uintptr_t)out % (4 * es) == 0;
-    const uint32_t per = vec ? 1024u : 256u, gy = (n + per - 1u) / per;
+    const uint32_t per = vec ? 4096u : 256u, gy = (n + per - 1u) / per;
     const dim3 grid(rows, gy < 16u ? gy : 16u), block(256);
     if (dt == kBF16) {
         if (vec) hipLaunchKernelGGL((mix_xielu_kernel<kBF16, true>), grid, block, 0, s, in, ld, act, out, n);
@@ -345,13 +370,88 @@ __global__ __launch_bounds__(1024) void group_norm_gate_kernel(const float* __re
     }
 }
 
+// Groups of at most 64 EP elements: a wave each, EP neighbouring elements per lane.
+template <int DT, int EP>
+__global__ __launch_bounds__(256) void group_norm_gate_wave_kernel(const float* __restrict__ o, const void* __restrict__ gate,
+                                                                   const uint32_t ld, const void* __restrict__ weight,
+                                                                   void* __restrict__ out, const uint32_t rows, const uint32_t groups,
+                                                                   const uint32_t n, const float eps, const int kind) {
+    using E = Elem<DT>;
+    const uint32_t lane = threadIdx.x & 63u, at = blockIdx.x * 4u + (threadIdx.x >> 6), r = at / groups, g = at - r * groups;
+    if (r >= rows) return;
+    const uint32_t i0 = lane * (uint32_t)EP;
+    const size_t base = ((size_t)r * groups + g) * n, gbase = (size_t)r * ld + (size_t)g * n;
+    float x[EP], z[EP], w[EP], ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < EP; ++e) {
+        const bool ok = i0 + e < n;
+        const uint32_t i = ok ? i0 + e : 0u;
+        x[e] = o[base + i];
+        z[e] = E::load(gate, gbase + i);
+        w[e] = E::load(weight, i);
+        ss += ok ? x[e] * x[e] : 0.f;
+    }
+    const float rs = 1.f / sqrtf(wave_sum(ss) / (float)n + eps);
+#pragma unroll
+    for (int e = 0; e < EP; ++e)
+        if (i0 + e < n) E::store(out, base + i0 + e, x[e] * rs * w[e] * (kind == DECDEC_GATE_SILU ? silu_f(z[e]) : sigmoid_f(z[e])));
+}
+
+// Longer groups: a workgroup each, four neighbouring elements per thread and pass.
+template <int DT, int PASSES>
+__global__ __launch_bounds__(1024) void group_norm_gate_vec_kernel(const float* __restrict__ o, const void* __restrict__ gate,
+                                                                   const uint32_t ld, const void* __restrict__ weight,
+                                                                   void* __restrict__ out, const uint32_t n, const float eps, const int kind) {
+    __shared__ float red[17];
+    const uint32_t tid = threadIdx.x;
+    const size_t base = ((size_t)blockIdx.x * gridDim.y + blockIdx.y) * n, gbase = (size_t)blockIdx.x * ld + (size_t)blockIdx.y * n;
+    float x[PASSES][4], z[PASSES][4], w[PASSES][4], ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < PASSES; ++k) {
+        const uint32_t i = 4u * (tid + (uint32_t)k * blockDim.x), ic = i < n ? i : 0u;
+        load4<kFP32>(o, base + ic, x[k]);
+        load4<DT>(gate, gbase + ic, z[k]);
+        load4<DT>(weight, ic, w[k]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss += i < n ? x[k][e] * x[k][e] : 0.f;
+    }
+    const float rs = 1.f / sqrtf(block_sum(ss, red) / (float)n + eps);
+#pragma unroll
+    for (int k = 0; k < PASSES; ++k) {
+        const uint32_t i = 4u * (tid + (uint32_t)k * blockDim.x);
+        if (i < n) {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) x[k][e] *= rs * w[k][e] * (kind == DECDEC_GATE_SILU ? silu_f(z[k][e]) : sigmoid_f(z[k][e]));
+            store4<DT>(out, base + i, x[k]);
+        }
+    }
+}
+
+template <int DT>
+static hipError_t group_norm_dt(const float* o, const void* gate, uint32_t ld, const void* weight, void* out, uint32_t rows,
+                                uint32_t groups, uint32_t n, float eps, int kind, hipStream_t s) {
+    const uint32_t es = Elem<DT>::bytes, waves = rows * groups;
+    if (n <= 128u) hipLaunchKernelGGL((group_norm_gate_wave_kernel<DT, 2>), dim3((waves + 3u) / 4u), dim3(256), 0, s, o, gate, ld, weight, out, rows, groups, n, eps, kind);
+    else if (n <= 256u) hipLaunchKernelGGL((group_norm_gate_wave_kernel<DT, 4>), dim3((waves + 3u) / 4u), dim3(256), 0, s, o, gate, ld, weight, out, rows, groups, n, eps, kind);
+    else {
+        uint32_t threads = 64;
+        const bool vec = n % 4u == 0 && ld % 4u == 0 && n <= 16384u && (uintptr_t)o % 16u == 0 &&
+                         ((uintptr_t)gate | (uintptr_t)weight | (uintptr_t)out) % (4u * es) == 0;
+        const uint32_t want = vec ? (n + 3u) / 4u : n;
+        while (threads < 1024u && threads < want) threads *= 2;
+        const dim3 grid(rows, groups), block(threads);
+        if (!vec) hipLaunchKernelGGL((group_norm_gate_kernel<DT>), grid, block, 0, s, o, gate, ld, weight, out, n, eps, kind);
+        else if (want <= threads) hipLaunchKernelGGL((group_norm_gate_vec_kernel<DT, 1>), grid, block, 0, s, o, gate, ld, weight, out, n, eps, kind);
+        else if (want <= 2u * threads) hipLaunchKernelGGL((group_norm_gate_vec_kernel<DT, 2>), grid, block, 0, s, o, gate, ld, weight, out, n, eps, kind);
+        else hipLaunchKernelGGL((group_norm_gate_vec_kernel<DT, 4>), grid, block, 0, s, o, gate, ld, weight, out, n, eps, kind);
+    }
+    return hipGetLastError();
+}
+
 hipError_t launch_mix_group_norm_gate(int dt, const float* o, const void* gate, uint32_t ld, const void* weight, void* out,
                                       uint32_t rows, uint32_t groups, uint32_t n, float eps, int kind, hipStream_t s) {
-    uint32_t threads = 64;
-    while (threads < 1024u && threads < n) threads *= 2;
-    if (dt == kBF16) hipLaunchKernelGGL((group_norm_gate_kernel<kBF16>), dim3(rows, groups), dim3(threads), 0, s, o, gate, ld, weight, out, n, eps, kind);
-    else hipLaunchKernelGGL((group_norm_gate_kernel<kFP32>), dim3(rows, groups), dim3(threads), 0, s, o, gate, ld, weight, out, n, eps, kind);
-    return hipGetLastError();
+    return dt == kBF16 ? group_norm_dt<kBF16>(o, gate, ld, weight, out, rows, groups, n, eps, kind, s)
+                       : group_norm_dt<kFP32>(o, gate, ld, weight, out, rows, groups, n, eps, kind, s);
 }
 
 }  // namespace decdec

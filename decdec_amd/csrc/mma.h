@@ -54,14 +54,19 @@ __device__ __forceinline__ Frag<kBF16> frag_gather(const uint16_t* p, uint32_t s
         f.v[i] = (uint32_t)p[(size_t)(2 * i) * stride] | ((uint32_t)p[(size_t)(2 * i + 1) * stride] << 16);
     return f;
 }
+__device__ __forceinline__ uint32_t pack_bf16(float a, float b) {
+    const bf16x2_t v = {(__bf16)a, (__bf16)b};
+    uint32_t r;
+    __builtin_memcpy(&r, &v, 4);
+    return r;
+}
 // fp32 values as operands: exact for fp32; for bf16 the sum of a leading and a trailing part (16 significant bits)
 __device__ __forceinline__ void frag_split(const float (&x)[8], Frag<kBF16>& hi, Frag<kBF16>& lo) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-        const uint32_t h0 = f32_to_bf16_bits(x[2 * i]), h1 = f32_to_bf16_bits(x[2 * i + 1]);
-        hi.v[i] = h0 | (h1 << 16);
-        lo.v[i] = (uint32_t)f32_to_bf16_bits(x[2 * i] - __uint_as_float(h0 << 16)) |
-                  ((uint32_t)f32_to_bf16_bits(x[2 * i + 1] - __uint_as_float(h1 << 16)) << 16);
+        const uint32_t h = pack_bf16(x[2 * i], x[2 * i + 1]);
+        hi.v[i] = h;
+        lo.v[i] = pack_bf16(x[2 * i] - __uint_as_float(h << 16), x[2 * i + 1] - __uint_as_float(h & 0xFFFF0000u));
     }
 }
 __device__ __forceinline__ void frag_split(const float (&x)[8], Frag<kFP32>& hi, Frag<kFP32>&) {
@@ -72,12 +77,25 @@ __device__ __forceinline__ void frag_split(const float (&x)[8], Frag<kFP32>& hi,
 template <int DT> struct LaneOf { using t = uint16_t; };
 template <> struct LaneOf<kFP32> { using t = float; };
 
+constexpr float kLog2e = 1.4426950408889634f;
+
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + __expf(-z)); }
 __device__ __forceinline__ float silu_f(float z) { return z * sigmoid_f(z); }
 __device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
-// xIELU with the softplus of its two numbers already taken
+// xIELU with the softplus of its two numbers already taken.  e^z - 1 - z by its series where the difference cancels.
 __device__ __forceinline__ float xielu_f(float z, float sp, float sq) {
-    return z > 0.f ? (sp * z + 0.5f) * z : (0.5f + sq) * (expm1f(z) - z) + 0.5f * z;
+    const float n = fminf(z, 0.f);
+    float s = 2.7557319e-7f;                               // 1 / 10!
+    s = __builtin_fmaf(s, n, 2.7557319e-6f);
+    s = __builtin_fmaf(s, n, 2.4801587e-5f);
+    s = __builtin_fmaf(s, n, 1.9841270e-4f);
+    s = __builtin_fmaf(s, n, 1.3888889e-3f);
+    s = __builtin_fmaf(s, n, 8.3333333e-3f);
+    s = __builtin_fmaf(s, n, 4.1666667e-2f);
+    s = __builtin_fmaf(s, n, 1.6666667e-1f);
+    s = __builtin_fmaf(s, n, 0.5f) * n * n;
+    const float e = n > -0.7f ? s : __expf(n) - 1.f - n;
+    return z > 0.f ? (sp * z + 0.5f) * z : (0.5f + sq) * e + 0.5f * z;
 }
 
 // Sum over a workgroup of `blockDim.x` (a multiple of 64) threads; red: at least 17 floats of LDS, free at the call.
