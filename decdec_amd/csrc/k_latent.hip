@@ -42,6 +42,19 @@ __device__ __forceinline__ void frag_values(const Frag<kFP32>& f, float (&x)[8])
     for (int i = 0; i < 8; ++i) x[i] = f.v[i];
 }
 
+__device__ __forceinline__ Frag<kBF16> frag_of(const float (&x)[8], const Frag<kBF16>&) {
+    Frag<kBF16> f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) f.v[i] = pack_bf16(x[2 * i], x[2 * i + 1]);
+    return f;
+}
+__device__ __forceinline__ Frag<kFP32> frag_of(const float (&x)[8], const Frag<kFP32>&) {
+    Frag<kFP32> f;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) f.v[i] = x[i];
+    return f;
+}
+
 // The new cache row of one token (a whole workgroup): normed latent, rotated shared key part.
 template <int DT>
 __device__ __forceinline__ void append_row(const decdec_latent& p, const void* proj, size_t row, long long pos, float* red) {
@@ -71,6 +84,29 @@ __global__ __launch_bounds__(256) void latent_append_kernel(const decdec_latent 
     const size_t row = (size_t)t * p.ld;
     append_row<DT>(p, p.proj, row, pos, red);
     const size_t trow = (size_t)(pos < 0 ? 0 : (pos < (long long)p.max_seq ? pos : (long long)p.max_seq - 1)) * half;
+    const bool wide = p.dim % 8u == 0 && p.rot % 8u == 0 && p.ld % 8u == 0 && p.off_q % 8u == 0 && ((uintptr_t)p.proj | (uintptr_t)q_out) % 16u == 0;
+    if (wide) {                                            // eight neighbouring elements: four pairs, or none to turn
+        using T = typename LaneOf<DT>::t;
+        const T* src = (const T*)p.proj + row + p.off_q;
+        for (uint32_t i = threadIdx.x; i < p.heads * (Dq / 8u); i += 256u) {
+            const uint32_t e = 8u * (i % (Dq / 8u));
+            Frag<DT> f = frag_load(src + 8u * i);
+            if (e >= p.dim) {
+                float x[8];
+                frag_values(f, x);
+#pragma unroll
+                for (uint32_t j = 0; j < 4u; ++j) {
+                    const size_t at = trow + (e - p.dim) / 2u + j;
+                    const float c = p.cos_table[at], s = p.sin_table[at], u = x[2 * j], v = x[2 * j + 1];
+                    x[2 * j] = u * c - v * s;
+                    x[2 * j + 1] = v * c + u * s;
+                }
+                f = frag_of(x, f);
+            }
+            store8((T*)q_out + (size_t)t * p.heads * Dq + 8u * i, f);
+        }
+        return;
+    }
     for (uint32_t i = threadIdx.x; i < p.heads * (Dq / 2u); i += 256u) {
         const uint32_t h = i / (Dq / 2u), e = 2u * (i % (Dq / 2u));
         const size_t at = (size_t)t * p.heads * Dq + h * Dq + e;
@@ -367,8 +403,8 @@ __host__ __device__ inline StepSplit step_split(uint32_t len, uint32_t max_split
     return {(tiles + per - 1u) / per, per * 64u};
 }
 static uint32_t step_max_splits(const decdec_latent& p) {
-    const uint32_t groups = (p.heads + 15u) / 16u, want = 128u / groups, tiles = (p.max_seq + 63u) / 64u;
-    const uint32_t n = want < 8u ? 8u : (want > 64u ? 64u : want);
+    const uint32_t groups = (p.heads + 15u) / 16u, want = 256u / groups, tiles = (p.max_seq + 63u) / 64u;
+    const uint32_t n = want < 8u ? 8u : (want > 128u ? 128u : want);
     return n < tiles ? n : tiles;
 }
 
@@ -419,7 +455,18 @@ __global__ __launch_bounds__(kStepThreads) void latent_step_kernel(const decdec_
         const uint32_t r = i / W8, c = (i - r * W8) * 8u;
         float x[8];
 #pragma unroll
-        for (uint32_t e = 0; e < 8u; ++e) x[e] = (h0 + r < p.heads && c + e < W) ? qa[(size_t)(h0 + r) * W + c + e] : 0.f;
+        for (uint32_t e = 0; e < 8u; ++e) x[e] = 0.f;
+        if (h0 + r < p.heads) {
+            const float* src = qa + (size_t)(h0 + r) * W + c;
+            if (vec && c + 8u <= W) {
+                const f32x4 a = *(const f32x4*)src, b = *(const f32x4*)(src + 4);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) { x[e] = a[e]; x[4 + e] = b[e]; }
+            } else {
+#pragma unroll
+                for (uint32_t e = 0; e < 8u; ++e) x[e] = c + e < W ? src[e] : 0.f;
+            }
+        }
         Frag<DT> hi, lo;
         frag_split(x, hi, lo);
         store8(Ql + r * KL + c, hi);
@@ -515,12 +562,12 @@ __global__ __launch_bounds__(1024) void latent_merge_kernel(const decdec_latent 
                                                             void* __restrict__ out, const uint32_t max_splits) {
     using E = Elem<DT>;
     using T = typename LaneOf<DT>::t;
-    __shared__ float lat[1024], share[1024], ws[64];
+    __shared__ float lat[1024], share[1024], ws[128];
     const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, h = blockIdx.x, R = p.rank, V = p.vdim;
     const long long pos = *p.pos;
     if (pos < 0) return;
     const uint32_t len = pos + 1 < (long long)p.max_seq ? (uint32_t)pos + 1u : p.max_seq;
-    const uint32_t n = step_split(len, max_splits).splits;               // at most 64
+    const uint32_t n = step_split(len, max_splits).splits;               // at most 128
     const float* ph = parts + (size_t)h * (R + 2u);
     const size_t ps = (size_t)p.heads * (R + 2u);
     const bool vec = R % 8u == 0;
@@ -537,13 +584,21 @@ __global__ __launch_bounds__(1024) void latent_merge_kernel(const decdec_latent 
     const bool mine = g < groups && r < R;
     if (wave == 0u) {
         const float sink = p.sink != nullptr ? E::load(p.sink, h) : -__builtin_inff();
-        const float m = lane < n ? ph[lane * ps + R] : -__builtin_inff(), l = lane < n ? ph[lane * ps + R + 1u] : 0.f;
-        float M = fmaxf(m, sink);
+        float m[2], l[2], M = sink;
+#pragma unroll
+        for (uint32_t e = 0; e < 2u; ++e) {
+            const uint32_t i = lane + 64u * e;
+            m[e] = i < n ? ph[i * ps + R] : -__builtin_inff();
+            l[e] = i < n ? ph[i * ps + R + 1u] : 0.f;
+            M = fmaxf(M, m[e]);
+        }
 #pragma unroll
         for (int off = 32; off >= 1; off >>= 1) M = fmaxf(M, __shfl_xor(M, off, 64));
-        const float w = lane < n ? __expf(m - M) : 0.f;
-        const float L = wave_sum(w * l) + (p.sink != nullptr ? __expf(sink - M) : 0.f);
-        ws[lane] = w / L;
+#pragma unroll
+        for (int e = 0; e < 2; ++e) m[e] = __expf(m[e] - M);               // exp(-inf) = 0 past the last split
+        const float L = wave_sum(m[0] * l[0] + m[1] * l[1]) + (p.sink != nullptr ? __expf(sink - M) : 0.f);
+        ws[lane] = m[0] / L;
+        ws[lane + 64u] = m[1] / L;
     }
     __syncthreads();
     float t = 0.f;

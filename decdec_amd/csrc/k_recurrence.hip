@@ -30,7 +30,7 @@ __global__ __launch_bounds__(1024) void recurrence_step_kernel(const decdec_recu
                                                                void* __restrict__ out, const void* __restrict__ norm_weight,
                                                                const float eps, const int kind, const uint32_t cw) {
     using E = Elem<DT>;
-    __shared__ float qs[512], ks[512], red[17], pa[1024], pb[1024];
+    __shared__ float qs[512], ks[512], red[32], pa[1024], pb[1024];
     const uint32_t tid = threadIdx.x, h = blockIdx.x, kg = tid / cw, KG = blockDim.x / cw;
     const uint32_t D = p.dim, V = p.vdim, col = blockIdx.y * cw + tid % cw;
     const bool live = col < V;
@@ -89,8 +89,7 @@ __global__ __launch_bounds__(1024) void recurrence_step_kernel(const decdec_recu
         if (live) v = conv(p.off_v + h * V + col, 2u * qk + h * V + col, p.conv_v, h * V + col, kg == 0u);
         g = expf(log_decay<DT>(p, p.proj, 0, h));
         beta = sigmoid_f(E::load(p.proj, p.off_b + h));
-        sq = block_sum(sq, red);
-        sk = block_sum(sk, red);
+        block_sum2(sq, sk, red);
         const float rq = 1.f / sqrtf(sq + 1e-6f) / sqrtf((float)D), rk = 1.f / sqrtf(sk + 1e-6f);
         for (uint32_t i = tid; i < D; i += blockDim.x) { qs[i] *= rq; ks[i] *= rk; }
     }
@@ -240,8 +239,9 @@ __global__ __launch_bounds__(256) void delta_inputs_kernel(const decdec_recurren
     }
 }
 
-// The same for at most TAPS taps and widths that are multiples of four: a workgroup takes eight tokens, a thread four
-// neighbouring channels, whose inputs (and the taps before them) are all requested at once.
+// The same for at most TAPS taps and widths that are multiples of four: a workgroup takes eight tokens and a group of query
+// and key heads or 1024 value channels (grid.y counts the groups), a thread four neighbouring channels, whose inputs (and
+// the taps before them) are all requested at once.
 constexpr uint32_t kInputRows = 8;
 
 template <int DT>
@@ -294,8 +294,9 @@ __global__ __launch_bounds__(256) void delta_inputs_quad_kernel(const decdec_rec
     auto put = [&](float* dst, uint32_t t, uint32_t width, uint32_t c, const float (&y)[4], float r) {
         if (t0 + t < rows) *(f32x4*)(dst + (size_t)(t0 + t) * width + c) = f32x4{y[0] * r, y[1] * r, y[2] * r, y[3] * r};
     };
-    const uint32_t c4 = (tid % gl) * 4u;                                   // gl threads share a head
-    for (uint32_t j = tid / gl; j < (2u * p.kv_heads + 256u / gl - 1u) / (256u / gl) * (256u / gl); j += 256u / gl) {
+    const uint32_t per = 256u / gl, hgroups = (2u * p.kv_heads + per - 1u) / per;   // gl threads share a head
+    if (blockIdx.y < hgroups) {
+        const uint32_t j = blockIdx.y * per + tid / gl, c4 = (tid % gl) * 4u;
         const bool isq = j < p.kv_heads, live = j < 2u * p.kv_heads && c4 < D;
         const uint32_t ch = live ? (isq ? j : j - p.kv_heads) * D + c4 : 0u;
         float y[N][4];
@@ -308,18 +309,22 @@ __global__ __launch_bounds__(256) void delta_inputs_quad_kernel(const decdec_rec
             if (isq) r /= sqrtf((float)D);
             if (live) put(isq ? q : k, (uint32_t)t, nqk, ch, y[t], r);
         }
-    }
-    for (uint32_t c = 4u * tid; c < nv; c += 1024u) {
-        float y[N][4];
-        conv(p.off_v, 2u * nqk + c, p.conv_v, c, y);
+    } else {
+        const uint32_t c = 1024u * (blockIdx.y - hgroups) + 4u * tid;
+        if (c < nv) {
+            float y[N][4];
+            conv(p.off_v, 2u * nqk + c, p.conv_v, c, y);
 #pragma unroll
-        for (int t = 0; t < N; ++t) put(v, (uint32_t)t, nv, c, y[t], 1.f);
+            for (int t = 0; t < N; ++t) put(v, (uint32_t)t, nv, c, y[t], 1.f);
+        }
     }
-    for (uint32_t i = tid; i < p.heads * kInputRows; i += 256u) {
-        const uint32_t t = t0 + i / p.heads, h = i % p.heads;
-        if (t < rows) {
-            lg[(size_t)t * p.heads + h] = log_decay<DT>(p, p.proj, (size_t)t * p.ld, h);
-            beta[(size_t)t * p.heads + h] = sigmoid_f(E::load(p.proj, (size_t)t * p.ld + p.off_b + h));
+    if (blockIdx.y + 1u == gridDim.y) {
+        for (uint32_t i = tid; i < p.heads * kInputRows; i += 256u) {
+            const uint32_t t = t0 + i / p.heads, h = i % p.heads;
+            if (t < rows) {
+                lg[(size_t)t * p.heads + h] = log_decay<DT>(p, p.proj, (size_t)t * p.ld, h);
+                beta[(size_t)t * p.heads + h] = sigmoid_f(E::load(p.proj, (size_t)t * p.ld + p.off_b + h));
+            }
         }
     }
 }
@@ -361,15 +366,16 @@ __device__ __forceinline__ Frag<kFP32> row_frag(const float* p, int valid, bool 
 // 64 rows x 32 columns of an array of rows (stride ld), requested into registers and later put into LDS [64][36]; rows past
 // n and columns past D are zero.
 struct Slice { f32x4 x[2]; };
+template <bool FULL>                                       // D is a multiple of 32
 __device__ __forceinline__ Slice slice_fetch(const float* src, size_t ld, uint32_t n, uint32_t c0, uint32_t D, bool vec) {
     Slice s;
 #pragma unroll
     for (uint32_t e = 0; e < 2; ++e) {
         const uint32_t i = threadIdx.x + 256u * e, r = i >> 3, c = c0 + (i & 7u) * 4u;
         const float* row = src + (size_t)(r < n ? r : 0u) * ld;
-        if (vec) {                                         // D is a multiple of four
-            s.x[e] = *(const f32x4*)(row + (c < D ? c : 0u));
-            if (r >= n || c >= D) s.x[e] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (FULL || vec) {                                 // D is a multiple of four
+            s.x[e] = *(const f32x4*)(row + (FULL || c < D ? c : 0u));
+            if (r >= n || (!FULL && c >= D)) s.x[e] = f32x4{0.f, 0.f, 0.f, 0.f};
         } else {
 #pragma unroll
             for (int j = 0; j < 4; ++j) s.x[e][j] = (r < n && c + (uint32_t)j < D) ? row[c + j] : 0.f;
@@ -386,12 +392,13 @@ __device__ __forceinline__ void slice_put(const Slice& s, float (*dst)[36]) {
 }
 
 // U and W of a chunk: grid (chunks, heads).
+template <bool FULL>
 __global__ __launch_bounds__(256) void delta_solve_kernel(const ChunkParams p) {
     __shared__ __align__(16) float Ks[C][36];
     __shared__ __align__(16) float A[C][C + 4];
     __shared__ __align__(16) float T[C][20];                // inverses of the diagonal blocks
     __shared__ double G[C];
-    __shared__ float beta[C];
+    __shared__ float beta[C], bg[C];
     const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, h = blockIdx.y, kvh = h / (p.heads / p.kv_heads);
     const uint32_t t0 = blockIdx.x * C, n = p.rows - t0 < C ? p.rows - t0 : C, D = p.dim, V = p.vdim;
     const float* k = p.k + ((size_t)t0 * p.kv_heads + kvh) * D;
@@ -400,16 +407,17 @@ __global__ __launch_bounds__(256) void delta_solve_kernel(const ChunkParams p) {
     if (wave == 0) {
         chunk_log_decay(p, t0, n, h, G);
         beta[lane] = lane < n ? p.beta[(size_t)(t0 + lane) * p.heads + h] : 0.f;
+        bg[lane] = beta[lane] * expf((float)G[lane]);
     }
     f32x4 acc[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-    Slice ks = slice_fetch(k, kld, n, 0u, D, vec);
+    Slice ks = slice_fetch<FULL>(k, kld, n, 0u, D, vec);
     for (uint32_t c0 = 0; c0 < D; c0 += 32u) {
         __syncthreads();
         slice_put(ks, Ks);
         __syncthreads();
-        if (c0 + 32u < D) ks = slice_fetch(k, kld, n, c0 + 32u, D, vec);
+        if (c0 + 32u < D) ks = slice_fetch<FULL>(k, kld, n, c0 + 32u, D, vec);
         const Frag<kFP32> a = frag_load(&Ks[16u * wave + (lane & 15u)][8u * (lane >> 4)]);
 #pragma unroll
         for (int j = 0; j < 4; ++j) mma(a, frag_load(&Ks[16u * j + (lane & 15u)][8u * (lane >> 4)]), acc[j]);
@@ -441,7 +449,7 @@ __global__ __launch_bounds__(256) void delta_solve_kernel(const ChunkParams p) {
     const uint32_t l16 = lane & 15u, lg = lane >> 4;
     for (uint32_t c0 = 16u * wave; c0 < V + D; c0 += 64u) {
         const uint32_t c = c0 + l16;
-        const bool isv = c < V, live = c < V + D;
+        const bool isv = c < V, live = FULL || c < V + D;
         const float* src = isv ? p.v + ((size_t)t0 * p.heads + h) * V + c : k + (live ? c - V : 0u);
         const size_t ld = isv ? (size_t)p.heads * V : kld;
         float* dst = isv ? p.u + ((size_t)t0 * p.heads + h) * V + c : p.w + ((size_t)t0 * p.heads + h) * D + (live ? c - V : 0u);
@@ -452,9 +460,14 @@ __global__ __launch_bounds__(256) void delta_solve_kernel(const ChunkParams p) {
 #pragma unroll
             for (uint32_t v = 0; v < 4u; ++v) {
                 const uint32_t i = 16u * b + 4u * lg + v;
-                float y = (live && i < n) ? src[(size_t)i * ld] * beta[i] : 0.f;
-                if (!isv) y *= expf((float)G[i]);
-                x[b][v] = y;
+                x[b][v] = live ? src[(size_t)(i < n ? i : 0u) * ld] : 0.f;
+            }
+#pragma unroll
+        for (uint32_t b = 0; b < 4u; ++b)
+#pragma unroll
+            for (uint32_t v = 0; v < 4u; ++v) {
+                const uint32_t i = 16u * b + 4u * lg + v;
+                x[b][v] *= isv ? beta[i] : bg[i];                          // zero past the chunk's last token
             }
 #pragma unroll
         for (uint32_t b = 0; b < 4u; ++b) {
@@ -482,18 +495,19 @@ __global__ __launch_bounds__(256) void delta_solve_kernel(const ChunkParams p) {
 
 // States: grid (heads, vdim / 16), one walk over the chunks.  Wave w owns the state's row tiles w, w + 4, ... (NT of them).
 // What the next chunk needs from memory is requested as soon as this chunk's copy has been used.
-template <bool DELTA, int NT>
+// FULL: dim is 64 NT and vdim a multiple of 16.
+template <bool DELTA, int NT, bool FULL>
 __global__ __launch_bounds__(256) void chunk_state_kernel(const ChunkParams p, const uint32_t chunks) {
     extern __shared__ __align__(16) float lds[];
     __shared__ double G[C];
     __shared__ __align__(16) float Vl[C][20];
     __shared__ float pw[C + 1];
     const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, l16 = lane & 15u, lg = lane >> 4;
-    const uint32_t h = blockIdx.x, kvh = h / (p.heads / p.kv_heads), D = p.dim, V = p.vdim, v0 = blockIdx.y * 16u;
+    const uint32_t h = blockIdx.x, kvh = h / (p.heads / p.kv_heads), D = FULL ? 64u * NT : p.dim, V = p.vdim, v0 = blockIdx.y * 16u;
     const uint32_t Dp = (D + 31u) & ~31u, KL = Dp + 4u, tiles = Dp / 16u;
     float* Kl = lds;                        // [C][KL]
     float* Sl = lds + C * KL;               // [Dp][20]
-    const bool fresh = *p.pos <= 0, vec = D % 4u == 0, vec8 = D % 8u == 0, col = v0 + l16 < V;
+    const bool fresh = *p.pos <= 0, vec = FULL || D % 4u == 0, vec8 = FULL || D % 8u == 0, col = FULL || v0 + l16 < V;
     float* S = p.state + (size_t)h * D * V + v0 + l16;
     if constexpr (!DELTA) { for (uint32_t i = tid; i <= C; i += 256u) pw[i] = p.decay[(size_t)h * 65u + i]; }
     f32x4 s[NT];
@@ -502,7 +516,7 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(const ChunkParams p, c
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
             const uint32_t r = 16u * (wave + 4u * (uint32_t)i) + 4u * lg + (uint32_t)v;
-            s[i][v] = (r < D && col && !fresh) ? S[(size_t)r * V] : 0.f;
+            s[i][v] = ((FULL || (r < D && col)) && !fresh) ? S[(size_t)r * V] : 0.f;
         }
     const uint32_t kr = tid >> 2, kc = (tid & 3u) * 4u;                    // a thread's row of the keys, and columns kc + 16 j
     f32x4 kreg[4 * NT];
@@ -515,8 +529,8 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(const ChunkParams p, c
         for (int j = 0; j < 4 * NT; ++j) {
             const uint32_t c = kc + 16u * (uint32_t)j;
             if (vec) {
-                kreg[j] = *(const f32x4*)(k + (c < D ? c : 0u));
-                if (kr >= n || c >= D) kreg[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+                kreg[j] = *(const f32x4*)(k + (FULL || c < D ? c : 0u));
+                if (kr >= n || (!FULL && c >= D)) kreg[j] = f32x4{0.f, 0.f, 0.f, 0.f};
             } else {
 #pragma unroll
                 for (int e = 0; e < 4; ++e) kreg[j][e] = (kr < n && c + (uint32_t)e < D) ? k[c + e] : 0.f;
@@ -531,7 +545,7 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(const ChunkParams p, c
 #pragma unroll
             for (int j = 0; j < 2 * NT; ++j) {
                 const uint32_t kk = 32u * (uint32_t)j + 8u * lg;
-                wreg[j] = row_frag(w + kk, ar < n ? (int)D - (int)kk : 0, vec8);
+                wreg[j] = FULL ? frag_load(w + kk) : row_frag(w + kk, ar < n ? (int)D - (int)kk : 0, vec8);   // rows past n write nothing
             }
         }
 #pragma unroll
@@ -547,7 +561,7 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(const ChunkParams p, c
         const uint32_t t0 = ch * C, n = p.rows - t0 < C ? p.rows - t0 : C;
 #pragma unroll
         for (int j = 0; j < 4 * NT; ++j)
-            if (kc + 16u * (uint32_t)j < Dp) *(f32x4*)&Kl[kr * KL + kc + 16u * (uint32_t)j] = kreg[j];
+            if (FULL || kc + 16u * (uint32_t)j < Dp) *(f32x4*)&Kl[kr * KL + kc + 16u * (uint32_t)j] = kreg[j];
         if constexpr (DELTA) {
             if (wave == 3u) {                                              // log-decays summed up, in double
                 double x = (double)lreg;
@@ -565,8 +579,8 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(const ChunkParams p, c
 #pragma unroll
             for (int v = 0; v < 4; ++v) {
                 const uint32_t r = 16u * (wave + 4u * (uint32_t)i) + 4u * lg + (uint32_t)v;
-                if (r < Dp) Sl[r * 20u + l16] = s[i][v];
-                if (r < D && col) st[(size_t)r * V] = s[i][v];
+                if (FULL || r < Dp) Sl[r * 20u + l16] = s[i][v];
+                if (FULL || (r < D && col)) st[(size_t)r * V] = s[i][v];
             }
         __syncthreads();
         if (ch + 1u < chunks) request_keys(t0 + C);
@@ -577,7 +591,7 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(const ChunkParams p, c
             if constexpr (DELTA) {
 #pragma unroll
                 for (int j = 0; j < 2 * NT; ++j)
-                    if (32u * (uint32_t)j < D) mma(wreg[j], frag_gather(Sl + (32u * (uint32_t)j + 8u * lg) * 20u + l16, 20u), acc);
+                    if (FULL || 32u * (uint32_t)j < D) mma(wreg[j], frag_gather(Sl + (32u * (uint32_t)j + 8u * lg) * 20u + l16, 20u), acc);
             }
 #pragma unroll
             for (int v = 0; v < 4; ++v) {
@@ -601,7 +615,7 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(const ChunkParams p, c
         for (int i = 0; i < NT; ++i) {
             const uint32_t tile = wave + 4u * (uint32_t)i;
             s[i] *= gend;
-            if (tile < tiles) {
+            if (FULL || tile < tiles) {
 #pragma unroll
                 for (uint32_t j0 = 0; j0 < C; j0 += 32u)
                     mma(frag_gather(Kl + (j0 + 8u * lg) * KL + 16u * tile + l16, KL), frag_gather(&Vl[j0 + 8u * lg][l16], 20u), s[i]);
@@ -614,12 +628,12 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(const ChunkParams p, c
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
             const uint32_t r = 16u * (wave + 4u * (uint32_t)i) + 4u * lg + (uint32_t)v;
-            if (r < D && col) S[(size_t)r * V] = s[i][v];
+            if (FULL || (r < D && col)) S[(size_t)r * V] = s[i][v];
         }
 }
 
-// Read-out: grid (chunks, heads, vdim / 64).
-template <bool DELTA>
+// Read-out: grid (chunks, heads, vdim / 64).  FULL: dim is a multiple of 32 and vdim of 64.
+template <bool DELTA, bool FULL>
 __global__ __launch_bounds__(256) void chunk_output_kernel(const ChunkParams p) {
     __shared__ __align__(16) float Qs[C][36];
     __shared__ __align__(16) float Ks[C][36];
@@ -640,13 +654,13 @@ __global__ __launch_bounds__(256) void chunk_output_kernel(const ChunkParams p) 
     if constexpr (DELTA) { if (wave == 0) chunk_log_decay(p, t0, n, h, G); }
     else { for (uint32_t i = tid; i <= C; i += 256u) pw[i] = p.decay[(size_t)h * 65u + i]; }
     // four neighbouring columns of a 64-column array per thread and pass, 16 rows a pass
-    const bool vecv = V % 4u == 0;
+    const bool vecv = FULL || V % 4u == 0;
     const uint32_t vr = tid >> 4, vc = (tid & 15u) * 4u;
     auto value4 = [&](const float* row, bool in) {
         f32x4 x = {0.f, 0.f, 0.f, 0.f};
         if (vecv) {
-            x = *(const f32x4*)(row + (v0 + vc < V ? v0 + vc : 0u));
-            if (!in || v0 + vc >= V) x = f32x4{0.f, 0.f, 0.f, 0.f};
+            x = *(const f32x4*)(row + (FULL || v0 + vc < V ? v0 + vc : 0u));
+            if (!in || (!FULL && v0 + vc >= V)) x = f32x4{0.f, 0.f, 0.f, 0.f};
         } else {
 #pragma unroll
             for (int e = 0; e < 4; ++e)
@@ -654,13 +668,13 @@ __global__ __launch_bounds__(256) void chunk_output_kernel(const ChunkParams p) 
         }
         return x;
     };
-    Slice qr = slice_fetch(q, kld, n, 0u, D, vec), kr = slice_fetch(k, kld, n, 0u, D, vec);
+    Slice qr = slice_fetch<FULL>(q, kld, n, 0u, D, vec), kr = slice_fetch<FULL>(k, kld, n, 0u, D, vec);
     f32x4 sr[2], val[4];
     auto fetch_state = [&](uint32_t c0) {
 #pragma unroll
         for (uint32_t e = 0; e < 2u; ++e) {
             const uint32_t r = c0 + vr + 16u * e;
-            sr[e] = value4(S + (size_t)(r < D ? r : 0u) * V, r < D);
+            sr[e] = value4(S + (size_t)(FULL || r < D ? r : 0u) * V, FULL || r < D);
         }
     };
     fetch_state(0u);
@@ -682,8 +696,8 @@ __global__ __launch_bounds__(256) void chunk_output_kernel(const ChunkParams p) 
         for (uint32_t e = 0; e < 2u; ++e) *(f32x4*)&Ss[vr + 16u * e][vc] = sr[e];
         __syncthreads();
         if (c0 + 32u < D) {
-            qr = slice_fetch(q, kld, n, c0 + 32u, D, vec);
-            kr = slice_fetch(k, kld, n, c0 + 32u, D, vec);
+            qr = slice_fetch<FULL>(q, kld, n, c0 + 32u, D, vec);
+            kr = slice_fetch<FULL>(k, kld, n, c0 + 32u, D, vec);
             fetch_state(c0 + 32u);
         }
         const Frag<kFP32> a = frag_load(&Qs[16u * wave + l16][8u * lg]);
@@ -720,7 +734,7 @@ __global__ __launch_bounds__(256) void chunk_output_kernel(const ChunkParams p) 
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
             const uint32_t r = 16u * wave + 4u * lg + (uint32_t)v, c = v0 + 16u * (uint32_t)j + l16;
-            if (r < n && c < V) p.o[((size_t)(t0 + r) * p.heads + h) * V + c] = o[j][v];
+            if (r < n && (FULL || c < V)) p.o[((size_t)(t0 + r) * p.heads + h) * V + c] = o[j][v];
         }
 }
 
@@ -757,8 +771,13 @@ size_t recurrence_workspace(const decdec_recurrence& p, uint32_t rows) {
 
 template <bool DELTA, int NT>
 static hipError_t launch_state(const ChunkParams& c, uint32_t chunks, dim3 grid, size_t lds, hipStream_t s) {
-    if (hipError_t e = allow_lds<chunk_state_kernel<DELTA, NT>>(lds); e != hipSuccess) return e;
-    hipLaunchKernelGGL((chunk_state_kernel<DELTA, NT>), grid, dim3(256), lds, s, c, chunks);
+    if (c.dim == 64u * NT && c.vdim % 16u == 0) {
+        if (hipError_t e = allow_lds<chunk_state_kernel<DELTA, NT, true>>(lds); e != hipSuccess) return e;
+        hipLaunchKernelGGL((chunk_state_kernel<DELTA, NT, true>), grid, dim3(256), lds, s, c, chunks);
+    } else {
+        if (hipError_t e = allow_lds<chunk_state_kernel<DELTA, NT, false>>(lds); e != hipSuccess) return e;
+        hipLaunchKernelGGL((chunk_state_kernel<DELTA, NT, false>), grid, dim3(256), lds, s, c, chunks);
+    }
     return hipGetLastError();
 }
 
@@ -766,11 +785,12 @@ template <bool DELTA>
 static hipError_t launch_chunks(const ChunkParams& c, hipStream_t s) {
     const uint32_t chunks = (c.rows + C - 1u) / C, Dp = (c.dim + 31u) & ~31u, nt = (Dp / 16u + 3u) / 4u;
     const size_t lds = ((size_t)C * (Dp + 4u) + (size_t)Dp * 20u) * sizeof(float);
-    const dim3 grid(c.heads, (c.vdim + 15u) / 16u), block(256);
-    hipError_t e = nt == 1u ? launch_state<DELTA, 1>(c, chunks, grid, lds, s) : nt == 2u ? launch_state<DELTA, 2>(c, chunks, grid, lds, s)
-                 : nt <= 4u ? launch_state<DELTA, 4>(c, chunks, grid, lds, s) : hipErrorInvalidValue;
+    const dim3 grid(c.heads, (c.vdim + 15u) / 16u), ogrid(chunks, c.heads, (c.vdim + 63u) / 64u), block(256);
+    const hipError_t e = nt == 1u ? launch_state<DELTA, 1>(c, chunks, grid, lds, s) : nt == 2u ? launch_state<DELTA, 2>(c, chunks, grid, lds, s)
+                       : nt <= 4u ? launch_state<DELTA, 4>(c, chunks, grid, lds, s) : hipErrorInvalidValue;
     if (e != hipSuccess) return e;
-    hipLaunchKernelGGL((chunk_output_kernel<DELTA>), dim3(chunks, c.heads, (c.vdim + 63u) / 64u), block, 0, s, c);
+    if (c.dim % 32u == 0 && c.vdim % 64u == 0) hipLaunchKernelGGL((chunk_output_kernel<DELTA, true>), ogrid, block, 0, s, c);
+    else hipLaunchKernelGGL((chunk_output_kernel<DELTA, false>), ogrid, block, 0, s, c);
     return hipGetLastError();
 }
 
@@ -785,7 +805,8 @@ static hipError_t rows_dt(const decdec_recurrence& p, const ChunkParams& c, hipS
     while (4u * gl < p.dim) gl *= 2;
     const bool quads = ((p.dim | p.ld | p.off_q | p.off_k | p.off_v | (p.heads * p.vdim)) & 3u) == 0 && p.taps <= 8u &&
                        (uintptr_t)p.proj % (4u * es) == 0 && (uintptr_t)p.ring % (4u * es) == 0;
-    const dim3 wide((c.rows + kInputRows - 1u) / kInputRows);
+    const dim3 wide((c.rows + kInputRows - 1u) / kInputRows,
+                    (2u * p.kv_heads + 256u / gl - 1u) / (256u / gl) + (p.heads * p.vdim + 1023u) / 1024u);
     if (quads && p.taps <= 4u)
         hipLaunchKernelGGL((delta_inputs_quad_kernel<DT, 4>), wide, dim3(256), 0, s, p, (float*)c.q, (float*)c.k, (float*)c.v, (float*)c.lg, (float*)c.beta, c.rows, gl);
     else if (quads)
@@ -794,7 +815,9 @@ static hipError_t rows_dt(const decdec_recurrence& p, const ChunkParams& c, hipS
         hipLaunchKernelGGL((delta_inputs_kernel<DT>), dim3(c.rows), dim3(256), 0, s, p, (float*)c.q, (float*)c.k, (float*)c.v, (float*)c.lg, (float*)c.beta);
     const uint32_t chans = 2u * p.kv_heads * p.dim + p.heads * p.vdim, keep = c.rows < p.taps ? c.rows : p.taps;
     hipLaunchKernelGGL((ring_update_kernel<DT>), dim3((chans + 255u) / 256u, keep), dim3(256), 0, s, p, c.rows);
-    hipLaunchKernelGGL(delta_solve_kernel, dim3((c.rows + C - 1u) / C, p.heads), dim3(256), 0, s, c);
+    const dim3 sgrid((c.rows + C - 1u) / C, p.heads);
+    if (c.dim % 32u == 0 && c.vdim % 16u == 0) hipLaunchKernelGGL(delta_solve_kernel<true>, sgrid, dim3(256), 0, s, c);
+    else hipLaunchKernelGGL(delta_solve_kernel<false>, sgrid, dim3(256), 0, s, c);
     return launch_chunks<true>(c, s);
 }
 

@@ -370,8 +370,8 @@ __global__ __launch_bounds__(1024) void group_norm_gate_kernel(const float* __re
     }
 }
 
-// Groups of at most 64 EP elements: a wave each, EP neighbouring elements per lane.
-template <int DT, int EP>
+// Groups of at most 64 EP elements: a wave each, EP neighbouring elements per lane.  FULL: exactly 64 EP, aligned to EP.
+template <int DT, int EP, bool FULL>
 __global__ __launch_bounds__(256) void group_norm_gate_wave_kernel(const float* __restrict__ o, const void* __restrict__ gate,
                                                                    const uint32_t ld, const void* __restrict__ weight,
                                                                    void* __restrict__ out, const uint32_t rows, const uint32_t groups,
@@ -382,9 +382,25 @@ __global__ __launch_bounds__(256) void group_norm_gate_wave_kernel(const float* 
     const uint32_t i0 = lane * (uint32_t)EP;
     const size_t base = ((size_t)r * groups + g) * n, gbase = (size_t)r * ld + (size_t)g * n;
     float x[EP], z[EP], w[EP], ss = 0.f;
+    if constexpr (FULL && EP == 4) {
+        load4<kFP32>(o, base + i0, x);
+        load4<DT>(gate, gbase + i0, z);
+        load4<DT>(weight, i0, w);
+        ss = x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
+    } else if constexpr (FULL && EP == 2) {
+        const u32x2 t = *(const u32x2*)(o + base + i0);
+        x[0] = __uint_as_float(t[0]);
+        x[1] = __uint_as_float(t[1]);
+        uint32_t a, b;
+        E::load_raw2(gate, gbase + i0, a, b);
+        z[0] = E::from_raw2_lo(a, b); z[1] = E::from_raw2_hi(a, b);
+        E::load_raw2(weight, i0, a, b);
+        w[0] = E::from_raw2_lo(a, b); w[1] = E::from_raw2_hi(a, b);
+        ss = x[0] * x[0] + x[1] * x[1];
+    } else
 #pragma unroll
     for (int e = 0; e < EP; ++e) {
-        const bool ok = i0 + e < n;
+        const bool ok = FULL || i0 + e < n;
         const uint32_t i = ok ? i0 + e : 0u;
         x[e] = o[base + i];
         z[e] = E::load(gate, gbase + i);
@@ -392,9 +408,17 @@ __global__ __launch_bounds__(256) void group_norm_gate_wave_kernel(const float* 
         ss += ok ? x[e] * x[e] : 0.f;
     }
     const float rs = 1.f / sqrtf(wave_sum(ss) / (float)n + eps);
+    if constexpr (FULL) {
+#pragma unroll
+        for (int e = 0; e < EP; ++e) x[e] *= rs * w[e] * (kind == DECDEC_GATE_SILU ? silu_f(z[e]) : sigmoid_f(z[e]));
+        if constexpr (EP == 4) store4<DT>(out, base + i0, x);
+        else if constexpr (DT == kBF16) *(uint32_t*)((uint16_t*)out + base + i0) = pack_bf16(x[0], x[1]);
+        else *(u32x2*)((float*)out + base + i0) = u32x2{__float_as_uint(x[0]), __float_as_uint(x[1])};
+        return;
+    }
 #pragma unroll
     for (int e = 0; e < EP; ++e)
-        if (i0 + e < n) E::store(out, base + i0 + e, x[e] * rs * w[e] * (kind == DECDEC_GATE_SILU ? silu_f(z[e]) : sigmoid_f(z[e])));
+        if (FULL || i0 + e < n) E::store(out, base + i0 + e, x[e] * rs * w[e] * (kind == DECDEC_GATE_SILU ? silu_f(z[e]) : sigmoid_f(z[e])));
 }
 
 // Longer groups: a workgroup each, four neighbouring elements per thread and pass.
@@ -431,8 +455,14 @@ template <int DT>
 static hipError_t group_norm_dt(const float* o, const void* gate, uint32_t ld, const void* weight, void* out, uint32_t rows,
                                 uint32_t groups, uint32_t n, float eps, int kind, hipStream_t s) {
     const uint32_t es = Elem<DT>::bytes, waves = rows * groups;
-    if (n <= 128u) hipLaunchKernelGGL((group_norm_gate_wave_kernel<DT, 2>), dim3((waves + 3u) / 4u), dim3(256), 0, s, o, gate, ld, weight, out, rows, groups, n, eps, kind);
-    else if (n <= 256u) hipLaunchKernelGGL((group_norm_gate_wave_kernel<DT, 4>), dim3((waves + 3u) / 4u), dim3(256), 0, s, o, gate, ld, weight, out, rows, groups, n, eps, kind);
+    const dim3 wgrid((waves + 3u) / 4u), wblock(256);
+    auto full = [&](uint32_t ep) {
+        return n == 64u * ep && ld % ep == 0 && (uintptr_t)o % (4u * ep) == 0 && ((uintptr_t)gate | (uintptr_t)weight | (uintptr_t)out) % (es * ep) == 0;
+    };
+    if (full(2u)) hipLaunchKernelGGL((group_norm_gate_wave_kernel<DT, 2, true>), wgrid, wblock, 0, s, o, gate, ld, weight, out, rows, groups, n, eps, kind);
+    else if (n <= 128u) hipLaunchKernelGGL((group_norm_gate_wave_kernel<DT, 2, false>), wgrid, wblock, 0, s, o, gate, ld, weight, out, rows, groups, n, eps, kind);
+    else if (full(4u)) hipLaunchKernelGGL((group_norm_gate_wave_kernel<DT, 4, true>), wgrid, wblock, 0, s, o, gate, ld, weight, out, rows, groups, n, eps, kind);
+    else if (n <= 256u) hipLaunchKernelGGL((group_norm_gate_wave_kernel<DT, 4, false>), wgrid, wblock, 0, s, o, gate, ld, weight, out, rows, groups, n, eps, kind);
     else {
         uint32_t threads = 64;
         const bool vec = n % 4u == 0 && ld % 4u == 0 && n <= 16384u && (uintptr_t)o % 16u == 0 &&

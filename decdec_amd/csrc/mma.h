@@ -109,5 +109,16 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
     for (uint32_t w = 0; w < nw; ++w) t += red[w];
     return t;
 }
+// Two at once; red: 32 floats.
+__device__ __forceinline__ void block_sum2(float& a, float& b, float* red) {
+    a = wave_sum(a);
+    b = wave_sum(b);
+    const uint32_t lane = threadIdx.x & 63u, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
+    __syncthreads();
+    if (lane == 0) { red[wave] = a; red[16 + wave] = b; }
+    __syncthreads();
+    a = b = 0.f;
+    for (uint32_t w = 0; w < nw; ++w) { a += red[w]; b += red[16 + w]; }
+}
 
 }  // namespace decdec

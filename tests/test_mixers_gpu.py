@@ -76,12 +76,14 @@ def test_embed_norm_and_activation_rows(dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("groups,n,kind", [(1, 140, M.GATE_SIGMOID), (3, 36, M.GATE_SILU), (2, 2048, M.GATE_SILU)])
-def test_group_norm_gate(groups, n, kind, dtype):
-    o, g, w = _rand(3, groups * n, seed=1).cuda(), _rand(3, groups * n + 5, seed=2).to(dtype).cuda(), _rand(n, seed=3).to(dtype).cuda()
+@pytest.mark.parametrize("groups,n,kind", [(1, 140, M.GATE_SIGMOID), (3, 36, M.GATE_SILU), (2, 2048, M.GATE_SILU), (3, 128, M.GATE_SILU),
+                                           (2, 256, M.GATE_SIGMOID), (2, 201, M.GATE_SILU), (1, 1030, M.GATE_SIGMOID)])
+@pytest.mark.parametrize("off,pad", [(2, 5), (8, 16)])
+def test_group_norm_gate(groups, n, kind, off, pad, dtype):
+    o, g, w = _rand(3, groups * n, seed=1).cuda(), _rand(3, groups * n + pad, seed=2).to(dtype).cuda(), _rand(n, seed=3).to(dtype).cuda()
     out = torch.empty(3, groups * n, dtype=dtype, device="cuda")
-    M.group_norm_gate(o, g[:, 2:], groups * n + 5, w, out, groups, 0.01, kind)
-    z = g[:, 2:2 + groups * n].double()
+    M.group_norm_gate(o, g[:, off:], groups * n + pad, w, out, groups, 0.01, kind)
+    z = g[:, off:off + groups * n].double()
     want = O.rms_norm(o.double().view(3, groups, n), w.double(), 0.01).view(3, -1) * (O.silu(z) if kind == M.GATE_SILU else O.sigmoid(z))
     _close(out, want, dtype)
 
