@@ -1,4 +1,4 @@
-"""Models by name and checkpoints by architecture.
+"""Checkpoints by architecture (models with random weights go by name: ``model.ModelArgs.from_name``).
 
 A checkpoint is a folder with ``config.json`` (whose "architecture" names the design) and ``model.safetensors``."""
 from __future__ import annotations
@@ -9,7 +9,6 @@ import os
 import torch
 
 from .hybrid import HybridDecoder
-from .model import Transformer, transformer_configs
 
 # architectures a checkpoint's config.json may name
 ARCHITECTURES = {"Fivitar": HybridDecoder}
@@ -39,7 +38,3 @@ def load_model(path: str, dtype=torch.bfloat16, device="cuda"):
     model.load_weights(load_file(os.path.join(path, "model.safetensors")))
     return model.eval()
 
-
-def available() -> dict:
-    """Every model the command line knows by name, and the checkpoint architectures."""
-    return {"named": sorted(transformer_configs), "architectures": sorted(ARCHITECTURES), "named_class": Transformer}
