@@ -140,7 +140,7 @@ def _portions(T, *sizes):
 
 RECURRENCES = [("lightning", cases.lightning(3, 32, 32)), ("lightning", cases.lightning(5, 12, 28, [0.0, 0.3, 0.95, 0.9999, 1.0])),
                ("lightning", cases.lightning(2, 128, 128)), ("lightning", cases.lightning(1, 200, 72, [0.98])), ("lightning", cases.lightning(2, 1, 1)),
-               ("delta", cases.delta(2, 1, 32, 64, 4)), ("delta", cases.delta(3, 3, 20, 36, 3)), ("delta", cases.delta(4, 2, 128, 128, 4)),
+               ("delta", cases.delta(4, 2, 48, 64, 4)), ("delta", cases.delta(3, 3, 20, 36, 3)), ("delta", cases.delta(4, 2, 128, 128, 4)),
                ("delta", cases.delta(2, 2, 64, 16, 1)), ("delta", cases.delta(6, 2, 9, 130, 2)), ("delta", cases.delta(1, 1, 256, 256, 7)),
                ("delta", cases.delta(2, 1, 16, 300, 5))]
 
@@ -185,7 +185,7 @@ def test_convolution_sees_exactly_its_taps_across_a_cut():
             b.proj.copy_(keep)
 
 
-LATENTS = [cases.latent(4, 64, 32, 64, 64, scaling=cases.YARN), cases.latent(3, 22, 10, 18, 30, base=500.0), cases.latent(17, 16, 8, 24, 48, scale=0.4),
+LATENTS = [cases.latent(3, 64, 32, 96, 80, scaling=cases.YARN), cases.latent(3, 22, 10, 18, 30, base=500.0), cases.latent(17, 16, 8, 24, 48, scale=0.4),
            cases.latent(2, 128, 64, 128, 512, base=10000.0), cases.latent(1, 200, 56, 200, 96), cases.latent(2, 32, 16, 40, 72, dims=8),
            cases.latent(1, 2, 2, 1, 1), cases.latent(2, 96, 64, 256, 136)]
 
