@@ -1,4 +1,4 @@
-"""Plain, slow restatement of the Fivitar decoder on the CPU (torch, float64 by default).
+"""Plain, slow restatement of the Fivitar and Fekulix decoders on the CPU (torch, float64 by default).
 
 TEST INFRASTRUCTURE ONLY: one function per mechanism, every recurrence walked token by token, every attention row
 formed on its own.  Shares no code with the product path (``decdec_amd``), which never imports it.
@@ -35,6 +35,14 @@ def xielu(z, p, q):
     neg = torch.clamp(z, max=0)
     down = (0.5 + softplus(q)) * (torch.exp(neg) - 1 - neg) + neg / 2
     return torch.where(z > 0, up, down)
+
+
+def gelu_tanh(z):
+    return z / 2 * (1 + torch.tanh(math.sqrt(2 / math.pi) * (z + 0.044715 * z ** 3)))
+
+
+def dynamic_tanh(x, alpha, weight, bias):
+    return torch.tanh(alpha * x) * weight + bias
 
 
 def unit(x):
@@ -81,6 +89,30 @@ def decayed_sum(q, k, v, decay, state=None):
     out = []
     for t in range(T):
         S = decay[:, None, None] * S + k[t][:, :, None] * v[t][:, None, :]
+        out.append((S * q[t][:, :, None]).sum(1))
+    return torch.stack(out), S
+
+
+def channel_decayed_sum(q, k, v, g, state=None):
+    """q, k, g [T, H, D], v [T, H, V]: S <- diag(g) S + k v^T, o = S^T q."""
+    T, H, D = q.shape
+    S = torch.zeros(H, D, v.shape[-1], dtype=q.dtype) if state is None else state
+    out = []
+    for t in range(T):
+        S = g[t][:, :, None] * S + k[t][:, :, None] * v[t][:, None, :]
+        out.append((S * q[t][:, :, None]).sum(1))
+    return torch.stack(out), S
+
+
+def channel_delta_rule(q, k, v, g, beta, state=None):
+    """The delta rule with one decay per head and key channel: g [T, H, D]."""
+    T, H, D = q.shape
+    S = torch.zeros(H, D, v.shape[-1], dtype=q.dtype) if state is None else state
+    out = []
+    for t in range(T):
+        S = g[t][:, :, None] * S
+        u = beta[t][:, None] * (v[t] - (S * k[t][:, :, None]).sum(1))
+        S = S + k[t][:, :, None] * u[:, None, :]
         out.append((S * q[t][:, :, None]).sum(1))
     return torch.stack(out), S
 
@@ -152,7 +184,66 @@ def delta(h, w, cfg, eps):
     return o.reshape(T, H * V) @ w["o"].T
 
 
-MIXERS = {"lightning": lightning, "latent_attention": latent_attention, "delta": delta}
+def sink_attention(q, k, v, scale, sink=0.0):
+    """q [H, T, D], k [G, T, D], v [G, T, V]: causal softmax attention, query head h on key head h // (H / G), with a
+    valueless score `sink` in the denominator; [T, H, V]."""
+    H, T, _ = q.shape
+    share = H // k.shape[0]
+    out = torch.zeros(T, H, v.shape[-1], dtype=q.dtype)
+    for h in range(H):
+        kh, vh = k[h // share], v[h // share]
+        for i in range(T):
+            s = kh[:i + 1] @ q[h, i] * scale
+            m = max(float(s.max()), sink)
+            e = torch.exp(s - m)
+            out[i, h] = (e[:, None] * vh[:i + 1]).sum(0) / (e.sum() + math.exp(sink - m))
+    return out
+
+
+def gated_attention(h, w, cfg, eps):
+    """Grouped-query attention with normed, partly rotated queries and keys, a sink and one gate per head: read-out."""
+    T, H, G, D, V = h.shape[0], cfg["heads"], cfg["kv_heads"], cfg["dim"], cfg["vdim"]
+    pos = torch.arange(T)
+    q = rms_norm((h @ w["q"].T).view(T, H, D), w["q.norm"], eps).transpose(0, 1)
+    k = rms_norm((h @ w["k"].T).view(T, G, D), w["k.norm"], eps).transpose(0, 1)
+    v = (h @ w["v"].T).view(T, G, V).transpose(0, 1)
+    o = sink_attention(rotate(q, pos, cfg["rot"]), rotate(k, pos, cfg["rot"]), v, cfg["scale"])
+    return (o * sigmoid(h @ w["g"].T)[:, :, None]).reshape(T, H * V)
+
+
+def gated_linear(h, w, cfg, eps):
+    """Gated linear attention with a decay per key channel: read-out."""
+    T, H, D, V = h.shape[0], cfg["heads"], cfg["dim"], cfg["vdim"]
+    q, k, v = ((h @ w[n].T).view(T, H, -1) for n in "qkv")
+    z = (h @ w["a1"].T) @ w["a2"].T + w["a2.b"]
+    decay = torch.exp(-softplus(-z) / cfg["tau"]).view(T, H, D)
+    o, _ = channel_decayed_sum(q * D ** -0.5, k, v, decay)
+    return rms_norm(o, w["norm"], eps).reshape(T, H * V) * silu(h @ w["g"].T)
+
+
+def parallel(h, w, cfg, eps):
+    part = lambda side: {n[len(side) + 1:]: t for n, t in w.items() if n.startswith(side + ".")}
+    left, right = part("left"), part("right")
+    a = gated_attention(h, left, cfg["left"], eps) @ left["o"].T
+    b = gated_linear(h, right, cfg["right"], eps) @ right["o"].T
+    return cfg["left_scale"] * a + cfg["right_scale"] * b
+
+
+def channel_delta(h, w, cfg, eps):
+    T, H, G, D, V = h.shape[0], cfg["heads"], cfg["kv_heads"], cfg["dim"], cfg["vdim"]
+    q, k, v = (silu(causal_conv(h @ w[n].T, w[n + ".conv"])) for n in "qkv")
+    q, k = unit(q.view(T, G, D)) * D ** -0.5, unit(k.view(T, G, D))
+    q, k = q.repeat_interleave(H // G, 1), k.repeat_interleave(H // G, 1)
+    beta = sigmoid(h @ w["b"].T)
+    step = softplus((h @ w["a1"].T) @ w["a2"].T + w["dt_bias"]).view(T, H, D)
+    g = torch.exp(-torch.exp(w["A_log"])[:, None] * step)
+    o, _ = channel_delta_rule(q, k, v.view(T, H, V), g, beta)
+    o = rms_norm(o, w["norm"], eps) * sigmoid((h @ w["g1"].T) @ w["g2"].T).view(T, H, V)
+    return o.reshape(T, H * V) @ w["o"].T
+
+
+MIXERS = {"lightning": lightning, "latent_attention": latent_attention, "delta": delta, "parallel": parallel,
+          "channel_delta": channel_delta}
 
 
 # ---- the decoder -----------------------------------------------------------------------------------------
@@ -161,23 +252,46 @@ def gated(y, h, w, b):
     return y * sigmoid(h @ w.T + b)
 
 
+def fivitar_layer(x, layer, w, eps):
+    """Norms and gates on the sublayers' outputs; w: the layer's tensors by name."""
+    y = MIXERS[layer["type"]](x, _under(w, "mix."), layer["mixer"], eps)
+    x = x + rms_norm(gated(y, x, w["rg1"], w["rg1.b"]), w["norm1"], eps)
+    if layer.get("mlp") is not None:
+        a = w["mlp.act"]
+        y = xielu(x @ w["mlp.up"].T, a[0], a[1]) @ w["mlp.down"].T
+        x = x + rms_norm(gated(y, x, w["rg2"], w["rg2.b"]), w["norm2"], eps)
+    return x
+
+
+def fekulix_layer(x, layer, w, eps):
+    """Dynamic tanh on the sublayers' inputs."""
+    x = x + MIXERS[layer["type"]](dyt(x, w, "norm1"), _under(w, "mix."), layer["mixer"], eps)
+    if layer.get("mlp") is not None:
+        x = x + gelu_tanh(dyt(x, w, "norm2") @ w["mlp.up"].T) @ w["mlp.down"].T
+    return x
+
+
+def dyt(x, w, name):
+    return dynamic_tanh(x, w[name + ".alpha"], w[name], w[name + ".b"])
+
+
+def _under(w, prefix):
+    return {n[len(prefix):]: t for n, t in w.items() if n.startswith(prefix)}
+
+
 def forward(config, weights, tokens, dtype=torch.float64, layers_out=None):
     """Logits [T, vocab] of one sequence; layers_out (a list) receives the residual stream after every layer."""
     W = {n: t.to(dtype) if t.is_floating_point() else t for n, t in weights.items()}
     eps = config["norm"]["eps"]
+    fekulix = config["architecture"] == "Fekulix"
     x = W["embed"][torch.as_tensor(tokens)]
     for i, layer in enumerate(config["layers"]):
         src = i
         while config["layers"][src].get("weights_of") is not None:
             src = config["layers"][src]["weights_of"]
-        p = f"l{src}."
-        mix = {n[len(p) + 4:]: t for n, t in W.items() if n.startswith(p + "mix.")}
-        y = MIXERS[layer["type"]](x, mix, layer["mixer"], eps)
-        x = x + rms_norm(gated(y, x, W[p + "rg1"], W[p + "rg1.b"]), W[p + "norm1"], eps)
-        if layer.get("mlp") is not None:
-            a = W[p + "mlp.act"]
-            y = xielu(x @ W[p + "mlp.up"].T, a[0], a[1]) @ W[p + "mlp.down"].T
-            x = x + rms_norm(gated(y, x, W[p + "rg2"], W[p + "rg2.b"]), W[p + "norm2"], eps)
+        x = (fekulix_layer if fekulix else fivitar_layer)(x, layer, _under(W, f"l{src}."), eps)
         if layers_out is not None:
             layers_out.append(x.clone())
+    if fekulix:
+        return dyt(x, W, "final.norm") @ W["head"].T * config["logit_scale"]
     return rms_norm(x, W["final.norm"], eps) @ W["head"].T
