@@ -108,8 +108,23 @@ def load():
 class Recurrence(ctypes.Structure):
     """Mirror of ``decdec_recurrence``."""
     _fields_ = ([("proj", _vp)] + [(n, _u32) for n in (
-        "ld", "off_q", "off_k", "off_v", "off_g", "off_a", "off_b", "heads", "kv_heads", "dim", "vdim", "taps", "delta")]
-        + [(n, _vp) for n in ("decay", "conv_q", "conv_k", "conv_v", "A_log", "dt_bias", "ring", "state", "pos")])
+        "ld", "off_q", "off_k", "off_v", "off_g", "off_a", "off_b", "heads", "kv_heads", "dim", "vdim", "taps", "delta", "channel",
+        "rank_a", "rank_g")] + [("a_sign", _f32), ("out_scale", _f32)]
+        + [(n, _vp) for n in ("decay", "conv_q", "conv_k", "conv_v", "A_log", "dt_bias", "rate", "a_bias", "a2", "g2", "a", "ring",
+                              "state", "pos")])
+
+
+class Grouped(ctypes.Structure):
+    """Mirror of ``decdec_grouped``."""
+    _fields_ = ([("proj", _vp)] + [(n, _u32) for n in (
+        "ld", "off_q", "off_k", "off_v", "off_g", "heads", "kv_heads", "dim", "vdim", "rot", "max_seq", "gated", "out_ld")]
+        + [(n, _f32) for n in ("eps", "scale", "sink", "out_scale")]
+        + [(n, _vp) for n in ("q_norm", "k_norm", "cos_table", "sin_table", "keys", "values", "pos")])
+
+
+class TanhNorm(ctypes.Structure):
+    """Mirror of ``decdec_tanh_norm``."""
+    _fields_ = [(n, _vp) for n in ("alpha", "weight", "bias")]
 
 
 class Latent(ctypes.Structure):
@@ -119,23 +134,28 @@ class Latent(ctypes.Structure):
         + [(n, _vp) for n in ("norm", "uk", "uv", "sink", "cos_table", "sin_table", "cache", "pos")])
 
 
-_rec, _lat = ctypes.POINTER(Recurrence), ctypes.POINTER(Latent)
+_rec, _lat, _grp, _tanh = (ctypes.POINTER(c) for c in (Recurrence, Latent, Grouped, TanhNorm))
 MIXERS_SIGNATURES = {
-    "decdec_mix_gemv": [_vp, _vp, _vp, _vp, _u32, _i32, _u32, _u32, _vp],
-    "decdec_mix_embed": [_vp, _vp, _vp, _vp, _i32, _u32, _u32, _u32, _vp],
+    "decdec_mix_gemv": [_vp, _vp, _vp, _vp, _u32, _i32, _f32, _i32, _u32, _u32, _vp],
+    "decdec_mix_embed": [_vp, _vp, _vp, _vp, _tanh, _i32, _u32, _u32, _u32, _vp],
+    "decdec_mix_residual_tanh": [_vp, _vp, _tanh, _vp, _i32, _u32, _u32, _vp],
     "decdec_mix_gated_residual": [_vp, _vp, _vp, _u32, _vp, _vp, _vp, _vp, _vp, _i32, _u32, _u32, _f32, _vp],
     "decdec_mix_rmsnorm": [_vp, _vp, _vp, _i32, _u32, _u32, _f32, _vp],
-    "decdec_mix_xielu": [_vp, _u32, _vp, _vp, _i32, _u32, _u32, _vp],
-    "decdec_mix_group_norm_gate": [_vp, _vp, _u32, _vp, _vp, _i32, _u32, _u32, _u32, _f32, _i32, _vp],
+    "decdec_mix_activation": [_vp, _u32, _vp, _i32, _vp, _i32, _u32, _u32, _vp],
+    "decdec_mix_group_norm_gate": [_vp, _vp, _u32, _vp, _vp, _u32, _i32, _u32, _u32, _u32, _f32, _i32, _f32, _vp],
     "decdec_mix_recurrence_step": [_rec, _vp, _vp, _vp, _f32, _i32, _i32, _vp],
     "decdec_mix_recurrence_step_fuses": [_u32, _u32],
     "decdec_mix_recurrence_rows": [_rec, _vp, _vp, _u64, _i32, _u32, _vp],
+    "decdec_mix_grouped_append": [_grp, _vp, _i32, _u32, _vp],
+    "decdec_mix_grouped_attention": [_grp, _vp, _vp, _i32, _u32, _u32, _vp],
+    "decdec_mix_grouped_step": [_grp, _vp, _vp, _u64, _i32, _vp],
     "decdec_mix_latent_append": [_lat, _vp, _i32, _u32, _vp],
     "decdec_mix_latent_attention": [_lat, _vp, _vp, _vp, _u32, _vp, _i32, _u32, _u32, _vp],
     "decdec_mix_latent_step": [_lat, _vp, _vp, _u64, _i32, _vp],
 }
 MIXERS_OTHER = {"decdec_mixers_last_error": ([], ctypes.c_char_p),
                 "decdec_mix_recurrence_workspace": ([_rec, _u32], _u64),
+                "decdec_mix_grouped_step_workspace": ([_grp], _u64),
                 "decdec_mix_latent_step_workspace": ([_lat], _u64)}
 
 

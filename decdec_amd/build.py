@@ -1,5 +1,5 @@
 """Builds the gfx950 libraries in-tree with hipcc: libdecdec_hip.so (quantised linears, DEC, decode helpers) and
-libdecdec_mixers.so (recurrences, latent attention and the row kernels of decoders built from them).
+libdecdec_mixers.so (recurrences, latent and grouped attention and the row kernels of decoders built from them).
 
 Usage: ``python -m decdec_amd.build`` or ``decdec_amd.build.build_library()``; ``build_library(["mixers"])`` builds one.
 hipcc cross-compiles for gfx950 without a GPU.  The translation units are compiled in parallel and
@@ -21,7 +21,7 @@ LIB_PATH = os.path.join(HERE, "libdecdec_hip.so")
 RESOURCES_PATH = os.path.join(OBJ_DIR, "kernel_resources.json")
 MIXERS_LIB_PATH = os.path.join(HERE, "libdecdec_mixers.so")
 SOURCES = ["k_dec.hip", "k_anyprec.hip", "k_lutgemm.hip", "k_sqllm.hip", "k_decode.hip", "capi.hip"]
-MIXERS_SOURCES = ["k_rows.hip", "k_recurrence.hip", "k_latent.hip", "capi_mixers.hip"]
+MIXERS_SOURCES = ["k_rows.hip", "k_recurrence.hip", "k_attention.hip", "k_latent.hip", "capi_mixers.hip"]
 LIBRARIES = {"linears": (LIB_PATH, SOURCES), "mixers": (MIXERS_LIB_PATH, MIXERS_SOURCES)}
 ARCH = "gfx950"
 

@@ -28,6 +28,29 @@ class KVCache(nn.Module):
         return []
 
 
+class GroupedCache:
+    """Keys by head [heads, positions, dim] and values transposed [heads * vdim, positions], as the attention products read
+    them.  The positions come in multiples of 64 and are finite from the start (tiles read past the last one)."""
+
+    def __init__(self, max_seq_length: int, kv_heads: int, dim: int, vdim: int, dtype, device):
+        self.positions = (max_seq_length + 63) // 64 * 64
+        self.keys = torch.zeros(kv_heads, self.positions, dim, dtype=dtype, device=device)
+        self.values = torch.zeros(kv_heads * vdim, self.positions, dtype=dtype, device=device)
+
+    def recurrent(self):
+        return []
+
+
+class JoinedState:
+    """The entries of mixers that run side by side in one layer."""
+
+    def __init__(self, parts):
+        self.parts = list(parts)
+
+    def recurrent(self):
+        return [t for p in self.parts for t in p.recurrent()]
+
+
 class LatentCache:
     """One row per position: a latent all heads' keys and values are linear in, and a rotated key part they share.
     The rows come in multiples of 64 and are finite from the start (tiles read past the last position)."""

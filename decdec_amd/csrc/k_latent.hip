@@ -2,7 +2,7 @@
 // holds, next to a rotated key part that the heads share.
 //
 // Many tokens: keys and values of the whole past are formed by two matrix products outside and attended by a tiled
-// kernel.  One token: the up projections are absorbed -- a query is carried into the latent space (absorb kernel), all
+// kernel (k_attention.hip).  One token: the up projections are absorbed -- a query is carried into the latent space (absorb kernel), all
 // heads attend the same cache rows (step kernel, sequence split over workgroups), and the attended latents are carried
 // to the values (merge kernel).  Scores, weights and sums are fp32; on bf16 storage a weight enters the value product as
 // the sum of two bf16 numbers.
@@ -10,50 +10,6 @@
 #include "mma.h"
 
 namespace decdec {
-
-template <int DT> __device__ __forceinline__ void store_elem(typename LaneOf<DT>::t* p, float v) { Elem<DT>::store(p, 0, v); }
-
-// eight elements of a row as a fragment, zero past `valid`
-template <int DT>
-__device__ __forceinline__ Frag<DT> load8(const typename LaneOf<DT>::t* p, int valid, bool vec) {
-    if (vec && valid >= 8) return frag_load(p);
-    Frag<DT> f;
-    if constexpr (DT == kFP32) {
-#pragma unroll
-        for (int i = 0; i < 8; ++i) f.v[i] = i < valid ? p[i] : 0.f;
-    } else {
-#pragma unroll
-        for (int i = 0; i < 4; ++i)
-            f.v[i] = (uint32_t)(2 * i < valid ? p[2 * i] : 0) | ((uint32_t)(2 * i + 1 < valid ? p[2 * i + 1] : 0) << 16);
-    }
-    return f;
-}
-__device__ __forceinline__ void store8(uint16_t* p, const Frag<kBF16>& f) { *(u32x4*)p = f.v; }
-__device__ __forceinline__ void store8(float* p, const Frag<kFP32>& f) {
-#pragma unroll
-    for (int i = 0; i < 8; i += 4) *(f32x4*)(p + i) = f32x4{f.v[i], f.v[i + 1], f.v[i + 2], f.v[i + 3]};
-}
-__device__ __forceinline__ void frag_values(const Frag<kBF16>& f, float (&x)[8]) {
-#pragma unroll
-    for (int i = 0; i < 4; ++i) { x[2 * i] = __uint_as_float(f.v[i] << 16); x[2 * i + 1] = __uint_as_float(f.v[i] & 0xFFFF0000u); }
-}
-__device__ __forceinline__ void frag_values(const Frag<kFP32>& f, float (&x)[8]) {
-#pragma unroll
-    for (int i = 0; i < 8; ++i) x[i] = f.v[i];
-}
-
-__device__ __forceinline__ Frag<kBF16> frag_of(const float (&x)[8], const Frag<kBF16>&) {
-    Frag<kBF16> f;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) f.v[i] = pack_bf16(x[2 * i], x[2 * i + 1]);
-    return f;
-}
-__device__ __forceinline__ Frag<kFP32> frag_of(const float (&x)[8], const Frag<kFP32>&) {
-    Frag<kFP32> f;
-#pragma unroll
-    for (int i = 0; i < 8; ++i) f.v[i] = x[i];
-    return f;
-}
 
 // The new cache row of one token (a whole workgroup): normed latent, rotated shared key part.
 template <int DT>
@@ -129,221 +85,16 @@ hipError_t launch_latent_append(int dt, const decdec_latent& p, void* q_out, uin
 }
 
 // ---- many tokens ------------------------------------------------------------------------------------------
-// Workgroups of four waves with 16 MT queries each, one per query block and head; the heads are dealt to the eight dies,
-// so that the tiles of a head's keys and values are shared in one L2.  The transposed scores (keys x queries) leave a query in one
-// lane column: its running maximum and sum are lane values, its weights are at once the right operand of the value
-// product (out^T = V^T P^T), and nothing passes through LDS but the key and value tiles.  The contraction of that product
-// visits keys 4 (lane / 16) + e of one 16-key tile, then of the next, in both operands.  The next tile is requested into
-// registers while the present one is worked on.  Scores are kept in units of log 2.
-constexpr uint32_t kKeys = 64;
-
-template <int DT, int MT, int NK, int NV, bool VEC>
-__global__ __launch_bounds__(256, DT == kFP32 ? 1 : 2) void latent_attention_kernel(const decdec_latent p, const void* __restrict__ q_in,
-                                                               const void* __restrict__ k_in, const void* __restrict__ vt_in,
-                                                               const uint32_t vt_ld, void* __restrict__ out,
-                                                               const uint32_t start, const uint32_t rows, const uint32_t blocks) {
-    using T = typename LaneOf<DT>::t;
-    using E = Elem<DT>;
-    constexpr uint32_t PAD = DT == kFP32 ? 4u : 8u, KL = 32u * NK + PAD, VL = kKeys + PAD;
-    extern __shared__ __align__(16) unsigned char smem[];
-    T* Kl = (T*)smem;                       // [kKeys][KL]
-    T* Vl = Kl + kKeys * KL;                // [16 NV][VL]
-    const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, l16 = lane & 15u, lg = lane >> 4;
-    const uint32_t turn = blockIdx.x >> 3, h = (blockIdx.x & 7u) + 8u * (turn / blocks);
-    if (h >= p.heads) return;
-    const uint32_t q0 = (blocks - 1u - turn % blocks) * (64u * MT);        // longest rows first
-    const uint32_t Dq = p.dim + p.rot, D = p.dim, V = p.vdim, keys_total = start + rows;
-    const T* q = (const T*)q_in;
-    Frag<DT> qf[MT][NK];
-    uint32_t qpos[MT];
-#pragma unroll
-    for (int m = 0; m < MT; ++m) {
-        const uint32_t r = q0 + 16u * (MT * wave + (uint32_t)m) + l16, rc = r < rows ? r : rows - 1u;
-        qpos[m] = start + rc;
-#pragma unroll
-        for (int s = 0; s < NK; ++s)
-            qf[m][s] = load8<DT>(q + ((size_t)rc * p.heads + h) * Dq + 32u * s + 8u * lg, (int)Dq - (int)(32u * s + 8u * lg), VEC);
-    }
-    const float scale2 = p.scale * kLog2e;
-    const float sink = p.sink != nullptr ? E::load(p.sink, h) * kLog2e : -__builtin_inff();
-    float mx[MT], sum[MT];
-    f32x4 o[MT][NV];
-#pragma unroll
-    for (int m = 0; m < MT; ++m) {
-        mx[m] = sink;
-        sum[m] = (p.sink != nullptr && lg == 0u) ? 1.f : 0.f;              // lane groups hold partial sums
-#pragma unroll
-        for (int n = 0; n < NV; ++n) o[m][n] = f32x4{0.f, 0.f, 0.f, 0.f};
-    }
-    const uint32_t last = q0 + 64u * MT < rows ? q0 + 64u * MT : rows;     // one past the block's last query
-    const uint32_t kend = start + last, wave_first = start + q0 + 16u * MT * wave, wave_last = wave_first + 16u * MT - 1u;
-    const size_t kld = (size_t)p.heads * D, cld = p.rank + p.rot;
-    const T* kb = (const T*)k_in + (size_t)h * D;
-    const T* cb = (const T*)p.cache + p.rank;
-    const T* vb = (const T*)vt_in + (size_t)h * V * vt_ld;
-    // A key row is [unrotated part of the head | shared rotated part]; keys past the end repeat the last one and are never
-    // weighted, value rows past vdim repeat the first one and are never stored.  A thread loads eight elements of every
-    // slice of one key, and of every 32nd value row.
-    Frag<DT> kr[VEC ? NK : 1], vr[VEC ? NV / 2 : 1];
-    const uint32_t krow = tid >> 2, kcol = (tid & 3u) * 8u, vrow = tid >> 3, vcol = (tid & 7u) * 8u;
-    auto request = [&](uint32_t k0) {
-        const uint32_t key = k0 + krow < keys_total ? k0 + krow : keys_total - 1u;
-        const T* un = kb + key * kld + kcol;
-        const T* ro = cb + key * cld + kcol;
-#pragma unroll
-        for (int j = 0; j < NK; ++j) {
-            const uint32_t c = 32u * j + kcol;
-            kr[j] = frag_load(c < D ? un + 32u * j : (c < Dq ? ro + (32 * j - (int)D) : cb));
-            if (c >= Dq) kr[j] = Frag<DT>{};
-        }
-        const T* vp = vb + k0 + vcol;
-#pragma unroll
-        for (int j = 0; j < NV / 2; ++j) vr[j] = frag_load(vp + (size_t)(vrow + 32u * j < V ? vrow + 32u * j : 0u) * vt_ld);
-    };
-    if constexpr (VEC) request(0u);
-    for (uint32_t k0 = 0; k0 < kend; k0 += kKeys) {
-        __syncthreads();
-        if constexpr (VEC) {
-#pragma unroll
-            for (int j = 0; j < NK; ++j) store8(Kl + krow * KL + kcol + 32u * j, kr[j]);
-#pragma unroll
-            for (int j = 0; j < NV / 2; ++j) store8(Vl + (vrow + 32u * j) * VL + vcol, vr[j]);
-        } else {
-            for (uint32_t i = tid; i < kKeys * 32u * NK; i += 256u) {
-                const uint32_t r = i / (32u * NK), c = i % (32u * NK), key = k0 + r < keys_total ? k0 + r : keys_total - 1u;
-                Kl[r * KL + c] = c < D ? kb[key * kld + c] : (c < Dq ? cb[key * cld + c - D] : (T)0);
-            }
-            for (uint32_t i = tid; i < 16u * NV * kKeys; i += 256u) {
-                const uint32_t d = i / kKeys, c = i % kKeys;
-                Vl[d * VL + c] = d < V ? vb[(size_t)d * vt_ld + k0 + c] : (T)0;
-            }
-        }
-        __syncthreads();
-        if constexpr (VEC) { if (k0 + kKeys < kend) request(k0 + kKeys); }
-        if (k0 > wave_last) continue;                                      // every key of the tile lies after the wave's queries
-        f32x4 sc[MT][4];
-#pragma unroll
-        for (int m = 0; m < MT; ++m)
-#pragma unroll
-            for (int t = 0; t < 4; ++t) sc[m][t] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int s = 0; s < NK; ++s)
-#pragma unroll
-            for (int t = 0; t < 4; ++t) {
-                const Frag<DT> a = frag_load(Kl + (16u * t + l16) * KL + 32u * s + 8u * lg);
-#pragma unroll
-                for (int m = 0; m < MT; ++m) mma(a, qf[m][s], sc[m][t]);
-            }
-        const bool edge = k0 + kKeys > wave_first + 1u;                    // some key may lie after some query of the wave
-        Frag<DT> hi[MT][2], lo[MT][2];
-#pragma unroll
-        for (int m = 0; m < MT; ++m) {
-            float best = mx[m];
-#pragma unroll
-            for (int t = 0; t < 4; ++t)
-#pragma unroll
-                for (int v = 0; v < 4; ++v) {
-                    float x = sc[m][t][v] * scale2;
-                    if (edge && k0 + 16u * t + 4u * lg + (uint32_t)v > qpos[m]) x = -__builtin_inff();
-                    sc[m][t][v] = x;
-                    best = fmaxf(best, x);
-                }
-            best = fmaxf(best, __shfl_xor(best, 16, 64));
-            best = fmaxf(best, __shfl_xor(best, 32, 64));
-            if (__any(best > mx[m])) {
-                const float corr = __builtin_amdgcn_exp2f(mx[m] - best);   // the first key is visible to every query: best is finite
-                mx[m] = best;
-                sum[m] *= corr;
-#pragma unroll
-                for (int n = 0; n < NV; ++n) o[m][n] *= corr;
-            }
-#pragma unroll
-            for (int t = 0; t < 2; ++t) {
-                float w[8];
-#pragma unroll
-                for (int e = 0; e < 8; ++e) {
-                    w[e] = __builtin_amdgcn_exp2f(sc[m][2 * t + (e >> 2)][e & 3] - best);
-                    sum[m] += w[e];
-                }
-                frag_split(w, hi[m][t], lo[m][t]);
-            }
-        }
-#pragma unroll
-        for (int n = 0; n < NV; ++n)
-#pragma unroll
-            for (int t = 0; t < 2; ++t) {
-                const T* vk = Vl + (16u * n + l16) * VL + 32u * t + 4u * lg;
-                Frag<DT> a;
-                if constexpr (DT == kFP32) {
-                    const f32x4 x = *(const f32x4*)vk, y = *(const f32x4*)(vk + 16);
-#pragma unroll
-                    for (int e = 0; e < 4; ++e) { a.v[e] = x[e]; a.v[4 + e] = y[e]; }
-                } else {
-                    const u32x2 x = *(const u32x2*)vk, y = *(const u32x2*)(vk + 16);
-                    a.v = u32x4{x[0], x[1], y[0], y[1]};
-                }
-#pragma unroll
-                for (int m = 0; m < MT; ++m) {
-                    mma(a, hi[m][t], o[m][n]);
-                    if constexpr (DT != kFP32) mma(a, lo[m][t], o[m][n]);
-                }
-            }
-    }
-#pragma unroll
-    for (int m = 0; m < MT; ++m) {
-        float t = sum[m];
-        t += __shfl_xor(t, 16, 64);
-        t += __shfl_xor(t, 32, 64);
-        const float r = 1.f / t;
-        const uint32_t row = q0 + 16u * (MT * wave + (uint32_t)m) + l16;
-        if (row < rows) {
-#pragma unroll
-            for (int n = 0; n < NV; ++n)
-#pragma unroll
-                for (int v = 0; v < 4; ++v) {
-                    const uint32_t d = 16u * n + 4u * lg + (uint32_t)v;
-                    if (d < V) E::store(out, ((size_t)row * p.heads + h) * V + d, o[m][n][v] * r);
-                }
-        }
-    }
-}
-
-template <int DT, int MT, int NK, int NV, bool VEC = true>
-static hipError_t attention_launch(const decdec_latent& p, const void* q, const void* k, const void* vt, uint32_t vt_ld, void* out,
-                                   uint32_t start, uint32_t rows, hipStream_t s) {
-    constexpr uint32_t PAD = DT == kFP32 ? 4u : 8u;
-    constexpr size_t lds = (size_t)(kKeys * (32u * NK + PAD) + 16u * NV * (kKeys + PAD)) * Elem<DT>::bytes;
-    static_assert(lds <= 160u * 1024u, "tiles must fit the LDS of a compute unit");
-    if (hipError_t e = allow_lds<latent_attention_kernel<DT, MT, NK, NV, VEC>>(lds); e != hipSuccess) return e;
-    const uint32_t blocks = (rows + 64u * MT - 1u) / (64u * MT);
-    hipLaunchKernelGGL((latent_attention_kernel<DT, MT, NK, NV, VEC>), dim3(blocks * ((p.heads + 7u) / 8u * 8u)), dim3(256), lds, s,
-                       p, q, k, vt, vt_ld, out, start, rows, blocks);
-    return hipGetLastError();
-}
-
-template <int DT, int MT, int NK>
-static hipError_t attention_nv(const decdec_latent& p, const void* q, const void* k, const void* vt, uint32_t vt_ld, void* out,
-                               uint32_t start, uint32_t rows, hipStream_t s) {
-    if (p.vdim <= 64u) return attention_launch<DT, MT, NK, 4>(p, q, k, vt, vt_ld, out, start, rows, s);
-    if (p.vdim <= 128u) return attention_launch<DT, MT, NK, 8>(p, q, k, vt, vt_ld, out, start, rows, s);
-    return attention_launch<DT, 1, NK, 16>(p, q, k, vt, vt_ld, out, start, rows, s);
-}
-
-template <int DT, int MT>
-static hipError_t attention_dt(const decdec_latent& p, const void* q, const void* k, const void* vt, uint32_t vt_ld, void* out,
-                               uint32_t start, uint32_t rows, hipStream_t s) {
-    const uint32_t Dq = p.dim + p.rot;
-    if (p.dim % 8u != 0 || p.rot % 8u != 0 || p.rank % 8u != 0) return attention_launch<DT, 1, 10, 16, false>(p, q, k, vt, vt_ld, out, start, rows, s);
-    if (Dq <= 128u) return attention_nv<DT, MT, 4>(p, q, k, vt, vt_ld, out, start, rows, s);
-    if (Dq <= 192u) return attention_nv<DT, MT, 6>(p, q, k, vt, vt_ld, out, start, rows, s);
-    return attention_nv<DT, 1, 10>(p, q, k, vt, vt_ld, out, start, rows, s);
-}
-
 hipError_t launch_latent_attention(int dt, const decdec_latent& p, const void* q, const void* k, const void* vt, uint32_t vt_ld,
                                    void* out, uint32_t start, uint32_t rows, hipStream_t s) {
-    if (p.dim + p.rot > 320u || p.vdim > 256u) return hipErrorInvalidValue;
-    if (dt == kBF16) return attention_dt<kBF16, 2>(p, q, k, vt, vt_ld, out, start, rows, s);
-    return attention_dt<kFP32, 1>(p, q, k, vt, vt_ld, out, start, rows, s);
+    TileAttention a{};
+    a.q = q; a.k = k; a.vt = vt; a.out = out; a.sink = p.sink;
+    a.shared = (const char*)p.cache + (size_t)p.rank * (dt == kBF16 ? 2u : 4u);
+    a.k_head = p.dim; a.k_row = (size_t)p.heads * p.dim;
+    a.shared_row = p.rank + p.rot; a.vt_ld = vt_ld; a.out_ld = p.heads * p.vdim;
+    a.heads = p.heads; a.share = 1; a.dim = p.dim; a.rot = p.rot; a.vdim = p.vdim;
+    a.scale = p.scale; a.sink_score = -__builtin_inff(); a.out_scale = 1.f;
+    return launch_tile_attention(dt, a, start, rows, s);
 }
 
 // ---- one token --------------------------------------------------------------------------------------------

@@ -1,5 +1,5 @@
 // Row-wise pieces of decoders with a 32-bit residual stream: one-token GEMV with an activation on its first rows,
-// embedding, gated residual + norm of the sublayer's output, norm, xIELU, normed and gated read-out of a recurrence.
+// embedding, gated residual + norm of the sublayer's output, residual + dynamic tanh, norm, activations, normed and gated read-out of a recurrence.
 #include "mixers.h"
 #include "mma.h"
 
@@ -29,7 +29,8 @@ __device__ __forceinline__ float dot16(const u32x4& w, const u32x4& x, float acc
 template <int DT, int ROWS, bool VEC>
 __global__ __launch_bounds__(256) void mix_gemv_kernel(const void* __restrict__ weight, const void* __restrict__ x,
                                                        void* __restrict__ out, const void* __restrict__ act,
-                                                       const uint32_t act_rows, const uint32_t N, const uint32_t K) {
+                                                       const uint32_t act_rows, const int act_kind, const float scale,
+                                                       const uint32_t N, const uint32_t K) {
     using E = Elem<DT>;
     constexpr uint32_t PE = Pack16<DT>::n, UN = ROWS >= 4 ? 2 : (ROWS == 2 ? 4 : 8);
     const uint32_t lane = threadIdx.x & 63u, wave = threadIdx.x >> 6;
@@ -79,28 +80,30 @@ __global__ __launch_bounds__(256) void mix_gemv_kernel(const void* __restrict__ 
         float v = acc[0];
 #pragma unroll
         for (int r = 1; r < ROWS; ++r) v = lane == (uint32_t)r ? acc[r] : v;
-        if (row0 + lane < act_rows) v = xielu_f(v, softplus_f(E::load(act, 0)), softplus_f(E::load(act, 1)));
+        v *= scale;
+        if (row0 + lane < act_rows)
+            v = act_kind == DECDEC_ACT_GELU_TANH ? gelu_tanh_f(v) : xielu_f(v, softplus_f(E::load(act, 0)), softplus_f(E::load(act, 1)));
         E::store(out, row0 + lane, v);
     }
 }
 
 template <int DT, bool VEC>
 static void gemv_rows(uint32_t N, uint32_t K, const void* w, const void* x, void* out, const void* act, uint32_t act_rows,
-                      hipStream_t s) {
-    if (N >= 16384u) hipLaunchKernelGGL((mix_gemv_kernel<DT, 4, VEC>), dim3((N + 15u) / 16u), dim3(256), 0, s, w, x, out, act, act_rows, N, K);
-    else if (N >= 4096u) hipLaunchKernelGGL((mix_gemv_kernel<DT, 2, VEC>), dim3((N + 7u) / 8u), dim3(256), 0, s, w, x, out, act, act_rows, N, K);
-    else hipLaunchKernelGGL((mix_gemv_kernel<DT, 1, VEC>), dim3((N + 3u) / 4u), dim3(256), 0, s, w, x, out, act, act_rows, N, K);
+                      int act_kind, float scale, hipStream_t s) {
+    if (N >= 16384u) hipLaunchKernelGGL((mix_gemv_kernel<DT, 4, VEC>), dim3((N + 15u) / 16u), dim3(256), 0, s, w, x, out, act, act_rows, act_kind, scale, N, K);
+    else if (N >= 4096u) hipLaunchKernelGGL((mix_gemv_kernel<DT, 2, VEC>), dim3((N + 7u) / 8u), dim3(256), 0, s, w, x, out, act, act_rows, act_kind, scale, N, K);
+    else hipLaunchKernelGGL((mix_gemv_kernel<DT, 1, VEC>), dim3((N + 3u) / 4u), dim3(256), 0, s, w, x, out, act, act_rows, act_kind, scale, N, K);
 }
 
-hipError_t launch_mix_gemv(int dt, const void* w, const void* x, void* out, const void* act, uint32_t act_rows, uint32_t N,
-                           uint32_t K, hipStream_t s) {
+hipError_t launch_mix_gemv(int dt, const void* w, const void* x, void* out, const void* act, uint32_t act_rows, int act_kind,
+                           float scale, uint32_t N, uint32_t K, hipStream_t s) {
     const bool al = ((uintptr_t)w % 16) == 0 && ((uintptr_t)x % 16) == 0;
     if (dt == kBF16) {
-        if (al && K % 8u == 0) gemv_rows<kBF16, true>(N, K, w, x, out, act, act_rows, s);
-        else gemv_rows<kBF16, false>(N, K, w, x, out, act, act_rows, s);
+        if (al && K % 8u == 0) gemv_rows<kBF16, true>(N, K, w, x, out, act, act_rows, act_kind, scale, s);
+        else gemv_rows<kBF16, false>(N, K, w, x, out, act, act_rows, act_kind, scale, s);
     } else if (dt == kFP32) {
-        if (al && K % 4u == 0) gemv_rows<kFP32, true>(N, K, w, x, out, act, act_rows, s);
-        else gemv_rows<kFP32, false>(N, K, w, x, out, act, act_rows, s);
+        if (al && K % 4u == 0) gemv_rows<kFP32, true>(N, K, w, x, out, act, act_rows, act_kind, scale, s);
+        else gemv_rows<kFP32, false>(N, K, w, x, out, act, act_rows, act_kind, scale, s);
     } else return hipErrorInvalidValue;
     return hipGetLastError();
 }
@@ -134,10 +137,12 @@ __device__ __forceinline__ void store4(void* p, size_t i, const float (&v)[4]) {
 }
 
 // ---- embedding --------------------------------------------------------------------------------------------
-template <int DT, bool VEC>
+template <int DT, bool VEC, bool NORM>
 __global__ __launch_bounds__(1024) void mix_embed_kernel(const void* __restrict__ table, const long long* __restrict__ tokens,
-                                                         float* __restrict__ x, void* __restrict__ xe, uint32_t vocab, uint32_t dim) {
+                                                         float* __restrict__ x, void* __restrict__ xe, const decdec_tanh_norm norm,
+                                                         uint32_t vocab, uint32_t dim) {
     using E = Elem<DT>;
+    const float alpha = NORM ? E::load(norm.alpha, 0) : 0.f;
     const size_t r = blockIdx.x;
     long long t = tokens[r];
     if (t < 0 || t >= (long long)vocab) t = 0;
@@ -146,32 +151,97 @@ __global__ __launch_bounds__(1024) void mix_embed_kernel(const void* __restrict_
             float v[4];
             load4<DT>(table, (size_t)t * dim + i, v);
             store4<kFP32>(x, r * dim + i, v);
+            if constexpr (NORM) {
+                float w[4], b[4];
+                load4<DT>(norm.weight, i, w);
+                load4<DT>(norm.bias, i, b);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) v[e] = __builtin_fmaf(tanhf(alpha * v[e]), w[e], b[e]);
+            }
             if (xe != nullptr) store4<DT>(xe, r * dim + i, v);
         }
     } else {
         for (uint32_t i = threadIdx.x; i < dim; i += blockDim.x) {
-            const float v = E::load(table, (size_t)t * dim + i);
+            float v = E::load(table, (size_t)t * dim + i);
             x[r * dim + i] = v;
+            if constexpr (NORM) v = __builtin_fmaf(tanhf(alpha * v), E::load(norm.weight, i), E::load(norm.bias, i));
             if (xe != nullptr) E::store(xe, r * dim + i, v);
         }
     }
 }
 
-template <int DT>
-static hipError_t embed_dt(const void* table, const long long* tokens, float* x, void* xe, uint32_t rows, uint32_t vocab, uint32_t dim,
-                           hipStream_t s) {
+template <int DT, bool NORM>
+static hipError_t embed_dt(const void* table, const long long* tokens, float* x, void* xe, const decdec_tanh_norm& norm, uint32_t rows,
+                           uint32_t vocab, uint32_t dim, hipStream_t s) {
     const uint32_t es = Elem<DT>::bytes;
-    const bool vec = dim % 4u == 0 && (uintptr_t)x % 16u == 0 && ((uintptr_t)table | (uintptr_t)xe) % (4u * es) == 0;
+    const bool vec = dim % 4u == 0 && (uintptr_t)x % 16u == 0 &&
+                     ((uintptr_t)table | (uintptr_t)xe | (uintptr_t)norm.weight | (uintptr_t)norm.bias) % (4u * es) == 0;
     uint32_t threads = 64;
     while (threads < 1024u && threads < (vec ? dim / 4u : dim)) threads *= 2;
-    if (vec) hipLaunchKernelGGL((mix_embed_kernel<DT, true>), dim3(rows), dim3(threads), 0, s, table, tokens, x, xe, vocab, dim);
-    else hipLaunchKernelGGL((mix_embed_kernel<DT, false>), dim3(rows), dim3(threads), 0, s, table, tokens, x, xe, vocab, dim);
+    if (vec) hipLaunchKernelGGL((mix_embed_kernel<DT, true, NORM>), dim3(rows), dim3(threads), 0, s, table, tokens, x, xe, norm, vocab, dim);
+    else hipLaunchKernelGGL((mix_embed_kernel<DT, false, NORM>), dim3(rows), dim3(threads), 0, s, table, tokens, x, xe, norm, vocab, dim);
     return hipGetLastError();
 }
 
-hipError_t launch_mix_embed(int dt, const void* table, const long long* tokens, float* x, void* xe, uint32_t rows,
-                            uint32_t vocab, uint32_t dim, hipStream_t s) {
-    return dt == kBF16 ? embed_dt<kBF16>(table, tokens, x, xe, rows, vocab, dim, s) : embed_dt<kFP32>(table, tokens, x, xe, rows, vocab, dim, s);
+hipError_t launch_mix_embed(int dt, const void* table, const long long* tokens, float* x, void* xe, const decdec_tanh_norm* norm,
+                            uint32_t rows, uint32_t vocab, uint32_t dim, hipStream_t s) {
+    const decdec_tanh_norm n = norm != nullptr ? *norm : decdec_tanh_norm{};
+    if (dt == kBF16) return norm != nullptr ? embed_dt<kBF16, true>(table, tokens, x, xe, n, rows, vocab, dim, s)
+                                            : embed_dt<kBF16, false>(table, tokens, x, xe, n, rows, vocab, dim, s);
+    return norm != nullptr ? embed_dt<kFP32, true>(table, tokens, x, xe, n, rows, vocab, dim, s)
+                           : embed_dt<kFP32, false>(table, tokens, x, xe, n, rows, vocab, dim, s);
+}
+
+// ---- residual with a dynamic tanh ahead of the next sublayer ------------------------------------------------
+// Element by element, 1024 elements of a row per workgroup.  Y: there is something to add.
+template <int DT, bool VEC, bool Y>
+__global__ __launch_bounds__(256) void residual_tanh_kernel(float* __restrict__ x, const void* __restrict__ y, const decdec_tanh_norm norm,
+                                                            void* __restrict__ out, const uint32_t dim) {
+    using E = Elem<DT>;
+    const size_t row = (size_t)blockIdx.x * dim;
+    const uint32_t i0 = blockIdx.y * 1024u;
+    if constexpr (VEC) {
+        const uint32_t i = i0 + 4u * threadIdx.x;
+        if (i >= dim) return;
+        float xv[4], yv[4], w[4], b[4];
+        load4<kFP32>(x, row + i, xv);
+        if constexpr (Y) load4<DT>(y, row + i, yv);
+        load4<DT>(norm.weight, i, w);
+        load4<DT>(norm.bias, i, b);
+        const float alpha = E::load(norm.alpha, 0);
+        if constexpr (Y) {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) xv[e] += yv[e];
+            store4<kFP32>(x, row + i, xv);
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) xv[e] = __builtin_fmaf(tanhf(alpha * xv[e]), w[e], b[e]);
+        store4<DT>(out, row + i, xv);
+    } else {
+        const float alpha = E::load(norm.alpha, 0);
+        for (uint32_t i = i0 + threadIdx.x; i < dim && i < i0 + 1024u; i += 256u) {
+            float v = x[row + i];
+            if constexpr (Y) { v += E::load(y, row + i); x[row + i] = v; }
+            E::store(out, row + i, __builtin_fmaf(tanhf(alpha * v), E::load(norm.weight, i), E::load(norm.bias, i)));
+        }
+    }
+}
+
+template <int DT, bool Y>
+static hipError_t residual_tanh_dt(float* x, const void* y, const decdec_tanh_norm& norm, void* out, uint32_t rows, uint32_t dim, hipStream_t s) {
+    const uint32_t es = Elem<DT>::bytes;
+    const bool vec = dim % 4u == 0 && (uintptr_t)x % 16u == 0 &&
+                     ((uintptr_t)y | (uintptr_t)out | (uintptr_t)norm.weight | (uintptr_t)norm.bias) % (4u * es) == 0;
+    const dim3 grid(rows, (dim + 1023u) / 1024u), block(256);
+    if (vec) hipLaunchKernelGGL((residual_tanh_kernel<DT, true, Y>), grid, block, 0, s, x, y, norm, out, dim);
+    else hipLaunchKernelGGL((residual_tanh_kernel<DT, false, Y>), grid, block, 0, s, x, y, norm, out, dim);
+    return hipGetLastError();
+}
+
+hipError_t launch_mix_residual_tanh(int dt, float* x, const void* y, const decdec_tanh_norm& norm, void* out, uint32_t rows,
+                                    uint32_t dim, hipStream_t s) {
+    if (dt == kBF16) return y != nullptr ? residual_tanh_dt<kBF16, true>(x, y, norm, out, rows, dim, s) : residual_tanh_dt<kBF16, false>(x, y, norm, out, rows, dim, s);
+    return y != nullptr ? residual_tanh_dt<kFP32, true>(x, y, norm, out, rows, dim, s) : residual_tanh_dt<kFP32, false>(x, y, norm, out, rows, dim, s);
 }
 
 // ---- gated residual with the norm on the sublayer's output -------------------------------------------------
@@ -307,12 +377,13 @@ hipError_t launch_mix_rmsnorm(int dt, const float* x, const void* weight, void* 
     return hipGetLastError();
 }
 
-// ---- xIELU ------------------------------------------------------------------------------------------------
-template <int DT, bool VEC>
-__global__ __launch_bounds__(256) void mix_xielu_kernel(const void* __restrict__ in, const uint32_t ld,
-                                                        const void* __restrict__ act, void* __restrict__ out, const uint32_t n) {
+// ---- activations ------------------------------------------------------------------------------------------
+template <int DT, bool VEC, int ACT>
+__global__ __launch_bounds__(256) void mix_activation_kernel(const void* in, const uint32_t ld,
+                                                        const void* __restrict__ act, void* out, const uint32_t n) {
     using E = Elem<DT>;
-    const float sp = softplus_f(E::load(act, 0)), sq = softplus_f(E::load(act, 1));
+    const float sp = ACT == DECDEC_ACT_XIELU ? softplus_f(E::load(act, 0)) : 0.f, sq = ACT == DECDEC_ACT_XIELU ? softplus_f(E::load(act, 1)) : 0.f;
+    auto f = [&](float z) { return ACT == DECDEC_ACT_XIELU ? xielu_f(z, sp, sq) : gelu_tanh_f(z); };
     const size_t irow = (size_t)blockIdx.x * ld, orow = (size_t)blockIdx.x * n;
     if constexpr (VEC) {
         // four quads a workgroup's width apart, requested together
@@ -323,30 +394,33 @@ __global__ __launch_bounds__(256) void mix_xielu_kernel(const void* __restrict__
 #pragma unroll
             for (uint32_t k = 0; k < 4u; ++k) {
 #pragma unroll
-                for (int e = 0; e < 4; ++e) v[k][e] = xielu_f(v[k][e], sp, sq);
+                for (int e = 0; e < 4; ++e) v[k][e] = f(v[k][e]);
                 if (i0 + 1024u * k < n) store4<DT>(out, orow + i0 + 1024u * k, v[k]);
             }
         }
     } else {
         for (uint32_t i = blockIdx.y * 256u + threadIdx.x; i < n; i += 256u * gridDim.y)
-            E::store(out, orow + i, xielu_f(E::load(in, irow + i), sp, sq));
+            E::store(out, orow + i, f(E::load(in, irow + i)));
     }
 }
 
-hipError_t launch_mix_xielu(int dt, const void* in, uint32_t ld, const void* act, void* out, uint32_t rows, uint32_t n,
-                            hipStream_t s) {
-    const uint32_t es = dt == kFP32 ? 4u : 2u;
+template <int DT, int ACT>
+static hipError_t activation_dt(const void* in, uint32_t ld, const void* act, void* out, uint32_t rows, uint32_t n, hipStream_t s) {
+    const uint32_t es = Elem<DT>::bytes;
     const bool vec = n % 4u == 0 && ld % 4u == 0 && (uintptr_t)in % (4 * es) == 0 && (uintptr_t)out % (4 * es) == 0;
     const uint32_t per = vec ? 4096u : 256u, gy = (n + per - 1u) / per;
     const dim3 grid(rows, gy < 16u ? gy : 16u), block(256);
-    if (dt == kBF16) {
-        if (vec) hipLaunchKernelGGL((mix_xielu_kernel<kBF16, true>), grid, block, 0, s, in, ld, act, out, n);
-        else hipLaunchKernelGGL((mix_xielu_kernel<kBF16, false>), grid, block, 0, s, in, ld, act, out, n);
-    } else {
-        if (vec) hipLaunchKernelGGL((mix_xielu_kernel<kFP32, true>), grid, block, 0, s, in, ld, act, out, n);
-        else hipLaunchKernelGGL((mix_xielu_kernel<kFP32, false>), grid, block, 0, s, in, ld, act, out, n);
-    }
+    if (vec) hipLaunchKernelGGL((mix_activation_kernel<DT, true, ACT>), grid, block, 0, s, in, ld, act, out, n);
+    else hipLaunchKernelGGL((mix_activation_kernel<DT, false, ACT>), grid, block, 0, s, in, ld, act, out, n);
     return hipGetLastError();
+}
+
+hipError_t launch_mix_activation(int dt, const void* in, uint32_t ld, const void* act, int kind, void* out, uint32_t rows,
+                                 uint32_t n, hipStream_t s) {
+    if (kind == DECDEC_ACT_GELU_TANH) return dt == kBF16 ? activation_dt<kBF16, DECDEC_ACT_GELU_TANH>(in, ld, act, out, rows, n, s)
+                                                         : activation_dt<kFP32, DECDEC_ACT_GELU_TANH>(in, ld, act, out, rows, n, s);
+    return dt == kBF16 ? activation_dt<kBF16, DECDEC_ACT_XIELU>(in, ld, act, out, rows, n, s)
+                       : activation_dt<kFP32, DECDEC_ACT_XIELU>(in, ld, act, out, rows, n, s);
 }
 
 // ---- normed, gated read-out of a recurrence ----------------------------------------------------------------
@@ -354,19 +428,19 @@ hipError_t launch_mix_xielu(int dt, const void* in, uint32_t ld, const void* act
 template <int DT>
 __global__ __launch_bounds__(1024) void group_norm_gate_kernel(const float* __restrict__ o, const void* __restrict__ gate,
                                                                const uint32_t ld, const void* __restrict__ weight,
-                                                               void* __restrict__ out, const uint32_t n, const float eps,
-                                                               const int kind) {
+                                                               void* __restrict__ out, const uint32_t out_ld, const uint32_t n,
+                                                               const float eps, const int kind, const float scale) {
     using E = Elem<DT>;
     __shared__ float red[17];
     const uint32_t r = blockIdx.x, g = blockIdx.y;
-    const size_t base = (size_t)r * n * gridDim.y + (size_t)g * n, gbase = (size_t)r * ld + (size_t)g * n;
+    const size_t base = (size_t)r * n * gridDim.y + (size_t)g * n, gbase = (size_t)r * ld + (size_t)g * n, obase = (size_t)r * out_ld + (size_t)g * n;
     float ss = 0.f;
     for (uint32_t i = threadIdx.x; i < n; i += blockDim.x) ss += o[base + i] * o[base + i];
-    const float rs = 1.f / sqrtf(block_sum(ss, red) / (float)n + eps);
+    const float rs = scale / sqrtf(block_sum(ss, red) / (float)n + eps);
     for (uint32_t i = threadIdx.x; i < n; i += blockDim.x) {
         const float z = E::load(gate, gbase + i);
         const float gt = kind == DECDEC_GATE_SILU ? silu_f(z) : sigmoid_f(z);
-        E::store(out, base + i, o[base + i] * rs * E::load(weight, i) * gt);
+        E::store(out, obase + i, o[base + i] * rs * E::load(weight, i) * gt);
     }
 }
 
@@ -374,13 +448,14 @@ __global__ __launch_bounds__(1024) void group_norm_gate_kernel(const float* __re
 template <int DT, int EP, bool FULL>
 __global__ __launch_bounds__(256) void group_norm_gate_wave_kernel(const float* __restrict__ o, const void* __restrict__ gate,
                                                                    const uint32_t ld, const void* __restrict__ weight,
-                                                                   void* __restrict__ out, const uint32_t rows, const uint32_t groups,
-                                                                   const uint32_t n, const float eps, const int kind) {
+                                                                   void* __restrict__ out, const uint32_t out_ld, const uint32_t rows,
+                                                                   const uint32_t groups, const uint32_t n, const float eps,
+                                                                   const int kind, const float scale) {
     using E = Elem<DT>;
     const uint32_t lane = threadIdx.x & 63u, at = blockIdx.x * 4u + (threadIdx.x >> 6), r = at / groups, g = at - r * groups;
     if (r >= rows) return;
     const uint32_t i0 = lane * (uint32_t)EP;
-    const size_t base = ((size_t)r * groups + g) * n, gbase = (size_t)r * ld + (size_t)g * n;
+    const size_t base = ((size_t)r * groups + g) * n, gbase = (size_t)r * ld + (size_t)g * n, obase = (size_t)r * out_ld + (size_t)g * n;
     float x[EP], z[EP], w[EP], ss = 0.f;
     if constexpr (FULL && EP == 4) {
         load4<kFP32>(o, base + i0, x);
@@ -407,28 +482,30 @@ __global__ __launch_bounds__(256) void group_norm_gate_wave_kernel(const float* 
         w[e] = E::load(weight, i);
         ss += ok ? x[e] * x[e] : 0.f;
     }
-    const float rs = 1.f / sqrtf(wave_sum(ss) / (float)n + eps);
+    const float rs = scale / sqrtf(wave_sum(ss) / (float)n + eps);
     if constexpr (FULL) {
 #pragma unroll
         for (int e = 0; e < EP; ++e) x[e] *= rs * w[e] * (kind == DECDEC_GATE_SILU ? silu_f(z[e]) : sigmoid_f(z[e]));
-        if constexpr (EP == 4) store4<DT>(out, base + i0, x);
-        else if constexpr (DT == kBF16) *(uint32_t*)((uint16_t*)out + base + i0) = pack_bf16(x[0], x[1]);
-        else *(u32x2*)((float*)out + base + i0) = u32x2{__float_as_uint(x[0]), __float_as_uint(x[1])};
+        if constexpr (EP == 4) store4<DT>(out, obase + i0, x);
+        else if constexpr (DT == kBF16) *(uint32_t*)((uint16_t*)out + obase + i0) = pack_bf16(x[0], x[1]);
+        else *(u32x2*)((float*)out + obase + i0) = u32x2{__float_as_uint(x[0]), __float_as_uint(x[1])};
         return;
     }
 #pragma unroll
     for (int e = 0; e < EP; ++e)
-        if (FULL || i0 + e < n) E::store(out, base + i0 + e, x[e] * rs * w[e] * (kind == DECDEC_GATE_SILU ? silu_f(z[e]) : sigmoid_f(z[e])));
+        if (FULL || i0 + e < n) E::store(out, obase + i0 + e, x[e] * rs * w[e] * (kind == DECDEC_GATE_SILU ? silu_f(z[e]) : sigmoid_f(z[e])));
 }
 
 // Longer groups: a workgroup each, four neighbouring elements per thread and pass.
 template <int DT, int PASSES>
 __global__ __launch_bounds__(1024) void group_norm_gate_vec_kernel(const float* __restrict__ o, const void* __restrict__ gate,
                                                                    const uint32_t ld, const void* __restrict__ weight,
-                                                                   void* __restrict__ out, const uint32_t n, const float eps, const int kind) {
+                                                                   void* __restrict__ out, const uint32_t out_ld, const uint32_t n,
+                                                                  const float eps, const int kind, const float scale) {
     __shared__ float red[17];
     const uint32_t tid = threadIdx.x;
     const size_t base = ((size_t)blockIdx.x * gridDim.y + blockIdx.y) * n, gbase = (size_t)blockIdx.x * ld + (size_t)blockIdx.y * n;
+    const size_t obase = (size_t)blockIdx.x * out_ld + (size_t)blockIdx.y * n;
     float x[PASSES][4], z[PASSES][4], w[PASSES][4], ss = 0.f;
 #pragma unroll
     for (int k = 0; k < PASSES; ++k) {
@@ -439,49 +516,50 @@ __global__ __launch_bounds__(1024) void group_norm_gate_vec_kernel(const float* 
 #pragma unroll
         for (int e = 0; e < 4; ++e) ss += i < n ? x[k][e] * x[k][e] : 0.f;
     }
-    const float rs = 1.f / sqrtf(block_sum(ss, red) / (float)n + eps);
+    const float rs = scale / sqrtf(block_sum(ss, red) / (float)n + eps);
 #pragma unroll
     for (int k = 0; k < PASSES; ++k) {
         const uint32_t i = 4u * (tid + (uint32_t)k * blockDim.x);
         if (i < n) {
 #pragma unroll
             for (int e = 0; e < 4; ++e) x[k][e] *= rs * w[k][e] * (kind == DECDEC_GATE_SILU ? silu_f(z[k][e]) : sigmoid_f(z[k][e]));
-            store4<DT>(out, base + i, x[k]);
+            store4<DT>(out, obase + i, x[k]);
         }
     }
 }
 
 template <int DT>
-static hipError_t group_norm_dt(const float* o, const void* gate, uint32_t ld, const void* weight, void* out, uint32_t rows,
-                                uint32_t groups, uint32_t n, float eps, int kind, hipStream_t s) {
+static hipError_t group_norm_dt(const float* o, const void* gate, uint32_t ld, const void* weight, void* out, uint32_t out_ld,
+                                uint32_t rows, uint32_t groups, uint32_t n, float eps, int kind, float scale, hipStream_t s) {
     const uint32_t es = Elem<DT>::bytes, waves = rows * groups;
     const dim3 wgrid((waves + 3u) / 4u), wblock(256);
     auto full = [&](uint32_t ep) {
-        return n == 64u * ep && ld % ep == 0 && (uintptr_t)o % (4u * ep) == 0 && ((uintptr_t)gate | (uintptr_t)weight | (uintptr_t)out) % (es * ep) == 0;
+        return n == 64u * ep && ld % ep == 0 && out_ld % ep == 0 && (uintptr_t)o % (4u * ep) == 0 && ((uintptr_t)gate | (uintptr_t)weight | (uintptr_t)out) % (es * ep) == 0;
     };
-    if (full(2u)) hipLaunchKernelGGL((group_norm_gate_wave_kernel<DT, 2, true>), wgrid, wblock, 0, s, o, gate, ld, weight, out, rows, groups, n, eps, kind);
-    else if (n <= 128u) hipLaunchKernelGGL((group_norm_gate_wave_kernel<DT, 2, false>), wgrid, wblock, 0, s, o, gate, ld, weight, out, rows, groups, n, eps, kind);
-    else if (full(4u)) hipLaunchKernelGGL((group_norm_gate_wave_kernel<DT, 4, true>), wgrid, wblock, 0, s, o, gate, ld, weight, out, rows, groups, n, eps, kind);
-    else if (n <= 256u) hipLaunchKernelGGL((group_norm_gate_wave_kernel<DT, 4, false>), wgrid, wblock, 0, s, o, gate, ld, weight, out, rows, groups, n, eps, kind);
+    if (full(2u)) hipLaunchKernelGGL((group_norm_gate_wave_kernel<DT, 2, true>), wgrid, wblock, 0, s, o, gate, ld, weight, out, out_ld, rows, groups, n, eps, kind, scale);
+    else if (n <= 128u) hipLaunchKernelGGL((group_norm_gate_wave_kernel<DT, 2, false>), wgrid, wblock, 0, s, o, gate, ld, weight, out, out_ld, rows, groups, n, eps, kind, scale);
+    else if (full(4u)) hipLaunchKernelGGL((group_norm_gate_wave_kernel<DT, 4, true>), wgrid, wblock, 0, s, o, gate, ld, weight, out, out_ld, rows, groups, n, eps, kind, scale);
+    else if (n <= 256u) hipLaunchKernelGGL((group_norm_gate_wave_kernel<DT, 4, false>), wgrid, wblock, 0, s, o, gate, ld, weight, out, out_ld, rows, groups, n, eps, kind, scale);
     else {
         uint32_t threads = 64;
-        const bool vec = n % 4u == 0 && ld % 4u == 0 && n <= 16384u && (uintptr_t)o % 16u == 0 &&
+        const bool vec = n % 4u == 0 && ld % 4u == 0 && out_ld % 4u == 0 && n <= 16384u && (uintptr_t)o % 16u == 0 &&
                          ((uintptr_t)gate | (uintptr_t)weight | (uintptr_t)out) % (4u * es) == 0;
         const uint32_t want = vec ? (n + 3u) / 4u : n;
         while (threads < 1024u && threads < want) threads *= 2;
         const dim3 grid(rows, groups), block(threads);
-        if (!vec) hipLaunchKernelGGL((group_norm_gate_kernel<DT>), grid, block, 0, s, o, gate, ld, weight, out, n, eps, kind);
-        else if (want <= threads) hipLaunchKernelGGL((group_norm_gate_vec_kernel<DT, 1>), grid, block, 0, s, o, gate, ld, weight, out, n, eps, kind);
-        else if (want <= 2u * threads) hipLaunchKernelGGL((group_norm_gate_vec_kernel<DT, 2>), grid, block, 0, s, o, gate, ld, weight, out, n, eps, kind);
-        else hipLaunchKernelGGL((group_norm_gate_vec_kernel<DT, 4>), grid, block, 0, s, o, gate, ld, weight, out, n, eps, kind);
+        if (!vec) hipLaunchKernelGGL((group_norm_gate_kernel<DT>), grid, block, 0, s, o, gate, ld, weight, out, out_ld, n, eps, kind, scale);
+        else if (want <= threads) hipLaunchKernelGGL((group_norm_gate_vec_kernel<DT, 1>), grid, block, 0, s, o, gate, ld, weight, out, out_ld, n, eps, kind, scale);
+        else if (want <= 2u * threads) hipLaunchKernelGGL((group_norm_gate_vec_kernel<DT, 2>), grid, block, 0, s, o, gate, ld, weight, out, out_ld, n, eps, kind, scale);
+        else hipLaunchKernelGGL((group_norm_gate_vec_kernel<DT, 4>), grid, block, 0, s, o, gate, ld, weight, out, out_ld, n, eps, kind, scale);
     }
     return hipGetLastError();
 }
 
 hipError_t launch_mix_group_norm_gate(int dt, const float* o, const void* gate, uint32_t ld, const void* weight, void* out,
-                                      uint32_t rows, uint32_t groups, uint32_t n, float eps, int kind, hipStream_t s) {
-    return dt == kBF16 ? group_norm_dt<kBF16>(o, gate, ld, weight, out, rows, groups, n, eps, kind, s)
-                       : group_norm_dt<kFP32>(o, gate, ld, weight, out, rows, groups, n, eps, kind, s);
+                                      uint32_t out_ld, uint32_t rows, uint32_t groups, uint32_t n, float eps, int kind,
+                                      float scale, hipStream_t s) {
+    return dt == kBF16 ? group_norm_dt<kBF16>(o, gate, ld, weight, out, out_ld, rows, groups, n, eps, kind, scale, s)
+                       : group_norm_dt<kFP32>(o, gate, ld, weight, out, out_ld, rows, groups, n, eps, kind, scale, s);
 }
 
 }  // namespace decdec

@@ -77,6 +77,48 @@ __device__ __forceinline__ void frag_split(const float (&x)[8], Frag<kFP32>& hi,
 template <int DT> struct LaneOf { using t = uint16_t; };
 template <> struct LaneOf<kFP32> { using t = float; };
 
+// eight elements of a row as a fragment, zero past `valid`
+template <int DT>
+__device__ __forceinline__ Frag<DT> load8(const typename LaneOf<DT>::t* p, int valid, bool vec) {
+    if (vec && valid >= 8) return frag_load(p);
+    Frag<DT> f;
+    if constexpr (DT == kFP32) {
+#pragma unroll
+        for (int i = 0; i < 8; ++i) f.v[i] = i < valid ? p[i] : 0.f;
+    } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+            f.v[i] = (uint32_t)(2 * i < valid ? p[2 * i] : 0) | ((uint32_t)(2 * i + 1 < valid ? p[2 * i + 1] : 0) << 16);
+    }
+    return f;
+}
+__device__ __forceinline__ void store8(uint16_t* p, const Frag<kBF16>& f) { *(u32x4*)p = f.v; }
+__device__ __forceinline__ void store8(float* p, const Frag<kFP32>& f) {
+#pragma unroll
+    for (int i = 0; i < 8; i += 4) *(f32x4*)(p + i) = f32x4{f.v[i], f.v[i + 1], f.v[i + 2], f.v[i + 3]};
+}
+__device__ __forceinline__ void frag_values(const Frag<kBF16>& f, float (&x)[8]) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) { x[2 * i] = __uint_as_float(f.v[i] << 16); x[2 * i + 1] = __uint_as_float(f.v[i] & 0xFFFF0000u); }
+}
+__device__ __forceinline__ void frag_values(const Frag<kFP32>& f, float (&x)[8]) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) x[i] = f.v[i];
+}
+
+__device__ __forceinline__ Frag<kBF16> frag_of(const float (&x)[8], const Frag<kBF16>&) {
+    Frag<kBF16> f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) f.v[i] = pack_bf16(x[2 * i], x[2 * i + 1]);
+    return f;
+}
+__device__ __forceinline__ Frag<kFP32> frag_of(const float (&x)[8], const Frag<kFP32>&) {
+    Frag<kFP32> f;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) f.v[i] = x[i];
+    return f;
+}
+
 constexpr float kLog2e = 1.4426950408889634f;
 
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + __expf(-z)); }
@@ -96,6 +138,11 @@ __device__ __forceinline__ float xielu_f(float z, float sp, float sq) {
     s = __builtin_fmaf(s, n, 0.5f) * n * n;
     const float e = n > -0.7f ? s : __expf(n) - 1.f - n;
     return z > 0.f ? (sp * z + 0.5f) * z : (0.5f + sq) * e + 0.5f * z;
+}
+
+// GELU, tanh form: z (1 + tanh u) / 2 = z sigmoid(2 u)
+__device__ __forceinline__ float gelu_tanh_f(float z) {
+    return z * sigmoid_f(1.5957691216057308f * (z + 0.044715f * z * z * z));
 }
 
 // Sum over a workgroup of `blockDim.x` (a multiple of 64) threads; red: at least 17 floats of LDS, free at the call.

@@ -8,10 +8,10 @@ import os
 
 import torch
 
-from .hybrid import HybridDecoder
+from .hybrid import HybridDecoder, PreNormDecoder
 
 # architectures a checkpoint's config.json may name
-ARCHITECTURES = {"Fivitar": HybridDecoder}
+ARCHITECTURES = {"Fivitar": HybridDecoder, "Fekulix": PreNormDecoder}
 
 
 def model_class(config: dict):

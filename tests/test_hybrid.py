@@ -124,7 +124,8 @@ def test_mixers_library_exports_what_the_header_declares():
     assert names == set(_lib.MIXERS_SIGNATURES) | set(_lib.MIXERS_OTHER)
     assert all(hasattr(lib, n) for n in names)
     # the ctypes mirrors list the fields of the C structs in order
-    for cls, tag in ((_lib.Recurrence, "decdec_recurrence"), (_lib.Latent, "decdec_latent")):
+    for cls, tag in ((_lib.Recurrence, "decdec_recurrence"), (_lib.Latent, "decdec_latent"), (_lib.Grouped, "decdec_grouped"),
+                     (_lib.TanhNorm, "decdec_tanh_norm")):
         body = re.sub(r"/\*.*?\*/", "", text, flags=re.S)
         body = body[:body.index("} " + tag + ";")]
         body = body[body.rindex("typedef struct {") + len("typedef struct {"):]
@@ -135,8 +136,8 @@ def test_mixers_library_exports_what_the_header_declares():
 def test_arguments_are_checked_before_any_launch():
     lib = _lib.load_mixers()
     err = lambda: lib.decdec_mixers_last_error().decode()
-    assert lib.decdec_mix_gemv(None, None, None, None, 0, 0, 8, 8, None) != 0 and "null pointer" in err()
-    assert lib.decdec_mix_gemv(8, 8, 8, None, 0, 1, 8, 8, None) != 0 and "fp32 or bf16" in err()
+    assert lib.decdec_mix_gemv(None, None, None, None, 0, 0, 1.0, 0, 8, 8, None) != 0 and "null pointer" in err()
+    assert lib.decdec_mix_gemv(8, 8, 8, None, 0, 0, 1.0, 1, 8, 8, None) != 0 and "fp32 or bf16" in err()
     r = _lib.Recurrence(proj=16, state=16, pos=16, heads=3, kv_heads=2, dim=8, vdim=8, ld=1000)
     assert lib.decdec_mix_recurrence_step(r, 16, None, None, 0.0, 0, 0, None) != 0 and "multiple of kv_heads" in err()
     r = _lib.Recurrence(proj=16, state=16, pos=16, heads=2, kv_heads=2, dim=300, vdim=8, ld=1000)
