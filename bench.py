@@ -520,23 +520,35 @@ def helpers_leg(torch):
 HYBRID_SIZES = {"2048": dict(width=2048, heads=16, kv_heads=8, ff=7168), "4096": dict(width=4096, heads=32, kv_heads=8, ff=14336)}
 
 
-def hybrid_config(kind, width, heads, ff, layers, vocab, kv_heads=None):
-    mixers = {"lightning": {"heads": heads, "dim": 128, "vdim": 128, "decay": [1.0 - 2.0 ** (-2 - 6 * i / heads) for i in range(heads)]},
-              "delta": {"heads": heads, "kv_heads": heads // 2, "dim": 128, "vdim": 128, "conv": 4},
-              "latent_attention": {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5,
-                                   "rot": {"base": 10000.0, "dims": 64, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
+def hybrid_config(kind, width, heads, ff, layers, vocab, kv_heads=None, design="Fivitar"):
+    """`kind`: one of the design's mixers for all layers, or "mixed": all of them in turn."""
+    mixers = {"Fivitar": {"lightning": {"heads": heads, "dim": 128, "vdim": 128, "decay": [1.0 - 2.0 ** (-2 - 6 * i / heads) for i in range(heads)]},
+                          "delta": {"heads": heads, "kv_heads": heads // 2, "dim": 128, "vdim": 128, "conv": 4},
+                          "latent_attention": {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5,
+                                               "rot": {"base": 10000.0, "dims": 64,
+                                                       "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}},
+              "Fekulix": {"parallel": {"left": {"heads": heads, "kv_heads": kv_heads, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                                                "rot": {"base": 10000.0, "dims": 64}},
+                                       "right": {"heads": heads // 2, "dim": 128, "vdim": 128, "tau": 16.0}, "left_scale": 0.7, "right_scale": 0.6},
+                          "channel_delta": {"heads": heads, "kv_heads": heads // 2, "dim": 128, "vdim": 128, "conv": 4}}}[design]
     kinds = list(mixers) if kind == "mixed" else [kind]
-    return {"architecture": "Fivitar", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+    return {"architecture": design, "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "logit_scale": 1.0,
             "layers": [{"type": kinds[i % len(kinds)], "mixer": mixers[kinds[i % len(kinds)]], "mlp": {"kind": "dense", "ff": ff}}
                        for i in range(layers)]}
 
 
-def hybrid_leg(torch, sizes, layers=6, prompts=(512, 2048, 8192), positions=(512, 2048, 8192), vocab=32000):
-    """Prefill and decode of `layers` layers (random bf16 weights, dense) per size: the Fivitar decoder with its three
-    mixers in turn and with each alone, and the plain decoder (grouped-query attention, SwiGLU) of the same width, head
-    count and feed-forward size with dense bf16 linears."""
+# models of a leg: (design, kind)
+HYBRID_LEGS = {"fivitar": [("plain", "plain")] + [("Fivitar", k) for k in ("mixed", "lightning", "delta", "latent_attention")],
+               "fekulix": [("plain", "plain"), ("Fivitar", "mixed"), ("Fivitar", "delta")] +
+                          [("Fekulix", k) for k in ("mixed", "parallel", "channel_delta")]}
+
+
+def hybrid_leg(torch, sizes, leg="fivitar", layers=6, prompts=(512, 2048, 8192), positions=(512, 2048, 8192), vocab=32000):
+    """Prefill and decode of `layers` layers (random bf16 weights, dense) per size: the leg's decoder with its mixers in turn
+    and with each alone, and beside it the plain decoder (grouped-query attention, SwiGLU) of the same width, head count and
+    feed-forward size with dense bf16 linears; the Fekulix leg also runs the Fivitar decoder, the closest of the others."""
     from decdec_amd.generate import DecodeStep, Session
-    from decdec_amd.hybrid import HybridDecoder
+    from decdec_amd import registry
     from decdec_amd.model import ModelArgs, Transformer
 
     def plain(width, heads, kv_heads, ff):
@@ -546,13 +558,14 @@ def hybrid_leg(torch, sizes, layers=6, prompts=(512, 2048, 8192), positions=(512
     rows = []
     for size in sizes:
         z = HYBRID_SIZES[size]
-        for kind in ("plain", "mixed", "lightning", "delta", "latent_attention"):
+        for design, kind in HYBRID_LEGS[leg]:
             if kind == "plain":
                 m = plain(**z)
             else:
-                m = HybridDecoder.from_config(hybrid_config(kind, layers=layers, vocab=vocab, **z), torch.bfloat16)
+                cfg = hybrid_config(kind, layers=layers, vocab=vocab, design=design, **z)
+                m = registry.model_class(cfg).from_config(cfg, torch.bfloat16)
                 m.init_random_weights(0)
-            row = {"size": size, "model": kind, "layers": layers, "parameters": sum(t.numel() for t in list(m.parameters()) + list(m.buffers()))}
+            row = {"size": size, "design": design, "model": kind, "layers": layers, "parameters": sum(t.numel() for t in list(m.parameters()) + list(m.buffers()))}
             gen = torch.Generator().manual_seed(0)
             toks = torch.randint(0, vocab, (max(prompts + positions) + 1,), generator=gen).cuda()
             for n in prompts:
@@ -640,15 +653,15 @@ def main():
     ap.add_argument("--n-tb", type=int, default=32, help="workgroups DEC may occupy (the sweep shows 8..64)")
     ap.add_argument("--sweep", action="store_true", help="also sweep k_chunk x n_tb (slower)")
     ap.add_argument("--no-cpu-baseline", action="store_true")
-    ap.add_argument("--leg", choices=["all", "token", "roofline", "kernels", "helpers", "link", "trace", "fivitar"], default="all",
+    ap.add_argument("--leg", choices=["all", "token", "roofline", "kernels", "helpers", "link", "trace", *HYBRID_LEGS], default="all",
                     help="token: only the token (batched, one launch per layer, graph branches; with DEC and base-only); "
                          "roofline: only the roofline kernel's launches and a 256 MiB device copy (short run for counter "
                          "collection); kernels: per-kernel table over the configuration shapes (k_chunk 32, n_tb 32); "
                          "helpers: the decode harness's helper kernels (output head, attention, norm, activation); "
                          "link: zero-copy reads of pinned host memory over workgroup counts and request widths; "
                          "trace: phase timings of DEC-only launches from the role's own cycle stamps; "
-                         "fivitar: prefill and decode of the Fivitar decoder beside the plain decoder of the same size")
-    ap.add_argument("--size", nargs="+", choices=sorted(HYBRID_SIZES), default=sorted(HYBRID_SIZES), help="widths of --leg fivitar")
+                         "fivitar, fekulix: prefill and decode of that decoder beside the plain decoder (fekulix: and Fivitar) of the same size")
+    ap.add_argument("--size", nargs="+", choices=sorted(HYBRID_SIZES), default=sorted(HYBRID_SIZES), help="widths of --leg fivitar and fekulix")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this path runs on one GPU; --gpus N with N > 1 is not part of this build", file=sys.stderr)
@@ -663,8 +676,8 @@ def main():
     if args.leg == "helpers":
         print(json.dumps({"helpers": helpers_leg(torch)}))
         return
-    if args.leg == "fivitar":
-        print(json.dumps({"fivitar": hybrid_leg(torch, args.size)}))
+    if args.leg in HYBRID_LEGS:
+        print(json.dumps({args.leg: hybrid_leg(torch, args.size, args.leg)}))
         return
     if args.leg == "link":
         print(json.dumps({"link": link_leg(torch, full=True)}))

@@ -230,33 +230,40 @@ hipError_t launch_tile_attention(int dt, const TileAttention& p, uint32_t start,
 // elements turned.  A lane takes elements 2 lane + 128 j and the next; dim is at most 320.
 constexpr int kPairs = 3;
 
+struct HeadRow { float x[kPairs][2], w[kPairs][2], c[kPairs], s[kPairs]; };
 template <int DT>
-__device__ __forceinline__ void norm_rotate(const void* proj, size_t at, const void* weight, const decdec_grouped& p, size_t trow,
-                                            float (&x)[kPairs][2]) {
+__device__ __forceinline__ HeadRow head_fetch(const void* proj, size_t at, const void* weight, const decdec_grouped& p, size_t trow) {
     using E = Elem<DT>;
     const uint32_t lane = threadIdx.x & 63u, D = p.dim;
-    float ss = 0.f, w[kPairs][2];
-#pragma unroll
-    for (int j = 0; j < kPairs; ++j)
-#pragma unroll
-        for (uint32_t e = 0; e < 2u; ++e) {
-            const uint32_t i = 2u * lane + 128u * (uint32_t)j + e;
-            x[j][e] = i < D ? E::load(proj, at + i) : 0.f;
-            w[j][e] = (weight != nullptr && i < D) ? E::load(weight, i) : 1.f;
-            ss += x[j][e] * x[j][e];
-        }
-    const float r = weight != nullptr ? 1.f / sqrtf(wave_sum(ss) / (float)D + p.eps) : 1.f;
+    HeadRow f;
 #pragma unroll
     for (int j = 0; j < kPairs; ++j) {
-        const uint32_t i = 2u * lane + 128u * (uint32_t)j;
-        float u = x[j][0] * r * w[j][0], v = x[j][1] * r * w[j][1];
-        if (i < p.rot) {
-            const float c = p.cos_table[trow + i / 2u], s = p.sin_table[trow + i / 2u], u0 = u;
-            u = u0 * c - v * s;
-            v = v * c + u0 * s;
+        const uint32_t i0 = 2u * lane + 128u * (uint32_t)j;
+        const bool turn = i0 < p.rot;
+#pragma unroll
+        for (uint32_t e = 0; e < 2u; ++e) {
+            const bool in = i0 + e < D;
+            f.x[j][e] = in ? E::load(proj, at + i0 + e) : 0.f;
+            f.w[j][e] = (weight != nullptr && in) ? E::load(weight, i0 + e) : 1.f;
         }
-        x[j][0] = u;
-        x[j][1] = v;
+        f.c[j] = turn ? p.cos_table[trow + i0 / 2u] : 1.f;
+        f.s[j] = turn ? p.sin_table[trow + i0 / 2u] : 0.f;
+    }
+    return f;
+}
+__device__ __forceinline__ void norm_rotate(const HeadRow& f, bool norm, const decdec_grouped& p, float (&x)[kPairs][2]) {
+    float r = 1.f;
+    if (norm) {
+        float ss = 0.f;
+#pragma unroll
+        for (int j = 0; j < kPairs; ++j) ss += f.x[j][0] * f.x[j][0] + f.x[j][1] * f.x[j][1];
+        r = 1.f / sqrtf(wave_sum(ss) / (float)p.dim + p.eps);
+    }
+#pragma unroll
+    for (int j = 0; j < kPairs; ++j) {
+        const float u = f.x[j][0] * r * f.w[j][0], v = f.x[j][1] * r * f.w[j][1];
+        x[j][0] = u * f.c[j] - v * f.s[j];
+        x[j][1] = v * f.c[j] + u * f.s[j];
     }
 }
 
@@ -285,11 +292,55 @@ __global__ __launch_bounds__(256) void grouped_append_kernel(const decdec_groupe
     if (pos < 0 || pos >= (long long)p.max_seq) return;
     const bool isq = j < p.heads;
     const uint32_t h = isq ? j : j - p.heads;
+    const void* weight = isq ? p.q_norm : p.k_norm;
     float x[kPairs][2];
-    norm_rotate<DT>(p.proj, (size_t)t * p.ld + (isq ? p.off_q : p.off_k) + h * p.dim, isq ? p.q_norm : p.k_norm, p,
-                    (size_t)pos * (p.rot / 2u), x);
+    norm_rotate(head_fetch<DT>(p.proj, (size_t)t * p.ld + (isq ? p.off_q : p.off_k) + h * p.dim, weight, p, (size_t)pos * (p.rot / 2u)),
+                weight != nullptr, p, x);
     if (isq) store_pairs<DT>(q_out, ((size_t)t * p.heads + h) * p.dim, p.dim, x);
     else store_pairs<DT>(p.keys, ((size_t)h * p.max_seq + (size_t)pos) * p.dim, p.dim, x);
+}
+
+// The same for dim a multiple of 8 and rot of 8: gl lanes share a head, eight neighbouring elements each.
+template <int DT>
+__global__ __launch_bounds__(256) void grouped_append_vec_kernel(const decdec_grouped p, void* __restrict__ q_out, const uint32_t rows,
+                                                                 const uint32_t gl) {
+    using T = typename LaneOf<DT>::t;
+    const uint32_t all = p.heads + p.kv_heads, D = p.dim, sub = threadIdx.x % gl, c = 8u * sub;
+    const uint32_t at = blockIdx.x * (256u / gl) + threadIdx.x / gl, t = at / all, j = at - t * all;
+    const long long pos = *p.pos + (long long)t;
+    const bool ok = t < rows && pos >= 0 && pos < (long long)p.max_seq, live = ok && c < D, isq = j < p.heads;
+    const uint32_t h = isq ? j : j - p.heads;
+    const void* weight = isq ? p.q_norm : p.k_norm;
+    const size_t trow = (size_t)(ok ? pos : 0) * (p.rot / 2u);
+    float x[8], w[8], cs[4], sn[4], ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) { x[e] = 0.f; w[e] = 1.f; }
+    if (live) {
+        frag_values(frag_load((const T*)p.proj + (size_t)t * p.ld + (isq ? p.off_q : p.off_k) + h * D + c), x);
+        if (weight != nullptr) frag_values(frag_load((const T*)weight + c), w);
+    }
+    const bool turn = live && c < p.rot;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+        cs[e] = turn ? p.cos_table[trow + c / 2u + e] : 1.f;
+        sn[e] = turn ? p.sin_table[trow + c / 2u + e] : 0.f;
+    }
+    float r = 1.f;
+    if (weight != nullptr) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) ss += x[e] * x[e];
+    }
+    for (uint32_t off = 1; off < gl; off <<= 1) ss += __shfl_xor(ss, (int)off, 64);
+    if (weight != nullptr) r = 1.f / sqrtf(ss / (float)D + p.eps);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+        const float u = x[2 * e] * r * w[2 * e], v = x[2 * e + 1] * r * w[2 * e + 1];
+        x[2 * e] = u * cs[e] - v * sn[e];
+        x[2 * e + 1] = v * cs[e] + u * sn[e];
+    }
+    if (!live) return;
+    T* dst = isq ? (T*)q_out + ((size_t)t * p.heads + h) * D + c : (T*)p.keys + ((size_t)h * p.max_seq + (size_t)pos) * D + c;
+    store8(dst, frag_of(x, Frag<DT>{}));
 }
 
 // Values, transposed, to the cache: grid (tokens / 64, channels / 64).
@@ -308,7 +359,13 @@ __global__ __launch_bounds__(256) void grouped_values_kernel(const decdec_groupe
 
 template <int DT>
 static hipError_t grouped_append_dt(const decdec_grouped& p, void* q_out, uint32_t rows, hipStream_t s) {
-    hipLaunchKernelGGL((grouped_append_kernel<DT>), dim3((rows * (p.heads + p.kv_heads) + 3u) / 4u), dim3(256), 0, s, p, q_out, rows);
+    const uint32_t all = rows * (p.heads + p.kv_heads);
+    uint32_t gl = 1;
+    while (8u * gl < p.dim) gl *= 2;                        // at most 64: dim is at most 320
+    const bool vec = (p.dim | p.rot | p.ld | p.off_q | p.off_k) % 8u == 0 &&
+                     ((uintptr_t)p.proj | (uintptr_t)p.q_norm | (uintptr_t)p.k_norm) % 16u == 0;
+    if (vec) hipLaunchKernelGGL((grouped_append_vec_kernel<DT>), dim3((all + 256u / gl - 1u) / (256u / gl)), dim3(256), 0, s, p, q_out, rows, gl);
+    else hipLaunchKernelGGL((grouped_append_kernel<DT>), dim3((all + 3u) / 4u), dim3(256), 0, s, p, q_out, rows);
     hipLaunchKernelGGL((grouped_values_kernel<DT>), dim3((rows + 63u) / 64u, (p.kv_heads * p.vdim + 63u) / 64u), dim3(256), 0, s, p, rows);
     return hipGetLastError();
 }
@@ -358,7 +415,7 @@ __global__ __launch_bounds__(256, 1) void grouped_step_kernel(const decdec_group
     constexpr uint32_t PAD = DT == kFP32 ? 4u : 8u, QL = 32u * NK + PAD, OL = 16u * NV + 4u, UNIT = 64u * KB;
     extern __shared__ __align__(16) float ol[];             // [4][16][OL]
     __shared__ __align__(16) T Ql[16][QL];
-    __shared__ T knew[32 * NK];
+    __shared__ T knew[32 * NK], vnew[256];
     __shared__ float mxs[4][16], sums[4][16], snew[16];
     const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, l16 = lane & 15u, lg = lane >> 4;
     const uint32_t kvh = blockIdx.y, share = p.heads / p.kv_heads, g0 = blockIdx.z * 16u, D = p.dim, V = p.vdim;
@@ -406,21 +463,33 @@ __global__ __launch_bounds__(256, 1) void grouped_step_kernel(const decdec_group
             }
         }
     };
+    // the wave's first query head and the new key ahead of the cache: memory answers in order
+    const size_t trow = (size_t)pos * (p.rot / 2u);
+    const HeadRow q0 = head_fetch<DT>(p.proj, p.off_q + (size_t)(h0 + (wave < nh ? wave : 0u)) * D, p.q_norm, p, trow);
+    HeadRow kn{};
+    T vn = (T)0;
+    if (first) {
+        if (wave == 3u) kn = head_fetch<DT>(p.proj, p.off_k + (size_t)kvh * D, p.k_norm, p, trow);
+        if (tid < V) vn = ((const T*)p.proj)[p.off_v + kvh * V + tid];
+    }
     uint32_t k0 = lo + wave * 16u * KB;
     if (k0 < hi) request(k0);
-    const size_t trow = (size_t)pos * (p.rot / 2u);
     for (uint32_t i = tid; i < 16u * 32u * NK; i += 256u) {                // zeros past dim and past the last head
         const uint32_t r = i / (32u * NK), c = i % (32u * NK);
         if (r >= nh || c >= D) Ql[r][c] = (T)0;
     }
     for (uint32_t j = wave; j < nh; j += 4u) {
         float x[kPairs][2];
-        norm_rotate<DT>(p.proj, p.off_q + (size_t)(h0 + j) * D, p.q_norm, p, trow, x);
+        norm_rotate(j == wave ? q0 : head_fetch<DT>(p.proj, p.off_q + (size_t)(h0 + j) * D, p.q_norm, p, trow), p.q_norm != nullptr, p, x);
         store_pairs<DT>(&Ql[j][0], 0, D, x);
+    }
+    if (first && tid < V) {
+        vnew[tid] = vn;
+        if (blockIdx.z == 0u) ((T*)p.values)[(size_t)(kvh * V + tid) * p.max_seq + (size_t)pos] = vn;
     }
     if (first && wave == 3u) {
         float x[kPairs][2];
-        norm_rotate<DT>(p.proj, p.off_k + (size_t)kvh * D, p.k_norm, p, trow, x);
+        norm_rotate(kn, p.k_norm != nullptr, p, x);
         store_pairs<DT>(knew, 0, D, x);
         if (blockIdx.z == 0u) store_pairs<DT>(p.keys, ((size_t)kvh * p.max_seq + (size_t)pos) * D, D, x);
     }
@@ -431,9 +500,6 @@ __global__ __launch_bounds__(256, 1) void grouped_step_kernel(const decdec_group
 #pragma unroll
     for (int n = 0; n < NV; ++n) o[n] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (first) {
-        if (blockIdx.z == 0u)
-            for (uint32_t d = tid; d < V; d += 256u)
-                ((T*)p.values)[(size_t)(kvh * V + d) * p.max_seq + (size_t)pos] = ((const T*)p.proj)[p.off_v + kvh * V + d];
         const uint32_t r = tid >> 4, c = tid & 15u;
         float x = 0.f;
         for (uint32_t i = c; i < D; i += 16u) x = __builtin_fmaf(E::load(&Ql[r][0], i), E::load(knew, i), x);
@@ -449,7 +515,7 @@ __global__ __launch_bounds__(256, 1) void grouped_step_kernel(const decdec_group
 #pragma unroll
                 for (int v = 0; v < 4; ++v) {
                     const uint32_t d = 16u * (uint32_t)n + 4u * lg + (uint32_t)v;
-                    o[n][v] = d < V ? E::load(p.proj, p.off_v + kvh * V + d) : 0.f;
+                    o[n][v] = d < V ? E::load(vnew, d) : 0.f;
                 }
         }
     }

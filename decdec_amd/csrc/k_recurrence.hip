@@ -591,9 +591,8 @@ __global__ __launch_bounds__(256) void delta_solve_kernel(const ChunkParams p) {
 
 // Decays per key channel: what the later kernels need of a chunk and head, and U and W for the delta rule: grid (chunks,
 // heads).  Exponents are sums of log-decays (in units of log 2) from a block's start to a token, from a token to its block's
-// end, and over whole blocks of 16 tokens: never a difference of sums, and never positive.  Scores between different blocks
-// are products of the scaled rows; inside a block the exponential of the difference of two tokens' sums is taken channel by
-// channel.
+// end, and over whole blocks of 16 tokens, none of them positive.  Scores between different blocks are products of the
+// scaled rows; inside a block the exponential of the difference of two tokens' sums is taken channel by channel.
 template <bool DELTA, bool FULL>
 __global__ __launch_bounds__(256) void channel_chunk_kernel(const ChunkParams p) {
     __shared__ __align__(16) float buf[5][C][36];
@@ -625,7 +624,8 @@ __global__ __launch_bounds__(256) void channel_chunk_kernel(const ChunkParams p)
 #pragma unroll
             for (uint32_t j = 0; j < 4u; ++j) {
                 const bool in = r < n && (FULL || c0 + c + j < D);
-                x[j] = in ? channel_log_decay(rate2, p.a_sign, as.x[e][j], p.a_bias[h * D + c0 + c + j]) : 0.f;
+                // no float is as small as 2^-160: a bound that changes no product and keeps later differences sharp
+                x[j] = in ? fmaxf(channel_log_decay(rate2, p.a_sign, as.x[e][j], p.a_bias[h * D + c0 + c + j]), -160.f) : 0.f;
             }
             *(f32x4*)&Ls[r][c] = x;
         }

@@ -201,14 +201,19 @@ def sink_attention(q, k, v, scale, sink=0.0):
 
 
 def gated_attention(h, w, cfg, eps):
-    """Grouped-query attention with normed, partly rotated queries and keys, a sink and one gate per head: read-out."""
+    """Grouped-query attention with partly rotated queries and keys: read-out.  Normed queries and keys where w has their
+    weights, one gate per head where it has one, a sink of score 0 unless cfg says otherwise (None: none)."""
     T, H, G, D, V = h.shape[0], cfg["heads"], cfg["kv_heads"], cfg["dim"], cfg["vdim"]
     pos = torch.arange(T)
-    q = rms_norm((h @ w["q"].T).view(T, H, D), w["q.norm"], eps).transpose(0, 1)
-    k = rms_norm((h @ w["k"].T).view(T, G, D), w["k.norm"], eps).transpose(0, 1)
-    v = (h @ w["v"].T).view(T, G, V).transpose(0, 1)
-    o = sink_attention(rotate(q, pos, cfg["rot"]), rotate(k, pos, cfg["rot"]), v, cfg["scale"])
-    return (o * sigmoid(h @ w["g"].T)[:, :, None]).reshape(T, H * V)
+    q, k, v = ((h @ w[n].T).view(T, g, -1) for n, g in (("q", H), ("k", G), ("v", G)))
+    if "q.norm" in w:
+        q, k = rms_norm(q, w["q.norm"], eps), rms_norm(k, w["k.norm"], eps)
+    sink = cfg.get("sink", 0.0)
+    o = sink_attention(rotate(q.transpose(0, 1), pos, cfg["rot"]), rotate(k.transpose(0, 1), pos, cfg["rot"]), v.transpose(0, 1),
+                       cfg["scale"], -math.inf if sink is None else sink)
+    if "g" in w:
+        o = o * sigmoid(h @ w["g"].T)[:, :, None]
+    return o.reshape(T, H * V)
 
 
 def gated_linear(h, w, cfg, eps):

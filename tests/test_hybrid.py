@@ -9,9 +9,10 @@ import pytest
 import torch
 
 from decdec_amd import _lib, registry
-from decdec_amd.cache import KVCache, LatentCache, RecurrentState, SequenceState
+from decdec_amd.cache import GroupedCache, JoinedState, KVCache, LatentCache, RecurrentState, SequenceState
 from decdec_amd.generate import Session
-from decdec_amd.hybrid import HybridConfig, HybridDecoder
+from decdec_amd.hybrid import HybridConfig, HybridDecoder, PreNormDecoder
+from decdec_amd.mixers import LinearRecurrence, Workspace
 from decdec_amd.model import ModelArgs, Transformer, rope_frequencies, rope_tables
 from oracle import hybrid_oracle as O
 import hybrid_cases as cases
@@ -23,18 +24,21 @@ ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 def test_every_tensor_of_a_configuration_is_expected_by_name_and_shape(name):
     cfg = cases.CONFIGS[name]()
     model = registry.model_class(cfg).from_config(cfg, torch.float32, device="cpu")
+    for i, layer in model.weights.items():
+        layer.fit({n[len(f"l{i}."):]: s for n, s in cases.shapes(cfg).items() if n.startswith(f"l{i}.")})
     assert {n: tuple(s) for n, s in model.weight_shapes().items()} == cases.shapes(cfg)
 
 
-def test_checkpoint_folder_round_trip(tmp_path):
+@pytest.mark.parametrize("make,gone", [(cases.config_odd, "l2.norm1"), (cases.config_fek_odd, "l0.norm1.alpha"), (cases.config_fek_odd, "l0.mix.a1")])
+def test_checkpoint_folder_round_trip(make, gone, tmp_path):
     from safetensors.torch import save_file
-    cfg = cases.config_odd()
+    cfg = make()
     w = cases.weights(cfg)
     (tmp_path / "config.json").write_text(json.dumps(cfg))
     assert registry.is_checkpoint(str(tmp_path)) and registry.read_config(str(tmp_path)) == cfg
-    del w["l2.norm1"]
+    del w[gone]
     save_file(w, str(tmp_path / "model.safetensors"))
-    with pytest.raises(KeyError, match="l2.norm1"):
+    with pytest.raises(KeyError, match=gone):
         registry.load_model(str(tmp_path), torch.float32, device="cpu")
     with pytest.raises(KeyError, match="Unknown architecture"):
         registry.model_class({"architecture": "no-such-design"})
@@ -55,6 +59,17 @@ def test_configuration_errors_are_named():
     cfg["layers"][0]["mixer"]["decay"] = [0.5, 0.5]
     with pytest.raises(ValueError, match="decays for 1 heads"):
         HybridDecoder.from_config(cfg, torch.float32, device="cpu")
+    cfg = cases.config_fek_odd()
+    cfg["layers"][1]["mixer"]["left"]["kv_heads"] = 4
+    with pytest.raises(ValueError, match="do not divide"):
+        PreNormDecoder.from_config(cfg, torch.float32, device="cpu")
+
+
+def test_a_recurrence_has_one_kind_of_decay():
+    ws = Workspace("cpu")
+    for bad in (dict(), dict(decay=[0.5, 0.5], conv=4), dict(channel=True), dict(channel=True, conv=4, tau=2.0), dict(conv=4, low_rank_gate=True)):
+        with pytest.raises(ValueError):
+            LinearRecurrence(2, 8, 8, ws, **bad)
 
 
 def test_layers_that_share_weights_keep_states_of_their_own():
@@ -66,7 +81,9 @@ def test_sequence_state_counts_and_restores():
     rec = RecurrentState(2, 4, 3, "cpu", taps=2, channels=5, dtype=torch.float32)
     lat = LatentCache(70, 6, 2, torch.float32, "cpu")
     assert lat.rows.shape == (128, 8)
-    st = SequenceState([rec, lat, KVCache(1, 8, 1, 4, torch.float32, "cpu")], max_tokens=10)
+    grp = GroupedCache(70, 2, 6, 5, torch.float32, "cpu")
+    assert grp.keys.shape == (2, 128, 6) and grp.values.shape == (10, 128)
+    st = SequenceState([JoinedState([grp, rec]), lat, KVCache(1, 8, 1, 4, torch.float32, "cpu")], max_tokens=10)
     st.advance(0, 4)
     with pytest.raises(ValueError, match="start at position 3"):
         st.advance(3, 1)
@@ -157,3 +174,48 @@ def test_oracle_is_causal_and_a_missing_mechanism_shows():
         other = dict(w)
         other[change] = w[change] + 1.0
         assert not torch.allclose(O.forward(cfg, other, toks), full, atol=1e-3), change
+
+
+def test_fekulix_oracle_is_causal_and_every_tensor_shows():
+    cfg = cases.config_fek_odd()
+    w, toks = cases.weights(cfg, 3), cases.tokens(cfg, 20)
+    full = O.forward(cfg, w, toks)
+    assert torch.allclose(O.forward(cfg, w, toks[:13]), full[:13])
+    for change in w:
+        other = {**w, change: w[change] * 1.3 + 0.2}
+        assert not torch.allclose(O.forward(cfg, other, toks), full, atol=1e-3), change
+
+
+def test_fekulix_oracle_tells_mistakes_apart(monkeypatch):
+    """Mistakes planted in the oracle move the logits by far more than the tolerance of the GPU tests."""
+    cfg = cases.config_fek_odd()
+    w, toks = cases.weights(cfg, 3), cases.tokens(cfg, 40)
+    full = O.forward(cfg, w, toks)
+    attention, rotate, O_sum = O.sink_attention, O.rotate, O.channel_decayed_sum
+
+    def half_layout(x, positions, rot):
+        n = rot["dims"]
+        order = torch.arange(n).view(2, n // 2).T.reshape(-1)
+        y = x.clone()
+        y[..., order] = rotate(x[..., :n][..., order], positions, rot)
+        return y
+
+    def late_decay(q, k, v, g, beta):                      # the decay after the write
+        T, H, D = q.shape
+        S, out = torch.zeros(H, D, v.shape[-1], dtype=q.dtype), []
+        for t in range(T):
+            u = beta[t][:, None] * (v[t] - (S * k[t][:, :, None]).sum(1))
+            S = S + k[t][:, :, None] * u[:, None, :]
+            out.append((S * q[t][:, :, None]).sum(1))
+            S = g[t][:, :, None] * S
+        return torch.stack(out), S
+    mistakes = {"no sink": ("sink_attention", lambda q, k, v, s, sink=0.0: attention(q, k, v, s, -math.inf)),
+                "other key heads": ("sink_attention", lambda q, k, v, s, sink=0.0: attention(q, k.flip(0), v.flip(0), s, sink)),
+                "half layout": ("rotate", half_layout),
+                "decay after the write": ("channel_delta_rule", late_decay),
+                "decay left out": ("channel_decayed_sum", lambda q, k, v, g: O_sum(q, k, v, torch.ones_like(g)))}
+    for what, (name, f) in mistakes.items():
+        with monkeypatch.context() as p:
+            p.setattr(O, name, f)
+            wrong = O.forward(cfg, w, toks)
+        assert float((wrong - full).std() / full.std()) > 0.05, what

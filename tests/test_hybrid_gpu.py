@@ -1,4 +1,4 @@
-"""The Fivitar decoder on the GPU against the plain oracle: logits over cuts of the prompt, states used again, captured
+"""The Fivitar and Fekulix decoders on the GPU against the plain oracle: logits over cuts of the prompt, states used again, captured
 steps, greedy generation through the command line's own path, and the trace runner."""
 import json
 import os
@@ -62,8 +62,9 @@ def test_logits_do_not_depend_on_the_cut(name, dtype):
         _close(_feed(m, toks, sizes), want, dtype, (name, sizes))
 
 
-def test_residual_after_every_layer():
-    m, cfg, w = _model("odd", torch.float32)
+@pytest.mark.parametrize("name", ["odd", "fek_odd"])
+def test_residual_after_every_layer(name):
+    m, cfg, w = _model(name, torch.float32)
     toks, want, got = cases.tokens(cfg, 70, seed=5), [], []
     O.forward(cfg, w, toks, layers_out=want)
     hooks = [l.register_forward_hook(lambda mod, inp, out: got.append(inp[0].double().cpu())) for l in m.weights.values()]
@@ -75,23 +76,25 @@ def test_residual_after_every_layer():
         assert float((a - b).abs().max() / b.abs().max()) < 1e-5, i
 
 
-def test_a_finished_request_leaves_nothing_behind():
-    m, cfg, w = _model("odd", torch.float32)
+@pytest.mark.parametrize("name", ["odd", "fek_odd"])
+def test_a_finished_request_leaves_nothing_behind(name):
+    m, cfg, w = _model(name, torch.float32)
     a, b = cases.tokens(cfg, 131), cases.tokens(cfg, 9, seed=2)
     _feed(m, a, (131,))
     first = _feed(m, b, (9,))
-    _close(first, _want("odd", cfg, w, b), torch.float32)
+    _close(first, _want(name, cfg, w, b), torch.float32)
     _feed(m, a, (50, 1))
     again = _feed(m, b, (9,))
     assert torch.equal(first, again)
     _feed(m, a, (131,))
-    _close(_feed(m, b, (1,)), _want("odd", cfg, w, b), torch.float32)
+    _close(_feed(m, b, (1,)), _want(name, cfg, w, b), torch.float32)
 
 
-def test_wanted_places_and_limits():
-    m, cfg, w = _model("tiny", torch.float32)
+@pytest.mark.parametrize("name", ["tiny", "fek_tiny"])
+def test_wanted_places_and_limits(name):
+    m, cfg, w = _model(name, torch.float32)
     toks = cases.tokens(cfg, 60)
-    want = _want("tiny", cfg, w, toks)
+    want = _want(name, cfg, w, toks)
     s = Session(m, 60, portion=16)
     _close(s.feed(toks[:50], [49, 0, 17, 17, 16]), want[[49, 0, 17, 17, 16]], torch.float32)
     assert s.feed(toks[50:51]).shape == (0, cfg["vocab"]) and s.feed(toks[51:57]).shape[0] == 0
@@ -100,7 +103,7 @@ def test_wanted_places_and_limits():
         s.feed([0] * 1000)
 
 
-@pytest.mark.parametrize("name", ["odd", "tiny"])
+@pytest.mark.parametrize("name", ["odd", "tiny", "fek_odd", "fek_tiny"])
 def test_graph_replays_equal_eager_steps(name):
     m, cfg, w = _model(name, torch.bfloat16)
     toks = cases.tokens(cfg, 40)
@@ -126,7 +129,7 @@ def test_graph_replays_equal_eager_steps(name):
 
 
 @pytest.mark.parametrize("graph", [True, False])
-@pytest.mark.parametrize("name,n", [("odd", 12), ("wide", 8), ("tiny", 150)])
+@pytest.mark.parametrize("name,n", [("odd", 12), ("wide", 8), ("tiny", 150), ("fek_odd", 12), ("fek_wide", 8), ("fek_tiny", 150)])
 def test_greedy_generation(name, n, graph):
     m, cfg, w = _model(name, torch.float32)
     prompt = torch.tensor(cases.tokens(cfg, 20, seed=7))
@@ -148,18 +151,20 @@ def _checkpoint(tmp_path, name):
     return cfg, w
 
 
-def test_command_line_generates_from_a_checkpoint_folder(tmp_path, capsys):
-    cfg, w = _checkpoint(tmp_path, "tiny")
+@pytest.mark.parametrize("name", ["tiny", "fek_tiny"])
+def test_command_line_generates_from_a_checkpoint_folder(name, tmp_path, capsys):
+    cfg, w = _checkpoint(tmp_path, name)
     G.main(["--model", str(tmp_path), "--dtype", "float32", "--prompt-tokens", "5,9,2", "--max-new-tokens", "6"])
     line = json.loads(capsys.readouterr().out.strip().splitlines()[-1])
-    assert line["model"] == "Fivitar" and len(line["tokens"]) == 6
+    assert line["model"] == cfg["architecture"] and len(line["tokens"]) == 6
     logits = O.forward(cfg, w, [5, 9, 2] + line["tokens"][:-1])
     for i, t in enumerate(line["tokens"]):
         assert float(logits[2 + i].max() - logits[2 + i][t]) < 1e-3 * float(logits[2 + i].std())
 
 
-def test_trace_runner(tmp_path):
-    cfg, w = _checkpoint(tmp_path, "odd")
+@pytest.mark.parametrize("name", ["odd", "fek_odd"])
+def test_trace_runner(name, tmp_path):
+    cfg, w = _checkpoint(tmp_path, name)
     a, b = cases.tokens(cfg, 30), cases.tokens(cfg, 9, seed=2)
     steps = [{"step": 0, "entries": [{"id": "x", "tokens": a[:25], "want": [0, 24]}], "end": []},
              {"step": 1, "entries": [{"id": "x", "tokens": a[25:29], "want": []}], "end": []},

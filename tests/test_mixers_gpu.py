@@ -3,24 +3,13 @@ token, in float32 (tight) and bfloat16."""
 import pytest
 import torch
 
-from decdec_amd import mixer_ops as M, mixers as X
+from decdec_amd import mixer_ops as M
 from oracle import hybrid_oracle as O
 import hybrid_cases as cases
+from mixer_bench import Bench, close as _close, portions as _portions, rand as _rand
 
 pytestmark = pytest.mark.gpu
 DTYPES = [torch.float32, torch.bfloat16]
-TOL = {torch.float32: 2e-5, torch.bfloat16: 2.5e-2}
-
-
-def _close(got, want, dtype, what="", factor=1.0):
-    got, want = got.detach().double().cpu(), want.double().cpu()
-    assert torch.isfinite(got).all(), what
-    err = float((got - want).abs().max() / (want.abs().max() + 1e-9))
-    assert err <= TOL[dtype] * factor, (what, err)
-
-
-def _rand(*shape, seed=0, scale=1.0):
-    return torch.randn(*shape, generator=torch.Generator().manual_seed(seed)) * scale
 
 
 # ---- rows --------------------------------------------------------------------------------------------------
@@ -33,6 +22,66 @@ def test_gemv_with_an_activation_on_its_first_rows(N, K, act, dtype):
     y = w.double() @ x.double()
     y[:act] = O.xielu(y[:act], a[0].double(), a[1].double())
     _close(out, y, dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("N,K", [(5, 3), (301, 200), (4100, 96)])
+def test_gemv_with_gelu_and_a_scale(N, K, dtype):
+    w, x = _rand(N, K, seed=N).to(dtype), _rand(K, seed=1).to(dtype)
+    y = w.double() @ x.double()
+    out = torch.empty(N, dtype=dtype, device="cuda")
+    M.gemv(w.cuda(), x.cuda(), out, None, N, M.ACT_GELU_TANH)
+    _close(out, O.gelu_tanh(y), dtype)
+    M.gemv(w.cuda(), x.cuda(), out, scale=0.3)
+    _close(out, 0.3 * y, dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("rows,dim", [(1, 84), (3, 33), (4, 4096), (2, 7001)])
+def test_residual_and_embedding_behind_a_dynamic_tanh(rows, dim, dtype):
+    x, y = _rand(rows, dim, seed=1, scale=3.0), _rand(rows, dim, seed=2).to(dtype)
+    x[0, :7] = torch.tensor([0.0, 1e-6, -1e-4, 1e-2, 40.0, -40.0, 300.0])     # near zero and far past saturation
+    a, w, b = torch.tensor(0.7).to(dtype), _rand(dim, seed=5).to(dtype), _rand(dim, seed=6).to(dtype)
+    norm = tuple(t.cuda() for t in (a, w, b))
+    want = lambda v: O.dynamic_tanh(v, a.double(), w.double(), b.double())
+    xd, out = x.cuda(), torch.empty(rows, dim, dtype=dtype, device="cuda")
+    M.residual_tanh(xd, None, norm, out)
+    assert torch.equal(xd.cpu(), x)
+    _close(out, want(x.double()), dtype)
+    M.residual_tanh(xd, y.cuda(), norm, out)
+    assert torch.equal(xd.cpu(), x + y.float())            # the residual stream is float32 whatever the storage type
+    _close(out, want(x.double() + y.double()), dtype)
+    no_bias = (norm[0], norm[1], torch.zeros_like(norm[2]))
+    small = (_rand(rows, dim, seed=7) * 1e-4).cuda()       # tanh keeps its relative accuracy there
+    M.residual_tanh(small, None, no_bias, out)
+    _close(out, torch.tanh(a.double() * small.double().cpu()) * w.double(), dtype)
+    table, toks = _rand(50, dim, seed=8).to(dtype).cuda(), torch.tensor([3, 49, 0, 3][:rows], device="cuda")
+    M.embed(table, toks, xd, out, norm)
+    assert torch.equal(xd, table[toks].float())
+    _close(out, want(table[toks].double().cpu()), dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("n,ld", [(52, 60), (7, 9), (5000, 5000)])
+def test_gelu_rows(n, ld, dtype):
+    inp = _rand(3, ld, seed=4, scale=3.0).to(dtype).cuda()
+    want = O.gelu_tanh(inp[:, :n].double().cpu())
+    out = inp if n == ld else torch.empty(3, n, dtype=dtype, device="cuda")   # in place where the rows are whole
+    M.activation(inp, n, None, out, M.ACT_GELU_TANH)
+    _close(out, want, dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("groups,n", [(3, 36), (3, 128), (2, 256), (2, 201), (2, 1028), (1, 1030)])
+@pytest.mark.parametrize("at,wide", [(0, 0), (8, 16), (3, 5)])
+def test_group_norm_gate_into_columns_with_a_scale(groups, n, at, wide, dtype):
+    o, g, w = _rand(3, groups * n, seed=1).cuda(), _rand(3, groups * n, seed=2).to(dtype).cuda(), _rand(n, seed=3).to(dtype).cuda()
+    buf = torch.full((3, groups * n + wide), 7.0, dtype=dtype, device="cuda")
+    out = buf[:, at:at + groups * n]
+    M.group_norm_gate(o, g, groups * n, w, out, groups, 0.01, M.GATE_SILU, 0.3)
+    want = 0.3 * O.rms_norm(o.double().view(3, groups, n), w.double(), 0.01).view(3, -1) * O.silu(g.double())
+    _close(out, want, dtype)
+    assert float((buf[:, :at] - 7).abs().sum() + (buf[:, at + groups * n:] - 7).abs().sum()) == 0
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -89,60 +138,18 @@ def test_group_norm_gate(groups, n, kind, off, pad, dtype):
 
 
 # ---- mixers ------------------------------------------------------------------------------------------------
-class Bench:
-    """A mixer on the GPU with random weights, and the oracle's read-out (before the output projection)."""
-
-    def __init__(self, kind, m, dtype, T, seed=0, width=40, eps=1e-5, edit=None, max_seq=None):
-        g = torch.Generator().manual_seed(seed)
-        self.w = {n: cases.random_tensor("mix." + n, s, g) for n, s in cases.mixer_shapes(kind, m, width).items()}
-        self.w["o"] = torch.eye(self.w["o"].shape[1]).to(torch.bfloat16)          # the oracle's output is the read-out itself
-        self.h = torch.randn(T, width, generator=g).to(torch.bfloat16)
-        self.m, self.kind, self.eps, self.dtype, self.T = m, kind, eps, dtype, T
-        if edit:
-            edit(self)
-        self.mixer = X.MIXER_TYPES[kind](m, X.Workspace(torch.device("cuda")))
-        names, off = [n for n, _ in self.mixer.inputs], {}
-        for n, r in self.mixer.inputs:
-            off[n] = sum(off_r for _, off_r in self.mixer.inputs[:names.index(n)])
-        rows = sum(r for _, r in self.mixer.inputs)
-        # projections in float64, rounded once to the storage type; the oracle sees the unrounded ones
-        proj = torch.cat([self.h.double() @ self.w[n].double().T for n in names], 1)
-        self.proj = torch.zeros(T, (rows + 7) // 8 * 8, dtype=dtype)
-        self.proj[:, :rows] = proj.to(dtype)
-        self.proj = self.proj.cuda()
-        self.mixer.bind({n: t.to(dtype).cuda() for n, t in self.w.items() if n not in names and n != "o"}, off, eps)
-        self.max_seq = max_seq or T
-        self.new_state()
-
-    def new_state(self):
-        self.state = self.mixer.new_state(self.max_seq, self.dtype, "cuda")
-
-    def want(self):
-        return O.MIXERS[self.kind](self.h.double(), {n: t.double() for n, t in self.w.items()}, self.m, self.eps)
-
-    def run(self, portions, t=0):
-        out = []
-        for n in portions:
-            y = torch.empty(n, self.mixer.width, dtype=self.dtype, device="cuda")
-            self.mixer(self.proj[t:t + n].contiguous(), self.state, torch.tensor([t], device="cuda"), t, y)
-            out.append(y)
-            t += n
-        return torch.cat(out)
-
-
-def _portions(T, *sizes):
-    out, i = [], 0
-    while sum(out) < T:
-        out.append(min(sizes[i % len(sizes)], T - sum(out)))
-        i += 1
-    return out
-
-
 RECURRENCES = [("lightning", cases.lightning(3, 32, 32)), ("lightning", cases.lightning(5, 12, 28, [0.0, 0.3, 0.95, 0.9999, 1.0])),
                ("lightning", cases.lightning(2, 128, 128)), ("lightning", cases.lightning(1, 200, 72, [0.98])), ("lightning", cases.lightning(2, 1, 1)),
                ("delta", cases.delta(4, 2, 48, 64, 4)), ("delta", cases.delta(3, 3, 20, 36, 3)), ("delta", cases.delta(4, 2, 128, 128, 4)),
                ("delta", cases.delta(2, 2, 64, 16, 1)), ("delta", cases.delta(6, 2, 9, 130, 2)), ("delta", cases.delta(1, 1, 256, 256, 7)),
-               ("delta", cases.delta(2, 1, 16, 300, 5))]
+               ("delta", cases.delta(2, 1, 16, 300, 5)),
+               ("gated_linear", cases.gated_linear(3, 32, 32, 16.0)), ("gated_linear", cases.gated_linear(5, 12, 28, 1.0)),
+               ("gated_linear", cases.gated_linear(2, 128, 128, 4.0)), ("gated_linear", cases.gated_linear(1, 200, 72, 0.5)),
+               ("gated_linear", cases.gated_linear(2, 1, 1, 2.0)), ("gated_linear", cases.gated_linear(2, 48, 2000, 8.0)),
+               ("channel_delta", cases.delta(4, 2, 48, 64, 4)), ("channel_delta", cases.delta(3, 3, 20, 36, 3)),
+               ("channel_delta", cases.delta(4, 2, 128, 128, 4)), ("channel_delta", cases.delta(2, 2, 64, 16, 1)),
+               ("channel_delta", cases.delta(6, 2, 9, 130, 2)), ("channel_delta", cases.delta(1, 1, 256, 256, 7)),
+               ("channel_delta", cases.delta(2, 1, 16, 300, 9)), ("channel_delta", cases.delta(1, 1, 30, 1100, 4))]
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -166,15 +173,17 @@ def test_delta_rule_with_decays_that_forget_at_once_and_never(dtype):
         _close(b.run(_portions(140, *sizes)), b.want(), dtype, sizes, factor=4.0)
 
 
-def test_convolution_sees_exactly_its_taps_across_a_cut():
+@pytest.mark.parametrize("kind", ["delta", "channel_delta"])
+def test_convolution_sees_exactly_its_taps_across_a_cut(kind):
     """One token's input is changed: the read-outs of a head without memory differ for `taps` tokens from there on, no
     more and no fewer, wherever the portions are cut."""
     taps, T = 4, 40
 
     def edit(b):                                           # a decay of e^-150: nothing but the convolution reaches back
-        b.w["A_log"], b.w["dt_bias"] = torch.tensor([5.0]).to(torch.bfloat16), torch.tensor([4.0]).to(torch.bfloat16)
-        b.w["a"] = torch.zeros_like(b.w["a"])
-    b = Bench("delta", cases.delta(1, 1, 16, 16, taps), torch.float32, T, edit=edit)
+        b.w["A_log"], b.w["dt_bias"] = torch.tensor([5.0]).to(torch.bfloat16), torch.full_like(b.w["dt_bias"], 4.0)
+        a = "a" if kind == "delta" else "a1"
+        b.w[a] = torch.zeros_like(b.w[a])
+    b = Bench(kind, cases.delta(1, 1, 16, 16, taps), torch.float32, T, edit=edit)
     for sizes in ((T,), (1,), (2,), (7, 1)):
         base = b.run(_portions(T, *sizes))
         keep = b.proj.clone()
@@ -183,6 +192,98 @@ def test_convolution_sees_exactly_its_taps_across_a_cut():
             moved = (b.run(_portions(T, *sizes)) - base).abs().amax(1) > 1e-4
             assert moved.nonzero().view(-1).tolist() == list(range(at, at + taps)), (sizes, at)
             b.proj.copy_(keep)
+
+
+def _channel_extremes(kind, H, D):
+    """Per channel: forgetting at once, never, and everything between, side by side in a head."""
+    def edit(b):
+        g = torch.Generator().manual_seed(3)
+        bias = torch.randn(H * D, generator=g) * 3.0
+        bias[::5], bias[1::5] = -30.0, 30.0
+        b.w["a2.b" if kind == "gated_linear" else "dt_bias"] = bias.to(torch.bfloat16)
+        if kind == "channel_delta":
+            b.w["A_log"] = torch.tensor([4.0, -9.0, 1.0][:H]).to(torch.bfloat16)
+    return edit
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("kind", ["gated_linear", "channel_delta"])
+def test_channel_decays_that_forget_at_once_and_never(kind, dtype):
+    m = cases.gated_linear(3, 40, 24, 0.25) if kind == "gated_linear" else cases.delta(3, 1, 40, 24, 4)
+    b = Bench(kind, m, dtype, 200, edit=_channel_extremes(kind, 3, 40))
+    want = b.want()
+    for sizes in ((200,), (37,), (1,)):
+        _close(b.run(_portions(200, *sizes)), want, dtype, (kind, sizes), factor=4.0)
+
+
+@pytest.mark.parametrize("kind", ["gated_linear", "channel_delta"])
+def test_tokens_that_forget_everything_between_tokens_that_keep(kind):
+    """Decays near one among decays of e^-160: what is written after a token that forgets lasts, whatever the sums hold."""
+    T, D, V = 140, 24, 16
+
+    def edit(b):
+        z = torch.full((T,), -6.0)
+        z[[5, 6, 7, 8, 20, 63, 64, 100]] = 60.0
+        b.h[:, 0] = (z if kind == "channel_delta" else -z).to(torch.bfloat16)
+        for n in ("q", "k", "v", "b", "g", "g1"):
+            if n in b.w:
+                b.w[n][:, 0] = 0
+        b.w["a1"].zero_(), b.w["a2"].zero_()
+        b.w["a1"][0, 0] = 1
+        b.w["a2"][:, 0] = 1
+        if kind == "channel_delta":
+            b.w["A_log"][:] = 1.0
+        b.w["dt_bias" if kind == "channel_delta" else "a2.b"].mul_(0.1)
+    m = cases.gated_linear(1, D, V, 0.35) if kind == "gated_linear" else cases.delta(1, 1, D, V, 2)
+    b = Bench(kind, m, torch.float32, T, edit=edit)
+    want = b.want()
+    for sizes in ((T,), (1,), (50, 3)):
+        _close(b.run(_portions(T, *sizes)), want, torch.float32, sizes)
+
+
+@pytest.mark.parametrize("kind", ["gated_linear", "channel_delta"])
+def test_every_key_channel_has_its_own_decay(kind):
+    """A head whose channels all forget at once but one: what a token wrote comes back through that channel alone, from any
+    distance and over any cut."""
+    T, D, V, keep = 150, 24, 16, 7
+    m = cases.gated_linear(1, D, V, 1.0) if kind == "gated_linear" else cases.delta(1, 1, D, V, 1)
+
+    def edit(b):
+        forget = -60.0 if kind == "gated_linear" else 60.0                     # sigmoid(-60), or exp(-e softplus(60))
+        bias = torch.full((D,), forget)
+        bias[keep] = -forget
+        b.w["a2.b" if kind == "gated_linear" else "dt_bias"] = bias.to(torch.bfloat16)
+        b.w["a1"] = torch.zeros_like(b.w["a1"])
+        if kind == "channel_delta":
+            b.w["A_log"] = torch.tensor([1.0]).to(torch.bfloat16)
+    b = Bench(kind, m, torch.float32, T, edit=edit)
+    want = b.want()
+    for sizes in ((T,), (1,), (50, 3), (65,)):
+        base = b.run(_portions(T, *sizes))
+        _close(base, want, torch.float32, sizes, factor=4.0)
+    k = b.mixer.params.off_k
+    saved = b.proj.clone()
+    b.proj[3, k + keep] += 3.0                                                 # the lasting channel of an early key
+    far = (b.run([T]) - base).abs().amax(1)
+    assert float(far[100:].max()) > 1e-3 and float(far[:3].max()) < 1e-6
+    if kind == "gated_linear":                                                 # (unit vectors couple the channels)
+        b.proj.copy_(saved)
+        b.proj[3, k + keep + 1] += 3.0
+        moved = (b.run([T]) - base).abs().amax(1) > 1e-5
+        assert moved.nonzero().view(-1).tolist() == [3]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("rank", [1, 7, 64, 200, 1024])
+def test_low_rank_maps_of_any_rank(rank, dtype):
+    def edit(b):
+        g, H, D, V = torch.Generator().manual_seed(rank), 2, 16, 24
+        put = lambda n, *s: b.w.__setitem__(n, (torch.randn(*s, generator=g) * 1.5 / s[1] ** 0.5).to(torch.bfloat16))
+        put("a1", rank, 40), put("a2", H * D, rank), put("g1", rank, 40), put("g2", H * V, rank)
+    b = Bench("channel_delta", cases.delta(2, 1, 16, 24, 4), dtype, 70, edit=edit)
+    want = b.want()
+    for sizes in ((70,), (1,)):
+        _close(b.run(_portions(70, *sizes)), want, dtype, (rank, sizes), factor=4.0)
 
 
 LATENTS = [cases.latent(3, 64, 32, 96, 80, scaling=cases.YARN), cases.latent(3, 22, 10, 18, 30, base=500.0), cases.latent(17, 16, 8, 24, 48, scale=0.4),
