@@ -624,8 +624,8 @@ __global__ __launch_bounds__(256) void channel_chunk_kernel(const ChunkParams p)
 #pragma unroll
             for (uint32_t j = 0; j < 4u; ++j) {
                 const bool in = r < n && (FULL || c0 + c + j < D);
-                // no float is as small as 2^-160: a bound that changes no product and keeps later differences sharp
-                x[j] = in ? fmaxf(channel_log_decay(rate2, p.a_sign, as.x[e][j], p.a_bias[h * D + c0 + c + j]), -160.f) : 0.f;
+                // what 2^-64 is left of does not show in a sum; the bound keeps the differences after such a token sharp
+                x[j] = in ? fmaxf(channel_log_decay(rate2, p.a_sign, as.x[e][j], p.a_bias[h * D + c0 + c + j]), -64.f) : 0.f;
             }
             *(f32x4*)&Ls[r][c] = x;
         }

@@ -218,7 +218,7 @@ def test_channel_decays_that_forget_at_once_and_never(kind, dtype):
 
 @pytest.mark.parametrize("kind", ["gated_linear", "channel_delta"])
 def test_tokens_that_forget_everything_between_tokens_that_keep(kind):
-    """Decays near one among decays of e^-160: what is written after a token that forgets lasts, whatever the sums hold."""
+    """Decays near one among decays of e^-160 and less: what is written after a token that forgets lasts, whatever the sums hold."""
     T, D, V = 140, 24, 16
 
     def edit(b):
@@ -238,7 +238,7 @@ def test_tokens_that_forget_everything_between_tokens_that_keep(kind):
     b = Bench(kind, m, torch.float32, T, edit=edit)
     want = b.want()
     for sizes in ((T,), (1,), (50, 3)):
-        _close(b.run(_portions(T, *sizes)), want, torch.float32, sizes)
+        _close(b.run(_portions(T, *sizes)), want, torch.float32, sizes, factor=2.0)
 
 
 @pytest.mark.parametrize("kind", ["gated_linear", "channel_delta"])
