@@ -612,7 +612,8 @@ __global__ __launch_bounds__(256) void channel_chunk_kernel(const ChunkParams p)
 #pragma unroll
     for (int j = 0; j < 4; ++j) pq[j] = pk[j] = f32x4{0.f, 0.f, 0.f, 0.f};
     float dq[4] = {0.f, 0.f, 0.f, 0.f}, dk[4] = {0.f, 0.f, 0.f, 0.f};
-    Slice qs = slice_fetch<FULL>(q, kld, n, 0u, D, vec), ks = slice_fetch<FULL>(k, kld, n, 0u, D, vec), as = slice_fetch<FULL>(p.a + hrow, hld, n, 0u, D, vec);
+    Slice qs = slice_fetch<FULL>(q, kld, n, 0u, D, vec), ks = slice_fetch<FULL>(k, kld, n, 0u, D, vec);
+    Slice as = slice_fetch<FULL>(p.a + hrow, hld, n, 0u, D, vec);
     for (uint32_t c0 = 0; c0 < D; c0 += 32u) {
         __syncthreads();
         slice_put(qs, Qs);

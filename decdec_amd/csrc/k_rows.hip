@@ -1,5 +1,6 @@
 // Row-wise pieces of decoders with a 32-bit residual stream: one-token GEMV with an activation on its first rows,
-// embedding, gated residual + norm of the sublayer's output, residual + dynamic tanh, norm, activations, normed and gated read-out of a recurrence.
+// embedding, gated residual + norm of the sublayer's output, residual + dynamic tanh, norm, activations, normed and gated
+// read-out of a recurrence.
 #include "mixers.h"
 #include "mma.h"
 
